@@ -44,6 +44,7 @@ class CacheStorage:
         self.pools = [maker.allocate_pool(len(m), n_pages, page_size, dtype, device)
                       for maker, m in zip(self._group_makers, members)]
         self.states: dict[int, torch.Tensor] = {}
+        self.records: dict[int, dict] = {}        # entry -> {name: [max_slots, ...]}, further records per slot
         self.entries: list[LayerCache] = []
         for i, (spec, share) in enumerate(zip(entry_specs, shares)):
             src = i if share is None else share
@@ -62,7 +63,10 @@ class CacheStorage:
                     state = spec.allocate_state(max_slots, device)
                     if state is not None:
                         self.states[src] = state
+                if src not in self.records:
+                    self.records[src] = spec.allocate_records(max_slots, device)
                 lc.state = self.states.get(src)
+                lc.records = self.records[src]
             self.entries.append(lc)
         self._bytes_per_token = sum(spec.bytes_per_token(torch.empty((), dtype=dtype).element_size())
                                     for spec, share in zip(entry_specs, shares) if spec is not None and share is None)
@@ -70,11 +74,15 @@ class CacheStorage:
     def zero_slots(self, slots) -> None:
         """Fixed-size state starts at zero for a newly claimed slot
         (crates/forward/src/core/scratch.rs:1530-1572 does the same per slot)."""
-        if not slots or not self.states:
+        tables = self._slot_tables()
+        if not slots or not tables:
             return
-        idx = torch.tensor(list(slots), dtype=torch.long, device=next(iter(self.states.values())).device)
-        for t in self.states.values():
+        idx = torch.tensor(list(slots), dtype=torch.long, device=tables[0].device)
+        for t in tables:
             t.index_fill_(0, idx, 0)
+
+    def _slot_tables(self) -> list:
+        return list(self.states.values()) + [t for named in self.records.values() for t in named.values()]
 
     def fill(self, value: float) -> None:
         """Overwrite every page of every pool (a debugging aid: with NaN, a read of a row that was
@@ -87,4 +95,4 @@ class CacheStorage:
 
     def nbytes(self) -> int:
         return sum(p.numel() * p.element_size() for p in self.pools) + sum(
-            t.numel() * t.element_size() for t in self.states.values())
+            t.numel() * t.element_size() for t in self._slot_tables())

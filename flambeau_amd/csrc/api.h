@@ -61,42 +61,70 @@ int fl_sample_count(unsigned short* counts, int V, int rows, const float* slot, 
 int fl_sample_history(unsigned short* counts, int V, int slot, const int* tokens, int n, hipStream_t stream);
 
 // ---- attention over one cached latent per token (latent.hip) ----
-// RMS norm of columns col0 .. col0 + width - 1 of float rows; with a block table the result goes to the
-// page row of the token's position (pool [n_pages][page_size][width]), else to out [n][width]
-int fl_norm_slice(const float* x, int ld, int col0, int width, const float* w, float eps, void* out,
-                  int out_dtype, int n, const int* positions, const int* tok_seq, const int* block_table,
-                  int max_blocks, int page_size, int n_pages, hipStream_t stream);
-// one small product per head: out[t][h][:] = x[t][h][:] W_h (transposed: W_h^T), optionally times the sigmoid of a gate logit per head
-int fl_heads_matmul(const float* x, int ldx, const void* w, int w_dtype, void* out, int out_dtype, int n,
-                    int H, int K, int J, int transposed, const float* gate, int ldg, int gate_col0,
-                    hipStream_t stream);
-// z[t][h][:] = softmax_j(scale * qa[t][h] . c_j) c_j over the latent rows j <= position of the token's request
+// From the joined projection of a step's tokens (float rows) to the normed query latent (columns 0 .. q_width - 1) in
+// q_out and, with write_cache, the token's row in its page: the normed latent (R columns from kv_col on) and behind it
+// a rotated key part of rot_dim columns (rot of them turned by cs [n][rot / 2][2]); pool [n_pages][page_size * (K + V)],
+// a page's rows [page_size][K] = (latent, zeros to V, rotated part, zeros) and its values transposed, [V][page_size]
+int fl_latent_prepare(const float* x, int ld, int q_width, const float* qw, void* q_out, int kv_col, int R,
+                      const float* kw, float eps, int rot_dim, int rot, const float* cs, void* pool, int dtype,
+                      int K, int V, int n, const int* positions, const int* tok_seq, const int* block_table,
+                      int max_blocks, int page_size, int n_pages, int write_cache, hipStream_t stream);
+// one small product per head: out[t][h][:] = x[t][h][:] W_h (transposed: W_h^T), optionally times the sigmoid of a gate
+// logit per head; heads lie hx apart in x and ho apart in out.  What an out row holds beyond the J results is zeroed, but
+// for the head's rotated part: the rot_dim values behind its K in x, turned, to column rot_at of its row (rot_dim 0: none)
+int fl_heads_matmul(const float* x, int ldx, int hx, const void* w, int w_dtype, void* out, int out_dtype, int ho, int n,
+                    int H, int K, int J, int transposed, const float* gate, int ldg, int gate_col0, int rot_dim, int rot,
+                    const float* cs, int rot_at, hipStream_t stream);
+// z[t][h][0:R] = sum_j softmax_j(scale * qa[t][h] . row_j) row_j[0:R] over the visible rows (K values each) of the
+// token's request: j <= position, with window > 0 the newest `window` of them
 int fl_latent_attention(const float* qa, float* z, const void* pool, int dtype, const int* positions,
-                        const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int R,
+                        const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                         int page_size, int n_pages, float scale, int window, hipStream_t stream);
 int fl_latent_max_width(void);
-// the same on the matrix cores for bfloat16 pools (latent_tuned.hip): qa bfloat16 [n][H][R], z float [n][H][R]
+// the same on the matrix cores for bfloat16 pools (latent_tuned.hip): qa bfloat16 [n][H][K], z float [n][H][R]
 int fl_latent_attention_mfma(const void* qa, float* z, const void* pool, const int* positions,
-                             const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int R,
+                             const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                              int page_size, int n_pages, float scale, int window, int n_split, float* part_o,
                              float* part_ml, hipStream_t stream);
-int fl_latent_attention_mfma_takes(int R, int page_size);
+int fl_latent_attention_mfma_takes(int K, int R, int page_size);
 // the same for prompt portions: blocks of four waves that share their keys through LDS; tiles [n_tiles][4] =
 // (first token, tokens, first group of 16 heads, groups), tokens x groups <= 4, the tokens of one request
 int fl_latent_attention_shared(const void* qa, float* z, const void* pool, const int* positions,
-                               const int* tok_seq, const int* block_table, int max_blocks, int H, int R,
+                               const int* tok_seq, const int* block_table, int max_blocks, int H, int K, int R,
                                int page_size, int n_pages, float scale, int window, const int* tiles, int n_tiles,
                                hipStream_t stream);
-long fl_latent_attention_shared_lds(int R);
+long fl_latent_attention_shared_lds(int K, int R);
 // and for steps of few rows: a block of four waves per (token, 16 heads, part of the keys) that deal the latent's dims out among them
 int fl_latent_attention_dealt(const void* qa, float* z, const void* pool, const int* positions,
-                              const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int R,
+                              const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                               int page_size, int n_pages, float scale, int window, int n_split, float* part_o,
                               float* part_ml, hipStream_t stream);
-// out[t][h][j] = sum_k x[t][h][k] w[h][j][k] on the matrix cores (w bfloat16 [H][J][K])
-int fl_heads_matmul_mfma(const void* x, int x_dtype, int ldx, const void* w, void* out, int out_dtype, int n,
-                         int H, int K, int J, const float* gate, int ldg, int gate_col0, hipStream_t stream);
+// out[t][h][j] = sum_k x[t][h][k] w[h][j][k] on the matrix cores (w bfloat16 [H][J][K]); strides and rotated part as for fl_heads_matmul
+int fl_heads_matmul_mfma(const void* x, int x_dtype, int ldx, int hx, const void* w, void* out, int out_dtype, int ho, int n,
+                         int H, int K, int J, const float* gate, int ldg, int gate_col0, int rot_dim, int rot,
+                         const float* cs, int rot_at, hipStream_t stream);
 int fl_heads_matmul_mfma_takes(int K, int J);
+
+// ---- around a sublayer that is normed on both sides (sublayer.hip) ----
+// resid += scale * norm(sigmoid(gate + gate_bias) * y); with next_w also out = norm(resid), the next sublayer's input.
+// centred: layer norm, else root-mean-square norm; place (or null): y holds the rows of a token's `top` experts, added
+// in rising rank; gate, gate_bias, b, scale, next_b may be null
+int fl_sublayer_step(const float* y, const int* place, int top, const float* gate, const float* gate_bias,
+                     int centred, const float* w, const float* b, const float* scale, float eps, float* resid,
+                     int next_centred, const float* next_w, const float* next_b, float next_eps, void* out,
+                     int out_dtype, int n, int W, hipStream_t stream);
+// out_t = h_t + sum_k w[k] h_(t - taps + 1 + k) per channel (w [taps][C]); ring [slots][taps][C]: the kept inputs
+int fl_input_conv(const void* h, int dtype, const float* w, float* ring, const int* positions, const int* tok_seq,
+                  const int* seq_q_start, const int* seq_q_len, const int* seq_slots, void* out, int n, int C,
+                  int taps, hipStream_t stream);
+// out[t] = table[token] + pairs[(previous * mul_prev + token * mul_cur) mod buckets], the row `buckets` at position 0;
+// last [slots][2]: every request's last tokens
+int fl_embed_bigram(const void* table, const void* pairs, int dtype, const int* tokens, const int* positions,
+                    const int* tok_seq, const int* seq_q_start, const int* seq_q_len, const int* seq_slots, int* last,
+                    float* out, int n, int H, int V, int buckets, long mul_prev, long mul_cur, hipStream_t stream);
+// out[r][i] = g sigmoid(alpha g) (u + shift), g = min(gu[r][i], limit), u = clamp(gu[r][I + i], -limit, limit) (stream_ops.hip)
+int fl_clamped_gate(const float* gu, void* out, int out_dtype, int n, int I, float alpha, float limit, float shift,
+                    hipStream_t stream);
 
 // ---- the mLSTM recurrence (mlstm.hip) ----
 int fl_mlstm_scan(const float* proj, int ld, int col_q, int col_k, int col_v, int col_i, int col_f,

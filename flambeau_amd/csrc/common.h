@@ -49,6 +49,11 @@ __device__ __forceinline__ float gate_activation(float z) {
     if (KIND == FL_GATE_GELU_ERF) return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
     return z / (1.0f + expf(-z));
 }
+// A gate whose halves are clamped first: g sigmoid(alpha g) (u + shift), g = min(zg, limit), u = clamp(zu, -limit, limit)
+__device__ __forceinline__ float clamped_gate(float zg, float zu, float alpha, float limit, float shift) {
+    const float g = fminf(zg, limit), u = fminf(fmaxf(zu, -limit), limit);
+    return g / (1.0f + expf(-alpha * g)) * (u + shift);
+}
 // f(constant of the kind): the choice is made once, outside the loops over a block's values (a branch per value
 // cost the tiled gate/up product 7 % of its time)
 template <typename F>

@@ -11,9 +11,13 @@
 // rows of different requests may lie in one block.  Keys beyond the query's position are given weight
 // zero and their values are set to zero before they are multiplied, so what an unused or reused page
 // holds (a NaN too) never reaches a sum.
+//
+// A row is K values wide as a key and R as a value (its first R values; K > R where a rotated key part stands behind
+// the latent); folded queries are K wide, the weighted sums R.
 #include "common.h"
 #include "api.h"
 #include "recordable.h"
+#include "query_tail.h"
 
 #define LT_WAVES 4
 #define LT_CHUNK 64
@@ -25,14 +29,14 @@ __device__ __forceinline__ bf16x8 zero_keys_beyond(bf16x8 v, int first_key, int 
     return v;
 }
 
-// qa: bfloat16 [n][H][R]; z: float [n][H][R]; pool: [n_pages][2][page_size * R]; R = 32 * ns, ns <= NS.
+// qa: bfloat16 [n][H][K]; z: float [n][H][R]; pool: [n_pages][page_size * (K + R)]; K = 32 * nk, nk <= NK, R = 32 * ns, ns <= NS.
 // n_split > 1: the keys of every token are dealt out to that many waves, which leave their sums in
 // part_o [n * groups * n_split * 16][R] and (maximum, sum of weights) in part_ml [...][2]; a second kernel adds them.
-template <int NS>
+template <int NK, int NS>
 __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
     const bf16_t* __restrict__ qa, float* __restrict__ z, const bf16_t* __restrict__ pool,
     const int* __restrict__ positions, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
-    int max_blocks, int n, int H, int R, int page_size, int n_pages, float scale, int window, int groups_per_token,
+    int max_blocks, int n, int H, int K, int R, int page_size, int n_pages, float scale, int window, int groups_per_token,
     int n_split, float* __restrict__ part_o, float* __restrict__ part_ml) {
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int unit = blockIdx.x * LT_WAVES + wave;                 // (token, group of 16 heads, part of the keys)
@@ -40,23 +44,21 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
     const int split = unit % n_split, tg = unit / n_split;
     const int token = tg / groups_per_token, h0 = (tg - token * groups_per_token) * 16;
     const int col = lane & 15, g = lane >> 4;                      // col: head (B columns) or row of an A tile
-    const int ns = R >> 5;
+    const int nk = K >> 5, ns = R >> 5;
     const int p = positions[token];
     const int* table = block_table + (size_t)tok_seq[token] * max_blocks;
     const int lo = window > 0 ? max(0, p - window + 1) : 0;
-    const size_t page_stride = (size_t)2 * page_size * R;
+    const size_t page_stride = (size_t)page_size * (K + R);
     const bool head_live = h0 + col < H;
 
-    // the folded queries of this lane's head, scaled: B operand of every score product
-    bf16x8 qreg[NS];
+    // the folded queries of this lane's head: B operand of every score product
+    bf16x8 qreg[NK];
     {
-        const bf16_t* qr = qa + ((size_t)token * H + h0 + (head_live ? col : 0)) * R;
+        const bf16_t* qr = qa + ((size_t)token * H + h0 + (head_live ? col : 0)) * K;
 #pragma unroll
-        for (int s = 0; s < NS; ++s) {
-            if (s < ns && head_live) {
-                const bf16x8 v = *(const bf16x8*)(qr + 32 * s + 8 * g);
-#pragma unroll
-                for (int e = 0; e < 8; ++e) qreg[s][e] = (bf16_t)((float)v[e] * scale);
+        for (int s = 0; s < NK; ++s) {
+            if (s < nk && head_live) {
+                qreg[s] = *(const bf16x8*)(qr + 32 * s + 8 * g);
             } else {
 #pragma unroll
                 for (int e = 0; e < 8; ++e) qreg[s][e] = (bf16_t)0.f;
@@ -86,10 +88,10 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
             const int kc = min(key, p);                            // a key beyond p: any loadable row, masked below
             int page = table[kc / page_size];
             page = min(max(page, 0), n_pages - 1);
-            const bf16_t* row = pool + (size_t)page * page_stride + (size_t)(kc % page_size) * R + 8 * g;
+            const bf16_t* row = pool + (size_t)page * page_stride + (size_t)(kc % page_size) * K + 8 * g;
 #pragma unroll
-            for (int s = 0; s < NS; ++s)
-                if (s < ns) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[s], sacc[a], 0, 0, 0);
+            for (int s = 0; s < NK; ++s)
+                if (s < nk) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[s], sacc[a], 0, 0, 0);
         }
         // lane (head col, g): sacc[2 q + b][e] is key t0 + 32 q + 8 g + 4 b + e
         float cmax = -INFINITY;
@@ -98,7 +100,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int key = t0 + 32 * (a >> 1) + 8 * g + 4 * (a & 1) + e;
-                if (key > p || key < lo) sacc[a][e] = -INFINITY;
+                sacc[a][e] = key > p || key < lo ? -INFINITY : sacc[a][e] * scale;
                 cmax = fmaxf(cmax, sacc[a][e]);
             }
         cmax = fmaxf(cmax, __shfl_xor(cmax, 16, FL_WAVE));
@@ -129,7 +131,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
             const int kc = min(key0[q], p);
             int page = table[kc / page_size];
             page = min(max(page, 0), n_pages - 1);
-            cols[q] = pool + (size_t)page * page_stride + (size_t)page_size * R + (key0[q] % page_size);
+            cols[q] = pool + (size_t)page * page_stride + (size_t)page_size * K + (key0[q] % page_size);
         }
 #pragma unroll
         for (int t = 0; t < 2 * NS; ++t) {
@@ -199,18 +201,19 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restri
     z[(size_t)unit * R + d] = acc * inv_l;
 }
 
-// Whether the kernel takes a pool's shape: rows of a multiple of 32 values up to 512, pages of a multiple of 16 rows.
-extern "C" int fl_latent_attention_mfma_takes(int R, int page_size) {
-    return R > 0 && R % 32 == 0 && R <= 512 && page_size > 0 && page_size % 16 == 0;
+// Whether the kernels take a pool's shape: values of a multiple of 32 up to 512, keys as wide or one or two steps of
+// 32 wider, pages of a multiple of 16 rows.
+extern "C" int fl_latent_attention_mfma_takes(int K, int R, int page_size) {
+    return R > 0 && R % 32 == 0 && R <= 512 && K % 32 == 0 && K >= R && K <= R + 64 && page_size > 0 && page_size % 16 == 0;
 }
 
 extern "C" int fl_latent_attention_mfma(const void* qa, float* z, const void* pool, const int* positions,
-                                        const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int R,
+                                        const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                                         int page_size, int n_pages, float scale, int window, int n_split, float* part_o,
                                         float* part_ml, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && n_pages > 0 && max_blocks > 0, "latent_attention_mfma: bad sizes");
     FL_CHECK(n_split >= 1 && n_split <= 64 && (n_split == 1 || (part_o && part_ml)), "latent_attention_mfma: %d parts of the keys (at most 64) need a workspace", n_split);
-    FL_CHECK(fl_latent_attention_mfma_takes(R, page_size), "latent_attention_mfma: rows of %d values in pages of %d are not taken", R, page_size);
+    FL_CHECK(fl_latent_attention_mfma_takes(K, R, page_size), "latent_attention_mfma: rows of %d and %d values in pages of %d are not taken", K, R, page_size);
     FL_CHECK((uintptr_t)qa % 16 == 0 && (uintptr_t)pool % 16 == 0 && (uintptr_t)z % 16 == 0, "latent_attention_mfma: operands must be 16-byte aligned");
     FL_CHECK(window >= 0, "latent_attention_mfma: negative window");
     if (n == 0) return 0;
@@ -219,15 +222,22 @@ extern "C" int fl_latent_attention_mfma(const void* qa, float* z, const void* po
     FL_CHECK(units < (1L << 30), "latent_attention_mfma: too many rows");
     const int blocks = (int)((units + LT_WAVES - 1) / LT_WAVES);
     const int ns = R / 32;
-#define FL_LT(NS)                                                                                                       \
-    latent_attention_mfma_kernel<NS><<<blocks, 64 * LT_WAVES, 0, stream>>>((const bf16_t*)qa, z, (const bf16_t*)pool,  \
+#define FL_LT(NK, NS)                                                                                                       \
+    latent_attention_mfma_kernel<NK, NS><<<blocks, 64 * LT_WAVES, 0, stream>>>((const bf16_t*)qa, z, (const bf16_t*)pool,  \
                                                                            positions, tok_seq, block_table, max_blocks, \
-                                                                           n, H, R, page_size, n_pages, scale, window, groups, \
+                                                                           n, H, K, R, page_size, n_pages, scale, window, groups, \
                                                                            n_split, part_o, part_ml)
-    if (ns <= 2) FL_LT(2);
-    else if (ns <= 4) FL_LT(4);
-    else if (ns <= 8) FL_LT(8);
-    else FL_LT(16);
+    if (K == R) {
+        if (ns <= 2) FL_LT(2, 2);
+        else if (ns <= 4) FL_LT(4, 4);
+        else if (ns <= 8) FL_LT(8, 8);
+        else FL_LT(16, 16);
+    } else {
+        if (ns <= 2) FL_LT(4, 2);
+        else if (ns <= 4) FL_LT(6, 4);
+        else if (ns <= 8) FL_LT(10, 8);
+        else FL_LT(18, 16);
+    }
 #undef FL_LT
     FL_LAUNCH_CHECK();
     if (n_split > 1) {
@@ -246,14 +256,14 @@ FL_RECORDABLE(fl_latent_attention_mfma)
 // there.  Without this every wave fetches every row itself and the kernel runs at the rate of the
 // caches, 16 flops a byte.  Rows are padded by 16 bytes so that the 16 rows (or dims) of an operand
 // start in different banks.  A wave whose token lies before a chunk sits the chunk out.
-template <int NS>
+template <int NK, int NS>
 __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
     const bf16_t* __restrict__ qa, float* __restrict__ z, const bf16_t* __restrict__ pool,
     const int* __restrict__ positions, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
-    int max_blocks, int H, int R, int page_size, int n_pages, float scale, int window, const int* __restrict__ tiles) {
+    int max_blocks, int H, int K, int R, int page_size, int n_pages, float scale, int window, const int* __restrict__ tiles) {
     extern __shared__ __attribute__((aligned(16))) unsigned char lt_smem[];
-    const int stride_r = R + 8, stride_c = LT_CHUNK + 8;
-    bf16_t* ks = (bf16_t*)lt_smem;                                  // [64 keys][R + 8]
+    const int stride_r = K + 8, stride_c = LT_CHUNK + 8;
+    bf16_t* ks = (bf16_t*)lt_smem;                                  // [64 keys][K + 8]
     bf16_t* vs = ks + (size_t)LT_CHUNK * stride_r;                  // [R dims][64 + 8]
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int t_first = tiles[4 * blockIdx.x], n_tok = tiles[4 * blockIdx.x + 1];
@@ -262,23 +272,21 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
     const bool active = tw < n_tok;
     const int token = t_first + (active ? tw : 0), h0 = (g_first + gw) * 16;
     const int col = lane & 15, g = lane >> 4;
-    const int ns = R >> 5;
+    const int nk = K >> 5, ns = R >> 5;
     const int p = active ? positions[token] : -1;
     const int p_max = positions[t_first + n_tok - 1];              // a request's tokens of a step stand in rising order
     const int* table = block_table + (size_t)tok_seq[t_first] * max_blocks;
     const int lo = window > 0 ? max(0, p - window + 1) : 0;
     const int lo_min = window > 0 ? max(0, positions[t_first] - window + 1) : 0;
-    const size_t page_stride = (size_t)2 * page_size * R;
+    const size_t page_stride = (size_t)page_size * (K + R);
     const bool head_live = active && h0 + col < H;
-    bf16x8 qreg[NS];
+    bf16x8 qreg[NK];
     {
-        const bf16_t* qr = qa + ((size_t)token * H + (head_live ? h0 + col : 0)) * R;
+        const bf16_t* qr = qa + ((size_t)token * H + (head_live ? h0 + col : 0)) * K;
 #pragma unroll
-        for (int s = 0; s < NS; ++s) {
-            if (s < ns && head_live) {
-                const bf16x8 v = *(const bf16x8*)(qr + 32 * s + 8 * g);
-#pragma unroll
-                for (int e = 0; e < 8; ++e) qreg[s][e] = (bf16_t)((float)v[e] * scale);
+        for (int s = 0; s < NK; ++s) {
+            if (s < nk && head_live) {
+                qreg[s] = *(const bf16x8*)(qr + 32 * s + 8 * g);
             } else {
 #pragma unroll
                 for (int e = 0; e < 8; ++e) qreg[s][e] = (bf16_t)0.f;
@@ -289,7 +297,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
 #pragma unroll
     for (int t = 0; t < 2 * NS; ++t) o[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
     float m = -INFINITY, l = 0.f;
-    const int pieces_r = R >> 3;                                    // 16-byte pieces of a row
+    const int pieces_r = K >> 3;                                    // 16-byte pieces of a row
     for (int t0 = lo_min & ~(LT_CHUNK - 1); t0 <= p_max; t0 += LT_CHUNK) {
         // ---- the chunk into LDS: rows as they are, and the pages' transposed copies dim by dim.  The pages of the
         // chunk's four runs of 16 keys are looked up first (pages hold a multiple of 16 rows), so that all copies
@@ -300,12 +308,12 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
             const int kc = min(t0 + 16 * j, p_max & ~15);
             int page = table[kc / page_size];
             page = min(max(page, 0), n_pages - 1);
-            run_rows[j] = pool + (size_t)page * page_stride + (size_t)(kc % page_size) * R;       // row kc of the page; its transposed copy lies page_size * R further, at column kc % page_size
+            run_rows[j] = pool + (size_t)page * page_stride + (size_t)(kc % page_size) * K;       // row kc of the page; the transposed values begin behind the page's page_size rows
         }
 #pragma unroll
         for (int i = 0; i < 16; ++i) {                             // wave w copies rows w, w + 4, ...: row 4 i + w lies in run i / 4
             const int row = 4 * i + wave;
-            const bf16_t* src = run_rows[i >> 2] + (size_t)(row & 15) * R;
+            const bf16_t* src = run_rows[i >> 2] + (size_t)(row & 15) * K;
             for (int c = lane; c < pieces_r; c += 64) *(bf16x8*)(ks + (size_t)row * stride_r + 8 * c) = *(const bf16x8*)(src + 8 * c);
         }
         {
@@ -314,7 +322,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
             const bf16_t* src = run_rows[0];
 #pragma unroll
             for (int j = 1; j < 4; ++j) src = (k8 >> 1) == j ? run_rows[j] : src;
-            src += (size_t)(page_size - (kc % page_size)) * R + (kc % page_size) + 8 * (k8 & 1);    // from row kc of the page to column kc (+ 8) of its transposed copy
+            src += (size_t)(page_size - (kc % page_size)) * K + (kc % page_size) + 8 * (k8 & 1);    // from row kc of the page to column kc (+ 8) of its transposed copy
             for (int dim = threadIdx.x >> 3; dim < R; dim += 32)
                 *(bf16x8*)(vs + (size_t)dim * stride_c + 8 * k8) = *(const bf16x8*)(src + (size_t)dim * page_size);
         }
@@ -326,8 +334,8 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
                 sacc[a] = (f32x4){0.f, 0.f, 0.f, 0.f};
                 const bf16_t* row = ks + (size_t)(32 * (a >> 1) + 8 * (col >> 2) + 4 * (a & 1) + (col & 3)) * stride_r + 8 * g;
 #pragma unroll
-                for (int s = 0; s < NS; ++s)
-                    if (s < ns) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[s], sacc[a], 0, 0, 0);
+                for (int s = 0; s < NK; ++s)
+                    if (s < nk) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[s], sacc[a], 0, 0, 0);
             }
             float cmax = -INFINITY;
 #pragma unroll
@@ -335,7 +343,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int key = t0 + 32 * (a >> 1) + 8 * g + 4 * (a & 1) + e;
-                    if (key > p || key < lo) sacc[a][e] = -INFINITY;
+                    sacc[a][e] = key > p || key < lo ? -INFINITY : sacc[a][e] * scale;
                     cmax = fmaxf(cmax, sacc[a][e]);
                 }
             cmax = fmaxf(cmax, __shfl_xor(cmax, 16, FL_WAVE));
@@ -393,38 +401,44 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
         if (t < 2 * ns) *(f32x4*)(zr + 16 * t + 4 * g) = o[t] * inv;
 }
 
-extern "C" long fl_latent_attention_shared_lds(int R) { return (long)LT_CHUNK * (R + 8) * 2 + (long)R * (LT_CHUNK + 8) * 2; }
+extern "C" long fl_latent_attention_shared_lds(int K, int R) { return (long)LT_CHUNK * (K + 8) * 2 + (long)R * (LT_CHUNK + 8) * 2; }
 
 // tiles [n_tiles][4] = (first token, tokens, first group of 16 heads, groups): tokens x groups <= 4, the tokens of one request
 extern "C" int fl_latent_attention_shared(const void* qa, float* z, const void* pool, const int* positions,
-                                          const int* tok_seq, const int* block_table, int max_blocks, int H, int R,
+                                          const int* tok_seq, const int* block_table, int max_blocks, int H, int K, int R,
                                           int page_size, int n_pages, float scale, int window, const int* tiles, int n_tiles,
                                           hipStream_t stream) {
     FL_CHECK(n_tiles >= 0 && H > 0 && n_pages > 0 && max_blocks > 0, "latent_attention_shared: bad sizes");
-    FL_CHECK(fl_latent_attention_mfma_takes(R, page_size), "latent_attention_shared: rows of %d values in pages of %d are not taken", R, page_size);
+    FL_CHECK(fl_latent_attention_mfma_takes(K, R, page_size), "latent_attention_shared: rows of %d and %d values in pages of %d are not taken", K, R, page_size);
     FL_CHECK((uintptr_t)qa % 16 == 0 && (uintptr_t)pool % 16 == 0 && (uintptr_t)z % 16 == 0, "latent_attention_shared: operands must be 16-byte aligned");
-    
     FL_CHECK(window >= 0, "latent_attention_shared: negative window");
     if (n_tiles == 0) return 0;
-    const size_t lds = (size_t)fl_latent_attention_shared_lds(R);
+    const size_t lds = (size_t)fl_latent_attention_shared_lds(K, R);
     const int ns = R / 32;
-#define FL_LTS(NS)                                                                                                     \
+#define FL_LTS(NK, NS)                                                                                                     \
     do {                                                                                                               \
         static bool sized = false;                                                                                     \
         if (!sized) {                                                                                                  \
-            hipError_t e_ = hipFuncSetAttribute((const void*)latent_attention_shared_kernel<NS>,                      \
+            hipError_t e_ = hipFuncSetAttribute((const void*)latent_attention_shared_kernel<NK, NS>,                      \
                                                 hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);              \
             FL_CHECK(e_ == hipSuccess, "latent_attention_shared: %s", hipGetErrorString(e_));                          \
             sized = true;                                                                                              \
         }                                                                                                              \
-        latent_attention_shared_kernel<NS><<<n_tiles, 64 * LT_WAVES, lds, stream>>>(                                  \
-            (const bf16_t*)qa, z, (const bf16_t*)pool, positions, tok_seq, block_table, max_blocks, H, R, page_size,   \
+        latent_attention_shared_kernel<NK, NS><<<n_tiles, 64 * LT_WAVES, lds, stream>>>(                                  \
+            (const bf16_t*)qa, z, (const bf16_t*)pool, positions, tok_seq, block_table, max_blocks, H, K, R, page_size,   \
             n_pages, scale, window, tiles);                                                                            \
     } while (0)
-    if (ns <= 2) FL_LTS(2);
-    else if (ns <= 4) FL_LTS(4);
-    else if (ns <= 8) FL_LTS(8);
-    else FL_LTS(16);
+    if (K == R) {
+        if (ns <= 2) FL_LTS(2, 2);
+        else if (ns <= 4) FL_LTS(4, 4);
+        else if (ns <= 8) FL_LTS(8, 8);
+        else FL_LTS(16, 16);
+    } else {
+        if (ns <= 2) FL_LTS(4, 2);
+        else if (ns <= 4) FL_LTS(6, 4);
+        else if (ns <= 8) FL_LTS(10, 8);
+        else FL_LTS(18, 16);
+    }
 #undef FL_LTS
     FL_LAUNCH_CHECK();
     return 0;
@@ -438,11 +452,11 @@ FL_RECORDABLE(fl_latent_attention_shared)
 // Each forms its share of the scores, the shares are added through LDS in a fixed order (every wave gets the
 // same sums, hence the same maxima and weights), and each adds the weighted rows of its own dims.  A wave then
 // holds a quarter of the accumulators and queries, and the reads of a chunk are all in flight at once.
-template <int NSW>
+template <int NKW, int NSW>
 __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
     const bf16_t* __restrict__ qa, float* __restrict__ z, const bf16_t* __restrict__ pool,
     const int* __restrict__ positions, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
-    int max_blocks, int n, int H, int R, int page_size, int n_pages, float scale, int window, int groups_per_token,
+    int max_blocks, int n, int H, int K, int R, int page_size, int n_pages, float scale, int window, int groups_per_token,
     int n_split, float* __restrict__ part_o, float* __restrict__ part_ml) {
     __shared__ f32x4 sx[LT_WAVES][4][64];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -450,22 +464,20 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
     const int split = unit % n_split, tg = unit / n_split;
     const int token = tg / groups_per_token, h0 = (tg - token * groups_per_token) * 16;
     const int col = lane & 15, g = lane >> 4;
-    const int ns = R >> 5;
+    const int nk = K >> 5, ns = R >> 5;
     const int p = positions[token];
     const int* table = block_table + (size_t)tok_seq[token] * max_blocks;
     const int lo = window > 0 ? max(0, p - window + 1) : 0;
-    const size_t page_stride = (size_t)2 * page_size * R;
+    const size_t page_stride = (size_t)page_size * (K + R);
     const bool head_live = h0 + col < H;
-    bf16x8 qreg[NSW];
+    bf16x8 qreg[NKW];
     {
-        const bf16_t* qr = qa + ((size_t)token * H + h0 + (head_live ? col : 0)) * R;
+        const bf16_t* qr = qa + ((size_t)token * H + h0 + (head_live ? col : 0)) * K;
 #pragma unroll
-        for (int i = 0; i < NSW; ++i) {
+        for (int i = 0; i < NKW; ++i) {
             const int s = wave + LT_WAVES * i;
-            if (s < ns && head_live) {
-                const bf16x8 v = *(const bf16x8*)(qr + 32 * s + 8 * g);
-#pragma unroll
-                for (int e = 0; e < 8; ++e) qreg[i][e] = (bf16_t)((float)v[e] * scale);
+            if (s < nk && head_live) {
+                qreg[i] = *(const bf16x8*)(qr + 32 * s + 8 * g);
             } else {
 #pragma unroll
                 for (int e = 0; e < 8; ++e) qreg[i][e] = (bf16_t)0.f;
@@ -491,11 +503,11 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
             const int kc = min(key, p);
             int page = table[kc / page_size];
             page = min(max(page, 0), n_pages - 1);
-            const bf16_t* row = pool + (size_t)page * page_stride + (size_t)(kc % page_size) * R + 8 * g;
+            const bf16_t* row = pool + (size_t)page * page_stride + (size_t)(kc % page_size) * K + 8 * g;
 #pragma unroll
-            for (int i = 0; i < NSW; ++i) {
+            for (int i = 0; i < NKW; ++i) {
                 const int s = wave + LT_WAVES * i;
-                if (s < ns) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[i], sacc[a], 0, 0, 0);
+                if (s < nk) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[i], sacc[a], 0, 0, 0);
             }
             sx[wave][a][lane] = sacc[a];
         }
@@ -507,7 +519,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int key = t0 + 32 * (a >> 1) + 8 * g + 4 * (a & 1) + e;
-                if (key > p || key < lo) sacc[a][e] = -INFINITY;
+                sacc[a][e] = key > p || key < lo ? -INFINITY : sacc[a][e] * scale;
                 cmax = fmaxf(cmax, sacc[a][e]);
             }
         }
@@ -539,7 +551,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
             const int kc = min(key0[q], p);
             int page = table[kc / page_size];
             page = min(max(page, 0), n_pages - 1);
-            cols[q] = pool + (size_t)page * page_stride + (size_t)page_size * R + (key0[q] % page_size);
+            cols[q] = pool + (size_t)page * page_stride + (size_t)page_size * K + (key0[q] % page_size);
         }
 #pragma unroll
         for (int t = 0; t < 2 * NSW; ++t) {
@@ -585,27 +597,29 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
 
 // fl_latent_attention_mfma with a block of four waves per (token, 16 heads, part of the keys): for steps of few rows
 extern "C" int fl_latent_attention_dealt(const void* qa, float* z, const void* pool, const int* positions,
-                                         const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int R,
+                                         const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                                          int page_size, int n_pages, float scale, int window, int n_split, float* part_o,
                                          float* part_ml, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && n_pages > 0 && max_blocks > 0, "latent_attention_dealt: bad sizes");
     FL_CHECK(n_split >= 1 && n_split <= 64 && (n_split == 1 || (part_o && part_ml)), "latent_attention_dealt: %d parts of the keys (at most 64) need a workspace", n_split);
-    FL_CHECK(fl_latent_attention_mfma_takes(R, page_size), "latent_attention_dealt: rows of %d values in pages of %d are not taken", R, page_size);
+    FL_CHECK(fl_latent_attention_mfma_takes(K, R, page_size), "latent_attention_dealt: rows of %d and %d values in pages of %d are not taken", K, R, page_size);
     FL_CHECK((uintptr_t)qa % 16 == 0 && (uintptr_t)pool % 16 == 0 && (uintptr_t)z % 16 == 0, "latent_attention_dealt: operands must be 16-byte aligned");
     FL_CHECK(window >= 0, "latent_attention_dealt: negative window");
     if (n == 0) return 0;
     const int groups = ceil_div(H, 16);
     const long units = (long)n * groups * n_split;
     FL_CHECK(units < (1L << 30), "latent_attention_dealt: too many rows");
-    const int nsw = ceil_div(R / 32, LT_WAVES);
-#define FL_LTD(NSW)                                                                                                       \
-    latent_attention_dealt_kernel<NSW><<<(unsigned)units, 64 * LT_WAVES, 0, stream>>>((const bf16_t*)qa, z, (const bf16_t*)pool, \
+    const int nkw = ceil_div(K / 32, LT_WAVES), nsw = ceil_div(R / 32, LT_WAVES);
+#define FL_LTD(NKW, NSW)                                                                                                       \
+    latent_attention_dealt_kernel<NKW, NSW><<<(unsigned)units, 64 * LT_WAVES, 0, stream>>>((const bf16_t*)qa, z, (const bf16_t*)pool, \
                                                                                       positions, tok_seq, block_table, max_blocks, \
-                                                                                      n, H, R, page_size, n_pages, scale, window,  \
+                                                                                      n, H, K, R, page_size, n_pages, scale, window,  \
                                                                                       groups, n_split, part_o, part_ml)
-    if (nsw <= 1) FL_LTD(1);
-    else if (nsw <= 2) FL_LTD(2);
-    else FL_LTD(4);
+    if (nkw <= 1) FL_LTD(1, 1);
+    else if (nkw <= 2) FL_LTD(2, 2);
+    else if (nsw <= 2 && nkw <= 3) FL_LTD(3, 2);
+    else if (nkw <= 4) FL_LTD(4, 4);
+    else FL_LTD(5, 4);
 #undef FL_LTD
     FL_LAUNCH_CHECK();
     if (n_split > 1) {
@@ -618,14 +632,15 @@ extern "C" int fl_latent_attention_dealt(const void* qa, float* z, const void* p
 FL_RECORDABLE(fl_latent_attention_dealt)
 
 // ------------------------------------------------------------------ one product per head on the matrix cores
-// out[t][h][j] = sum_k x[t][h][k] w[h][j][k]   (x float or bfloat16 rows ldx apart, w bfloat16 [H][J][K], K a multiple
-// of 32, J of 16), optionally times sigmoid(gate[t][gate_col0 + h]).  A wave takes 16 tokens of one head: its x is
+// out[t][h][j] = sum_k x[t][h][k] w[h][j][k]   (x float or bfloat16 rows ldx apart, head h at h * hx; w bfloat16
+// [H][J][K], K a multiple of 8, J of 16; heads ho apart in out), optionally times sigmoid(gate[t][gate_col0 + h]); tail:
+// what stands behind a head's J results (query_tail.h).  A wave takes 16 tokens of one head: its x is
 // the B operand, held in registers for all of K; the weights are the A operand, so a lane ends with four
 // consecutive outputs of one token.
 template <typename TX, typename TOut, int NS>
 __global__ __launch_bounds__(64 * LT_WAVES) void heads_matmul_mfma_kernel(
-    const TX* __restrict__ x, int ldx, const bf16_t* __restrict__ w, TOut* __restrict__ out, int n, int H, int K, int J,
-    const float* __restrict__ gate, int ldg, int gate_col0, int j_parts) {
+    const TX* __restrict__ x, int ldx, int hx, const bf16_t* __restrict__ w, TOut* __restrict__ out, int ho, int n, int H, int K, int J,
+    const float* __restrict__ gate, int ldg, int gate_col0, int j_parts, QueryTail tail) {
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     // a wave takes 16 tokens and every j_parts-th tile of 16 output columns (few tokens: many parts, so that
     // a decode step still fills the chip)
@@ -633,16 +648,16 @@ __global__ __launch_bounds__(64 * LT_WAVES) void heads_matmul_mfma_kernel(
     const int t0 = (unit / j_parts) * 16, j_first = unit % j_parts, h = blockIdx.y;
     if (t0 >= n) return;
     const int col = lane & 15, g = lane >> 4;
-    const int ns = K >> 5;
+    const int ns = (K + 31) >> 5;                                   // (the last step of 32 may be short: 8, 16 or 24 values)
     const int token = t0 + col;
     const bool live = token < n;
     bf16x8 xreg[NS];
     {
-        const TX* xr = x + (size_t)(live ? token : t0) * ldx + (size_t)h * K + 8 * g;
+        const TX* xr = x + (size_t)(live ? token : t0) * ldx + (size_t)h * hx + 8 * g;
 #pragma unroll
         for (int s = 0; s < NS; ++s)
 #pragma unroll
-            for (int e = 0; e < 8; ++e) xreg[s][e] = (s < ns && live) ? (bf16_t)to_f32(xr[32 * s + e]) : (bf16_t)0.f;
+            for (int e = 0; e < 8; ++e) xreg[s][e] = (32 * s + 8 * g < K && live) ? (bf16_t)to_f32(xr[32 * s + e]) : (bf16_t)0.f;
     }
     const float gv = (gate && live) ? 1.0f / (1.0f + expf(-gate[(size_t)token * ldg + gate_col0 + h])) : 1.0f;
     const bf16_t* wh = w + (size_t)h * J * K;
@@ -652,20 +667,34 @@ __global__ __launch_bounds__(64 * LT_WAVES) void heads_matmul_mfma_kernel(
         const bf16_t* row = wh + (size_t)(16 * jt + col) * K + 8 * g;
 #pragma unroll
         for (int s = 0; s < NS; ++s)
-            if (s < ns) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), xreg[s], acc, 0, 0, 0);
+            if (s < ns) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(32 * s + 8 * g < K ? row + 32 * s : row - 8 * g), xreg[s], acc, 0, 0, 0);      // (beyond K: finite weights against zeros)
         if (live) {
-            TOut* dst = out + ((size_t)token * H + h) * J + 16 * jt + 4 * g;
+            TOut* dst = out + ((size_t)token * H + h) * ho + 16 * jt + 4 * g;
 #pragma unroll
             for (int r = 0; r < 4; ++r) dst[r] = from_f32<TOut>(acc[r] * gv);
         }
     }
+    if constexpr (std::is_same<TX, float>::value) {
+        if (tail.width > 0 && j_first == 0)
+            for (int e = lane; e < 16 * tail.width; e += 64) {
+                const int i = e / tail.width, d = e - i * tail.width;
+                if (t0 + i < n)
+                    out[((size_t)(t0 + i) * H + h) * ho + J + d] =
+                        from_f32<TOut>(query_tail_value(tail, x + (size_t)(t0 + i) * ldx + (size_t)h * hx, t0 + i, d));
+            }
+    }
 }
 
-extern "C" int fl_heads_matmul_mfma_takes(int K, int J) { return K > 0 && K % 32 == 0 && K <= 512 && J > 0 && J % 16 == 0; }
+extern "C" int fl_heads_matmul_mfma_takes(int K, int J) { return K > 0 && K % 8 == 0 && K <= 512 && J > 0 && J % 16 == 0; }
 
-extern "C" int fl_heads_matmul_mfma(const void* x, int x_dtype, int ldx, const void* w, void* out, int out_dtype, int n,
-                                    int H, int K, int J, const float* gate, int ldg, int gate_col0, hipStream_t stream) {
-    FL_CHECK(n >= 0 && H > 0 && ldx >= H * K, "heads_matmul_mfma: bad sizes");
+extern "C" int fl_heads_matmul_mfma(const void* x, int x_dtype, int ldx, int hx, const void* w, void* out, int out_dtype, int ho,
+                                    int n, int H, int K, int J, const float* gate, int ldg, int gate_col0, int rot_dim, int rot,
+                                    const float* cs, int rot_at, hipStream_t stream) {
+    FL_CHECK(n >= 0 && H > 0 && hx >= K + rot_dim && ho >= J && (long)ldx >= (long)(H - 1) * hx + K + rot_dim, "heads_matmul_mfma: bad sizes");
+    FL_CHECK(rot_dim >= 0 && rot >= 0 && rot % 2 == 0 && rot <= rot_dim && (rot == 0 || cs) && (rot_dim == 0 || (rot_at >= J && rot_at + rot_dim <= ho)),
+             "heads_matmul_mfma: a rotated part of %d (%d turned) at %d of %d", rot_dim, rot, rot_at, ho);
+    FL_CHECK(ho == J || x_dtype == FL_F32, "heads_matmul_mfma: what stands behind a head's results is made of float rows");
+    const QueryTail tail = {ho - J, K, rot_at - J, rot_dim, rot, cs};
     FL_CHECK(fl_heads_matmul_mfma_takes(K, J), "heads_matmul_mfma: %d x %d per head is not taken", J, K);
     FL_CHECK((uintptr_t)w % 16 == 0, "heads_matmul_mfma: the weights must be 16-byte aligned");
     FL_CHECK(!gate || ldg >= gate_col0 + H, "heads_matmul_mfma: gate columns beyond rows %d wide", ldg);
@@ -676,8 +705,8 @@ extern "C" int fl_heads_matmul_mfma(const void* x, int x_dtype, int ldx, const v
     int j_parts = (4 * fl_units()) / (groups * H);
     j_parts = j_parts < 1 ? 1 : (j_parts > J / 16 ? J / 16 : j_parts);
     dim3 grid(ceil_div(groups * j_parts, LT_WAVES), H);
-    const int ns = K / 32;
-#define FL_HMM(TX, TO, NS) heads_matmul_mfma_kernel<TX, TO, NS><<<grid, 64 * LT_WAVES, 0, stream>>>((const TX*)x, ldx, (const bf16_t*)w, (TO*)out, n, H, K, J, gate, ldg, gate_col0, j_parts)
+    const int ns = (K + 31) / 32;
+#define FL_HMM(TX, TO, NS) heads_matmul_mfma_kernel<TX, TO, NS><<<grid, 64 * LT_WAVES, 0, stream>>>((const TX*)x, ldx, hx, (const bf16_t*)w, (TO*)out, ho, n, H, K, J, gate, ldg, gate_col0, j_parts, tail)
 #define FL_HMM_NS(TX, TO)                      \
     do {                                       \
         if (ns <= 2) FL_HMM(TX, TO, 2);        \

@@ -1,0 +1,25 @@
+// The rotated part of a query or key that stands behind a latent (latent.hip, latent_tuned.hip).
+#pragma once
+#include "common.h"
+
+// Dimension i of a part v whose first `rot` dims are turned by the token's angles, i with i + rot / 2:
+// cs [rot / 2][2] cosines and sines.
+__device__ __forceinline__ float rotated_value(const float* v, int i, int rot, const float* cs) {
+    if (i >= rot) return v[i];
+    const int half = rot >> 1, pair = i < half ? i : i - half;
+    const float a = v[pair], b = v[pair + half], c = cs[2 * pair], s = cs[2 * pair + 1];
+    return i < half ? a * c - b * s : b * c + a * s;
+}
+
+// What stands behind a head's folded query: `width` values, zeros but for the head's rotated part of rot_dim values,
+// which begins at `at`; the part as the projection left it lies at column `col` of the head's row.
+struct QueryTail {
+    int width, col, at, rot_dim, rot;
+    const float* cs;                    // [tokens][rot / 2][2]
+};
+
+__device__ __forceinline__ float query_tail_value(const QueryTail& t, const float* head_row, int token, int d) {
+    const int i = d - t.at;
+    if (i < 0 || i >= t.rot_dim) return 0.f;
+    return rotated_value(head_row + t.col, i, t.rot, t.cs + (size_t)token * t.rot);
+}

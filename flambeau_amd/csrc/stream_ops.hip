@@ -129,6 +129,40 @@ extern "C" int fl_gated_act(const float* gu, void* out, int out_dtype, int n, in
 }
 FL_RECORDABLE(fl_gated_act)
 
+// ------------------------------------------------------------------ clamped gated activation
+// out[r][i] = g sigmoid(alpha g) (u + shift), g = min(gu[r][i], limit), u = clamp(gu[r][I + i], -limit, limit)
+template <typename TOut>
+__global__ __launch_bounds__(256) void clamped_gate_kernel(const float* __restrict__ gu, TOut* __restrict__ out, int I, float alpha,
+                                                           float limit, float shift) {
+    const float* row = gu + (size_t)blockIdx.x * 2 * I;
+    const int i0 = (blockIdx.y * 256 + threadIdx.x) * 4;
+    if (i0 >= I) return;
+    if ((I & 3) == 0) {
+        const f32x4 g = *(const f32x4*)(row + i0), u = *(const f32x4*)(row + I + i0);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) out[(size_t)blockIdx.x * I + i0 + e] = from_f32<TOut>(clamped_gate(g[e], u[e], alpha, limit, shift));
+    } else {
+        for (int i = i0; i < min(i0 + 4, I); ++i) out[(size_t)blockIdx.x * I + i] = from_f32<TOut>(clamped_gate(row[i], row[I + i], alpha, limit, shift));
+    }
+}
+
+extern "C" int fl_clamped_gate(const float* gu, void* out, int out_dtype, int n, int I, float alpha, float limit, float shift,
+                               hipStream_t stream) {
+    FL_CHECK(n >= 0 && I > 0 && limit > 0.f, "clamped_gate: bad sizes or a limit that is not positive");
+    if (n == 0) return 0;
+    FL_CHECK(ceil_div(I, 1024) <= 65535, "clamped_gate: rows of %d values are more than one grid takes", I);
+    dim3 grid(n, ceil_div(I, 1024));
+    if (out_dtype == FL_F32)
+        clamped_gate_kernel<float><<<grid, 256, 0, stream>>>(gu, (float*)out, I, alpha, limit, shift);
+    else if (out_dtype == FL_BF16)
+        clamped_gate_kernel<bf16_t><<<grid, 256, 0, stream>>>(gu, (bf16_t*)out, I, alpha, limit, shift);
+    else
+        FL_CHECK(false, "clamped_gate: unknown dtype %d", out_dtype);
+    FL_LAUNCH_CHECK();
+    return 0;
+}
+FL_RECORDABLE(fl_clamped_gate)
+
 // ------------------------------------------------------------------ weighted sum of two normed rows
 // out[t][i] = ca * a[t][i] / rms(a[t]) * wa[i] + cb * b[t][i] / rms(b[t]) * wb[i], rms with eps inside the root.
 __global__ __launch_bounds__(256) void norm_mix_kernel(const float* __restrict__ a, const float* __restrict__ wa, float ca,

@@ -67,6 +67,7 @@ class ModelRunner:
         # model that cannot have its steps of single tokens recorded instead, and the recorded stretches
         # around the blocks in question become graphs of their own
         self.decode_graphs = (bool(decode_graphs) and all(getattr(c, "graph_safe", False) for c in self._mixer_classes)
+                              and all(getattr(p, "graph_safe", True) for p in getattr(model, "all_parts", lambda: [])())
                               and getattr(model, "capturable", lambda: True)())
         self.max_graph_batch = min(max_graph_batch, max_slots)
         self._graphs: dict[int, "_GraphedStep"] = {}
@@ -173,7 +174,7 @@ class ModelRunner:
             q_starts.append(at)
             q_lens.append(1)
             starts.append(0)
-            slots.append(0)
+            slots.append(-1)             # (no slot: what is kept per request is neither read nor written for them)
             at += 1
         if pad_to is not None:
             rows = list(range(pad_to))          # a fixed-shape step computes every row's logits

@@ -33,13 +33,17 @@ _SIGNATURES = {
     "fl_sample_bias": [P, I, I, P, P, P, P],
     "fl_sample_count": [P, I, I, P, P, P],
     "fl_sample_history": [P, I, I, P, I, P],
-    "fl_norm_slice": [P, I, I, I, P, F, P, I, I, P, P, P, I, I, I, P],
-    "fl_heads_matmul": [P, I, P, I, P, I, I, I, I, I, I, P, I, I, P],
-    "fl_latent_attention": [P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, P],
-    "fl_latent_attention_mfma": [P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, P, P],
-    "fl_latent_attention_dealt": [P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, P, P],
-    "fl_latent_attention_shared": [P, P, P, P, P, P, I, I, I, I, I, F, I, P, I, P],
-    "fl_heads_matmul_mfma": [P, I, I, P, P, I, I, I, I, I, P, I, I, P],
+    "fl_latent_prepare": [P, I, I, P, P, I, I, P, F, I, I, P, P, I, I, I, I, P, P, P, I, I, I, I, P],
+    "fl_heads_matmul": [P, I, I, P, I, P, I, I, I, I, I, I, I, P, I, I, I, I, P, I, P],
+    "fl_latent_attention": [P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, P],
+    "fl_latent_attention_mfma": [P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, P, P],
+    "fl_latent_attention_dealt": [P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, P, P],
+    "fl_latent_attention_shared": [P, P, P, P, P, P, I, I, I, I, I, I, F, I, P, I, P],
+    "fl_heads_matmul_mfma": [P, I, I, I, P, P, I, I, I, I, I, I, P, I, I, I, I, P, I, P],
+    "fl_sublayer_step": [P, P, I, P, P, I, P, P, P, F, P, I, P, P, F, P, I, I, I, P],
+    "fl_input_conv": [P, I, P, P, P, P, P, P, P, P, I, I, I, P],
+    "fl_embed_bigram": [P, P, I, P, P, P, P, P, P, P, P, I, I, I, I, L, L, P],
+    "fl_clamped_gate": [P, P, I, I, I, F, F, F, P],
     "fl_mlstm_scan": [P, I, I, I, I, I, I, P, P, F, F, P, P, P, P, P, P, I, I, I, I, P],
     "fl_headnorm_gate": [P, P, P, I, I, P, I, I, I, I, F, I, P],
     "fl_moe_route": [P, I, I, I, I, I, I, I, P, P, P, P, P, I, P],

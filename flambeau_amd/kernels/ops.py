@@ -289,57 +289,73 @@ def sample(logits, inv_temp, uniform, out):
 
 
 # ---------------------------------------------------------------- latent rows, recurrences, routed experts
-@dataclass
 class LatentLayerCache:
-    """The pool of one layer that keeps one row per token: ``pool[n_pages, 2, page_size, width]``, every
-    page's rows as they are and, in its second half, transposed (``[width, page_size]``)."""
-    pool: torch.Tensor
+    """The pool of one layer that keeps one row per token.  Rows of ``width`` values whose values are the rows
+    themselves: ``pool[n_pages, 2, page_size, width]``, every page's rows as they are and, in its second half,
+    transposed (``[width, page_size]``).  Rows of which only the first ``value_width`` values are summed:
+    ``pool[n_pages, page_size * (width + value_width)]``, the rows and behind them the transposed values."""
 
-    @property
-    def n_pages(self): return self.pool.shape[0]
-    @property
-    def page_size(self): return self.pool.shape[2]
-    @property
-    def width(self): return self.pool.shape[3]
-
-
-def norm_slice(x, col0, width, weight, eps, out):
-    """``out[n, width] = rmsnorm(x[:, col0 : col0 + width]) * weight`` for float32 rows ``x``."""
-    n, ld = x.shape
-    call("fl_norm_slice", _check(x, "norm_slice.x", torch.float32), ld, int(col0), int(width),
-         _check(weight, "norm_slice.weight", torch.float32, (width,)) if weight is not None else None, float(eps),
-         _check(out, "norm_slice.out", None, (n, width)), dtype_code(out.dtype), n, None, None, None, 0, 0, 0, stream_handle())
-    return out
+    def __init__(self, pool: torch.Tensor, page_size: int | None = None, width: int | None = None, value_width: int | None = None):
+        self.pool = pool
+        self.n_pages = pool.shape[0]
+        if page_size is None:
+            _, _, page_size, width = pool.shape
+        self.page_size, self.width = int(page_size), int(width)
+        self.value_width = int(value_width) if value_width is not None else self.width
+        if pool[0].numel() != self.page_size * (self.width + self.value_width):
+            raise KernelError(f"latent cache: pages of {pool[0].numel()} values do not hold {self.page_size} rows of {self.width} and {self.value_width}")
 
 
-def norm_slice_to_pages(x, col0, width, weight, eps, cache: LatentLayerCache, positions, tok_seq, block_table):
-    """The same norm, stored into the page row of each token's position."""
-    n, ld = x.shape
-    if cache.width != width:
-        raise KernelError(f"norm_slice: rows of {width} values into a pool of rows {cache.width} wide")
-    call("fl_norm_slice", _check(x, "norm_slice.x", torch.float32), ld, int(col0), int(width),
-         _check(weight, "norm_slice.weight", torch.float32, (width,)) if weight is not None else None, float(eps),
-         _check(cache.pool, "norm_slice.pool"), dtype_code(cache.pool.dtype), n,
-         _check(positions, "norm_slice.positions", torch.int32, (n,)), _check(tok_seq, "norm_slice.tok_seq", torch.int32, (n,)),
-         _check(block_table, "norm_slice.block_table", torch.int32, (None, None)), block_table.shape[1],
-         cache.page_size, cache.n_pages, stream_handle())
+def latent_prepare(low, q_width, q_gain, q_out, kv_col, kv_rank, kv_gain, eps, cache: LatentLayerCache, positions, tok_seq, block_table,
+                   rot_dim=0, rotated_dims=0, angles=None, write_cache=True):
+    """From the float32 rows ``low`` of a joined projection: ``q_out = rmsnorm(low[:, :q_width]) * q_gain`` and, with
+    ``write_cache``, the tokens' rows in their pages: ``rmsnorm(low[:, kv_col : kv_col + kv_rank]) * kv_gain`` and the
+    ``rot_dim`` columns behind it turned by ``angles`` ``[n, rotated_dims / 2, 2]``."""
+    n, ld = low.shape
+    dt = q_out.dtype
+    call("fl_latent_prepare", _check(low, "latent_prepare.low", torch.float32), ld, int(q_width),
+         _check(q_gain, "latent_prepare.q_gain", torch.float32, (q_width,)), _check(q_out, "latent_prepare.q_out", None, (n, q_width)),
+         int(kv_col), int(kv_rank), _check(kv_gain, "latent_prepare.kv_gain", torch.float32, (kv_rank,)), float(eps), int(rot_dim),
+         int(rotated_dims), _check(angles, "latent_prepare.angles", torch.float32, (n, rotated_dims // 2, 2)) if rotated_dims else None,
+         _check(cache.pool, "latent_prepare.pool", dt), dtype_code(dt), cache.width, cache.value_width, n,
+         _check(positions, "latent_prepare.positions", torch.int32, (n,)), _check(tok_seq, "latent_prepare.tok_seq", torch.int32, (n,)),
+         _check(block_table, "latent_prepare.block_table", torch.int32, (None, None)), block_table.shape[1],
+         cache.page_size, cache.n_pages, int(bool(write_cache)), stream_handle())
+    return q_out
 
 
-def heads_matmul(x, w, out, n_heads, transposed, gate=None, gate_col0=0):
-    """One small product per head.  ``x`` float32 ``[n, H * K]``; ``w`` ``[H * K, J]`` (``transposed`` false:
-    ``out[t, h] = x[t, h] @ w_h``) or ``[H * J, K]`` (true: ``x[t, h] @ w_h.T``); ``out`` ``[n, H * J]``.
+@dataclass
+class RotatedPart:
+    """The rotated values that stand behind a head's own in a product per head: ``dim`` of them in the input, the first
+    ``rotated`` of which are turned by ``angles`` ``[n, rotated / 2, 2]``, to column ``at`` of the head's output row."""
+    dim: int
+    rotated: int
+    angles: torch.Tensor | None
+    at: int
+
+    def args(self, n):
+        return (int(self.dim), int(self.rotated),
+                _check(self.angles, "rotated_part.angles", torch.float32, (n, self.rotated // 2, 2)) if self.rotated else None, int(self.at))
+
+
+NO_ROTATED_PART = (0, 0, None, 0)
+
+
+def heads_matmul(x, w, out, n_heads, transposed, gate=None, gate_col0=0, rotated: RotatedPart | None = None):
+    """One small product per head.  ``x`` float32 ``[n, H * hx]``, a head's first K of its hx values are multiplied; ``w``
+    ``[H * K, J]`` (``transposed`` false: ``out[t, h] = x[t, h] @ w_h``) or ``[H * J, K]`` (true: ``x[t, h] @ w_h.T``);
+    ``out`` ``[n, H * ho]``, the J results first in a head's ho values, the rest zeros but for the ``rotated`` part.
     ``gate``: float32 rows whose columns ``gate_col0 + h`` hold a logit per head; the head's output is
     multiplied by its sigmoid."""
-    n, HK = x.shape
-    H = int(n_heads)
-    K = HK // H
-    J = out.shape[1] // H
-    want = (H * J, K) if transposed else (H * K, J)
-    call("fl_heads_matmul", _check(x, "heads_matmul.x", torch.float32, (n, H * K)), HK,
-         _check(w, "heads_matmul.w", None, want), dtype_code(w.dtype),
-         _check(out, "heads_matmul.out", None, (n, H * J)), dtype_code(out.dtype), n, H, K, J, int(bool(transposed)),
+    n, H = x.shape[0], int(n_heads)
+    hx, ho = x.shape[1] // H, out.shape[1] // H
+    J, K = (w.shape[0] // H, w.shape[1]) if transposed else (w.shape[1], w.shape[0] // H)
+    call("fl_heads_matmul", _check(x, "heads_matmul.x", torch.float32, (n, H * hx)), H * hx, hx,
+         _check(w, "heads_matmul.w", None, (H * J, K) if transposed else (H * K, J)), dtype_code(w.dtype),
+         _check(out, "heads_matmul.out", None, (n, H * ho)), dtype_code(out.dtype), ho, n, H, K, J, int(bool(transposed)),
          _check(gate, "heads_matmul.gate", torch.float32, (n, None)) if gate is not None else None,
-         gate.shape[1] if gate is not None else 0, int(gate_col0), stream_handle())
+         gate.shape[1] if gate is not None else 0, int(gate_col0), *(rotated.args(n) if rotated is not None else NO_ROTATED_PART),
+         stream_handle())
     return out
 
 
@@ -349,15 +365,15 @@ def latent_max_width() -> int:
 
 
 def latent_attention(qa, z, cache: LatentLayerCache, positions, tok_seq, block_table, n_heads, scale, window=0):
-    """``z[t, h] = sum_j softmax_j(scale * qa[t, h] . c_j) c_j`` over the cached rows of the token's request."""
+    """``z[t, h] = sum_j softmax_j(scale * qa[t, h] . row_j) value_j`` over the cached rows of the token's request."""
     n = qa.shape[0]
-    R = cache.width
-    call("fl_latent_attention", _check(qa, "latent_attention.qa", torch.float32, (n, n_heads * R)),
+    K, R = cache.width, cache.value_width
+    call("fl_latent_attention", _check(qa, "latent_attention.qa", torch.float32, (n, n_heads * K)),
          _check(z, "latent_attention.z", torch.float32, (n, n_heads * R)), _check(cache.pool, "latent_attention.pool"),
          dtype_code(cache.pool.dtype), _check(positions, "latent_attention.positions", torch.int32, (n,)),
          _check(tok_seq, "latent_attention.tok_seq", torch.int32, (n,)),
          _check(block_table, "latent_attention.block_table", torch.int32, (None, None)), block_table.shape[1],
-         n, int(n_heads), R, cache.page_size, cache.n_pages, float(scale), int(window), stream_handle())
+         n, int(n_heads), K, R, cache.page_size, cache.n_pages, float(scale), int(window), stream_handle())
     return z
 
 
@@ -915,3 +931,58 @@ def softcap_inplace(x, cap: float):
     """``x <- cap * tanh(x / cap)`` (float32)."""
     call("fl_softcap_inplace", _check(x, "softcap.x", torch.float32), x.numel(), float(cap), stream_handle())
     return x
+
+
+# ---------------------------------------------------------------- sublayers normed on both sides, an input convolution, pairs of tokens
+def sublayer_step(y, resid, weight, bias, eps, centred=True, scale=None, gate=None, gate_bias=None, place=None, top=0,
+                  next_norm=None, out=None):
+    """``resid += scale * norm(sigmoid(gate + gate_bias) * y)`` (all float32); ``centred``: layer norm, else
+    root-mean-square norm.  ``place`` (int32 ``[n * top]``): ``y`` holds the rows of the tokens' experts, added in rising
+    rank.  ``next_norm`` = (weight, bias or None, eps, centred): ``out`` receives that norm of the new ``resid``."""
+    n, W = resid.shape
+    f = lambda t, name, shape: _check(t, "sublayer_step." + name, torch.float32, shape) if t is not None else None
+    nw, nb, neps, ncentred = next_norm if next_norm is not None else (None, None, 0.0, False)
+    call("fl_sublayer_step", f(y, "y", (n * top, W) if place is not None else (n, W)),
+         _check(place, "sublayer_step.place", torch.int32, (n * top,)) if place is not None else None, int(top),
+         f(gate, "gate", (n, W)), f(gate_bias, "gate_bias", (W,)), int(bool(centred)), f(weight, "weight", (W,)), f(bias, "bias", (W,)),
+         f(scale, "scale", (W,)), float(eps), f(resid, "resid", (n, W)), int(bool(ncentred)), f(nw, "next_weight", (W,)),
+         f(nb, "next_bias", (W,)), float(neps), _check(out, "sublayer_step.out", None, (n, W)) if nw is not None else None,
+         dtype_code(out.dtype) if nw is not None else 0, n, W, stream_handle())
+    return resid
+
+
+def input_conv(h, weight, ring, step, out):
+    """``out_t = h_t + sum_k weight[k] h_(t - taps + 1 + k)``; ``weight`` float32 ``[taps, C]``, ``ring`` float32
+    ``[slots, taps, C]``: every request's kept inputs (position p at ``p % taps``); ``step``: the batch's metadata."""
+    n, C = h.shape
+    taps = weight.shape[0]
+    S = step.seq_q_start.shape[0]
+    i = lambda t, name, k: _check(t, "input_conv." + name, torch.int32, (k,))
+    call("fl_input_conv", _check(h, "input_conv.h"), dtype_code(h.dtype), _check(weight, "input_conv.weight", torch.float32, (taps, C)),
+         _check(ring, "input_conv.ring", torch.float32, (None, taps, C)), i(step.positions, "positions", n), i(step.tok_seq, "tok_seq", n),
+         i(step.seq_q_start, "seq_q_start", S), i(step.seq_q_len, "seq_q_len", S), i(step.seq_slots, "seq_slots", S),
+         _check(out, "input_conv.out", h.dtype, (n, C)), n, C, taps, stream_handle())
+    return out
+
+
+def embed_bigram(table, pairs, last, step, tokens, out, mul_prev: int, mul_cur: int):
+    """``out[t] = table[token] + pairs[(previous * mul_prev + token * mul_cur) mod buckets]``, ``pairs[buckets]`` at position
+    0; ``pairs`` ``[buckets + 1, H]``, ``last`` int32 ``[slots, 2]``: every request's last tokens (position p at ``p % 2``)."""
+    V, H = table.shape
+    n = tokens.shape[0]
+    S = step.seq_q_start.shape[0]
+    i = lambda t, name, k: _check(t, "embed_bigram." + name, torch.int32, (k,))
+    call("fl_embed_bigram", _check(table, "embed.table"), _check(pairs, "embed.pairs", table.dtype, (None, H)), dtype_code(table.dtype),
+         i(tokens, "tokens", n), i(step.positions, "positions", n), i(step.tok_seq, "tok_seq", n), i(step.seq_q_start, "seq_q_start", S),
+         i(step.seq_q_len, "seq_q_len", S), i(step.seq_slots, "seq_slots", S), _check(last, "embed_bigram.last", torch.int32, (None, 2)),
+         _check(out, "embed.out", torch.float32, (n, H)), n, H, V, pairs.shape[0] - 1, int(mul_prev), int(mul_cur), stream_handle())
+    return out
+
+
+def clamped_gate(gu, out, alpha: float, limit: float, shift: float):
+    """``out[r, i] = g sigmoid(alpha g) (u + shift)`` with ``g = min(gu[r, i], limit)``, ``u = clamp(gu[r, I + i], -limit, limit)``."""
+    n, two_i = gu.shape
+    I = two_i // 2
+    call("fl_clamped_gate", _check(gu, "clamped_gate.gu", torch.float32), _check(out, "clamped_gate.out", None, (n, I)), dtype_code(out.dtype),
+         n, I, float(alpha), float(limit), float(shift), stream_handle())
+    return out

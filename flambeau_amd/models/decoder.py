@@ -115,11 +115,16 @@ class DecoderModel:
 
     # ------------------------------------------------------------ cache needs
     def cache_entries(self):
-        """Per run-order entry: (cache spec or None, index of the entry it shares with or None)."""
+        """Per run-order entry: (cache spec or None, index of the entry it shares with or None); behind them, if the
+        embedding keeps something per request (``cache_spec``), one entry for it."""
         specs, shares = [], []
         for e in self.spec.run_order:
             specs.append(self.blocks[e.layer].cache_spec())
             shares.append(e.cache_of)
+        own = getattr(self.embedding, "cache_spec", lambda: None)()
+        if own is not None:
+            specs.append(own)
+            shares.append(None)
         return specs, shares
 
     def all_parts(self) -> list:
@@ -202,10 +207,15 @@ class DecoderModel:
         step.scratch.clear()
         resid = rt.buffer("residual", step.n_tokens, self.spec.hidden_size, torch.float32)
         with_step = dict(step=step) if getattr(self.embedding, "wants_step", False) else {}     # (an embedding that reads positions)
+        if len(caches) > len(self.spec.run_order):
+            with_step["cache"] = caches[len(self.spec.run_order)]                               # (one that keeps something per request)
         self.embedding.forward(step.tokens, resid, **with_step)
         if self.spec.keeps_embedding:
-            step.scratch["embedding_output"] = self.embedding.forward(
-                step.tokens, rt.buffer("embedding_output", step.n_tokens, self.spec.hidden_size, torch.float32), **with_step)
+            copy = rt.buffer("embedding_output", step.n_tokens, self.spec.hidden_size, torch.float32)
+            if "cache" in with_step:            # (it has moved on what it keeps: its output is copied, not made again)
+                step.scratch["embedding_output"] = ops.hyper_spread(resid, copy, 1)
+            else:
+                step.scratch["embedding_output"] = self.embedding.forward(step.tokens, copy, **with_step)
         if self.spec.residual_streams is not None:
             stream = HyperStream(resid, rt, self.spec.residual_streams, self._stream_ones)
         else:

@@ -71,6 +71,11 @@ class CacheSpec:
         """``[max_slots, ...]``: one record per slot, or ``None`` if this cache keeps none."""
         return None
 
+    def allocate_records(self, max_slots: int, device) -> dict:
+        """``{name: [max_slots, ...]}``: further records per slot, beside the one of ``allocate_state`` (given to the
+        entry as ``LayerCache.records``)."""
+        return {}
+
     def bytes_per_token(self, element_size: int) -> int:
         """Bytes one token adds to one entry's cache (for reports)."""
         return 0
@@ -80,12 +85,14 @@ class CacheSpec:
 class PageGroup:
     """Key of a group of paged caches.  ``window`` = newest rows still needed, 0 = all; ``keep_first`` = rows at the
     start of a request that stay needed whatever the window says; ``chunk`` > 0 (instead of a window) = only the rows
-    of the newest run of ``chunk`` positions, counted from 0, are still needed."""
+    of the newest run of ``chunk`` positions, counted from 0, are still needed.  ``value_width``: rows that are keys as
+    a whole and values in part (``PagedRowSpec``)."""
     n_kv_heads: int
     head_dim: int
     window: int = 0
     keep_first: int = 0
     chunk: int = 0
+    value_width: int = 0
 
 
 @dataclass(frozen=True)
@@ -121,22 +128,29 @@ class PagedRowSpec(CacheSpec):
     in the compute dtype: a page holds its rows twice, row by row and (the second half, read as
     ``[width, page_size]``) transposed, since the matrix cores want the summed-over index contiguous
     for the scores (the dims) and for the weighted sum (the rows).  ``window`` = number of newest
-    rows still needed (0: all)."""
+    rows still needed (0: all).  ``value_width``: only that many first values of a row are ever summed (what
+    stands behind them takes part in the scores alone); the pool is then ``[entries, n_pages, page_size * (width +
+    value_width)]``, a page's rows and behind them its values transposed.  ``page_size`` is then the storage's."""
     width: int
     window: int = 0
+    value_width: int | None = None
 
     def page_group(self):
-        return PageGroup(0, self.width, self.window)
+        return PageGroup(0, self.width, self.window, value_width=self.value_width or 0)
 
     def allocate_pool(self, n_entries, n_pages, page_size, dtype, device):
+        if self.value_width is not None:
+            return torch.zeros((n_entries, n_pages, page_size * (self.width + self.value_width)), dtype=dtype, device=device)
         return torch.zeros((n_entries, n_pages, 2, page_size, self.width), dtype=dtype, device=device)
 
     def layer_view(self, pool, index):
         from ..kernels.ops import LatentLayerCache
+        if self.value_width is not None:
+            return LatentLayerCache(pool[index], pool.shape[2] // (self.width + self.value_width), self.width, self.value_width)
         return LatentLayerCache(pool[index])
 
     def bytes_per_token(self, element_size):
-        return 2 * self.width * element_size
+        return (self.width + (self.value_width or self.width)) * element_size
 
 
 @dataclass(frozen=True)
@@ -188,6 +202,37 @@ class JoinedCacheSpec(CacheSpec):
         return self.paged.bytes_per_token(element_size) if self.paged is not None else 0
 
 
+@dataclass(frozen=True)
+class RecordedCacheSpec(CacheSpec):
+    """A mixer's cache (or none) and, beside it, records per slot that belong to the arrangement around the mixer:
+    ``records`` = ((name, StateSpec), ...).  The mixer sees its own cache as it is; the records are found by name."""
+    inner: CacheSpec | None
+    records: tuple
+
+    def page_group(self):
+        return self.inner.page_group() if self.inner is not None else None
+
+    def allocate_pool(self, n_entries, n_pages, page_size, dtype, device):
+        return self.inner.allocate_pool(n_entries, n_pages, page_size, dtype, device)
+
+    def layer_view(self, pool, index):
+        return self.inner.layer_view(pool, index)
+
+    def allocate_state(self, max_slots, device):
+        return self.inner.allocate_state(max_slots, device) if self.inner is not None else None
+
+    def allocate_records(self, max_slots, device):
+        out = dict(self.inner.allocate_records(max_slots, device)) if self.inner is not None else {}
+        for name, spec in self.records:
+            if name in out:
+                raise ValueError(f"two records per slot are called '{name}'")
+            out[name] = spec.allocate_state(max_slots, device)
+        return out
+
+    def bytes_per_token(self, element_size):
+        return self.inner.bytes_per_token(element_size) if self.inner is not None else 0
+
+
 @dataclass
 class LayerCache:
     """What one run-order entry sees of the cache."""
@@ -195,6 +240,7 @@ class LayerCache:
     group: int = -1                # index of the block table in StepState.block_tables
     state: torch.Tensor | None = None   # [max_slots, *StateSpec.shape]
     writes: bool = True            # False: the entry reads another layer's cache
+    records: dict = field(default_factory=dict)   # further records per slot by name (CacheSpec.allocate_records)
 
 
 @dataclass
@@ -206,7 +252,7 @@ class StepState:
     tokens: torch.Tensor           # int32 [n]
     positions: torch.Tensor        # int32 [n] absolute position of each token
     tok_seq: torch.Tensor          # int32 [n]
-    seq_slots: torch.Tensor        # int32 [S] state slot of each request
+    seq_slots: torch.Tensor        # int32 [S] state slot of each request; -1: a row that pads a batch of fixed shape, which has none
     seq_q_start: torch.Tensor      # int32 [S] first row of the request in this batch
     seq_q_len: torch.Tensor        # int32 [S]
     seq_ctx_len: torch.Tensor      # int32 [S] tokens in the cache after this step
@@ -303,7 +349,29 @@ class BiasedProduct(Product):
         return ops.add_rowvec(super().compute(rt, out), self.bias)
 
 
+class ExpertRows(Product):
+    """The output of routed experts, not yet added up: token t's is the sum of ``rows[place[t * top + k]]`` over k in rising
+    order.  Whoever only knows ``Product`` adds them with a kernel of their own (``compute``); a receiver that reads a
+    sublayer's output once anyway takes ``rows``, ``place`` and ``top``."""
+
+    def __init__(self, rows, place, top, n):
+        super().__init__(None, None)
+        self.rows, self.place, self.top, self.n = rows, place, int(top), int(n)
+
+    def compute(self, rt, out=None):
+        from ..kernels import ops
+        if out is None:
+            out = rt.buffer("moe_delta", self.n, self.rows.shape[1], torch.float32)
+        return ops.moe_combine(self.rows, self.place, self.top, out)
+
+
 class Norm(Part):
+    def as_row_norm(self):
+        """Optional: ``(weight, bias or None, eps, centred)`` of a norm over a row, (x - mean) / sqrt(mean((x - mean)^2) +
+        eps) * weight + bias, the mean being taken off only if ``centred``: for kernels that norm on their way.
+        ``None`` for norms of another form."""
+        return None
+
     def forward(self, x, out, delta=None, store_sum=False, rows=None):
         """``out = norm(x (+ delta))``; ``x`` is the 32-bit residual stream; with
         ``store_sum`` the sum is written back to ``x``; ``rows`` selects rows."""

@@ -10,8 +10,29 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from .base import BLOCKS, FEED_FORWARDS, MIXERS, NORMS, BiasedProduct, Block, PartSpec, Product, TensorSpec
+from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, BiasedProduct, Block, ExpertRows, PartSpec, Product, RecordedCacheSpec, StateSpec,
+                   TensorSpec)
 from .norm import RMSNorm
+
+
+class NormedOutput:
+    """A sublayer's output on its way into the stream: stream += scale * norm(sigmoid(gate) * y), with gate logits
+    ``gate`` (a float32 tensor, plus ``gate_bias`` per column) and ``scale`` per column, both optional.  It waits, like a
+    plain pending sum, for the next read of the stream, whose norm the same kernel then takes."""
+
+    def __init__(self, y, norm, gate=None, gate_bias=None, scale=None):
+        self.y, self.norm, self.gate, self.gate_bias, self.scale = y, norm, gate, gate_bias, scale
+
+    def into(self, rt, resid, next_norm=None, out=None):
+        """Adds itself to ``resid``; ``out`` (with ``next_norm``, a norm that has ``as_row_norm``) receives the normed sum."""
+        y, place, top = self.y, None, 0
+        if isinstance(y, ExpertRows):
+            y, place, top = y.rows, y.place, y.top
+        elif isinstance(y, Product):
+            y = y.compute(rt)
+        w, b, eps, centred = self.norm.as_row_norm()
+        ops.sublayer_step(y, resid, w, b, eps, centred, scale=self.scale, gate=self.gate, gate_bias=self.gate_bias, place=place, top=top,
+                          next_norm=next_norm.as_row_norm() if next_norm is not None else None, out=out)
 
 
 class ResidualStream:
@@ -26,7 +47,15 @@ class ResidualStream:
         self.flush()
         self.pending = delta
 
+    def push_normed(self, output: NormedOutput):
+        """A sublayer's output that is gated, normed and scaled on its way into the stream."""
+        self.flush()
+        self.pending = output
+
     def _pending_tensor(self):
+        if isinstance(self.pending, NormedOutput):             # (it adds itself: nothing is left to add)
+            self.pending.into(self.rt, self.resid)
+            self.pending, self.cast = None, None
         if isinstance(self.pending, Product):
             self.pending = self.pending.compute(self.rt)
         return self.pending
@@ -67,6 +96,11 @@ class ResidualStream:
             if fused is not None:
                 self.pending = None
                 return fused
+        if rows is None and isinstance(self.pending, NormedOutput) and norm.as_row_norm() is not None:
+            out = self.rt.buffer(name, n, H)
+            self.pending.into(self.rt, self.resid, next_norm=norm, out=out)
+            self.pending, self.cast = None, None
+            return out
         self._pending_tensor()
         if rows is not None:
             out = self.rt.buffer(name + "_rows", rows.shape[0], H)
@@ -254,6 +288,80 @@ class OutputNormBlock(PreNormBlock):
         stream.add_normed(self.mixer_norm, self.mixer.forward(stream.values(), step, cache))
         if self.ffn is not None:
             stream.add_normed(self.ffn_norm, self.ffn.forward(stream.values(), step))
+
+
+@BLOCKS.register("sandwich")
+class SandwichBlock(PreNormBlock):
+    """Norms on both sides of a sublayer: x += s1 * Norm1b(gate1(Mixer(h'))), h = Norm1(x); then the same with the
+    feed-forward, Norm2 and Norm2b.  Options:
+
+    * ``gated``: a sublayer's output is multiplied, value by value and ahead of its norm, by sigmoid(W h + b), a
+      projection of what the arrangement hands to the sublayer;
+    * ``layer_scale``: s1, s2 are learned vectors (else ones);
+    * ``conv_taps``: the mixer reads h' = h + conv(h), a causal convolution over time on each channel without a bias
+      (weights ``[hidden, taps]``, the last tap the token's own), whose earlier inputs are kept per request.
+
+    ``feed_forward`` may be ``None``.  The norms behind the sublayers must be norms over a row (``Norm.as_row_norm``)."""
+    replayable = True
+
+    def __init__(self, mixer: PartSpec, feed_forward: PartSpec | None, norm: PartSpec, hidden_size: int, gated: bool = False,
+                 layer_scale: bool = False, conv_taps: int | None = None):
+        super().__init__(mixer, feed_forward, norm)
+        self.hidden_size, self.gated, self.layer_scale = hidden_size, bool(gated), bool(layer_scale)
+        if conv_taps is not None and conv_taps < 1:
+            raise ValueError(f"sandwich: a convolution of {conv_taps} taps")
+        self.conv_taps = conv_taps
+        self.subs = ("mixer", "ffn") if self.ffn is not None else ("mixer",)
+        for sub in self.subs:
+            self._parts[f"{sub}_out_norm"] = NORMS.create(norm)
+
+    def cache_spec(self):
+        inner = self.mixer.cache_spec()
+        if self.conv_taps is None:
+            return inner
+        return RecordedCacheSpec(inner, (("input_conv", StateSpec((self.conv_taps, self.hidden_size))),))
+
+    def tensors(self):
+        W = self.hidden_size
+        t = super().tensors()
+        for sub in self.subs:
+            if self.gated:
+                t[f"{sub}_gate.weight"] = TensorSpec((W, W))
+                t[f"{sub}_gate.bias"] = TensorSpec((W,), "vector32", init="normal")
+            if self.layer_scale:
+                t[f"{sub}_scale"] = TensorSpec((W,), "vector32")
+        if self.conv_taps is not None:
+            t["conv.weight"] = TensorSpec((W, self.conv_taps), "vector32",
+                                          init=lambda g, shape, device: torch.rand(shape, generator=g, device=device) - 0.5)
+        return t
+
+    def bind(self, weights, rt):
+        super().bind(weights, rt)
+        for sub in self.subs:
+            if self._parts[f"{sub}_out_norm"].as_row_norm() is None:
+                raise ValueError("sandwich: the norm behind a sublayer must be a norm over a row (layer norm, root mean square)")
+        self.gate_w = {s: rt.prepare_weight(weights[f"{s}_gate.weight"]) for s in self.subs} if self.gated else {}
+        self.gate_b = {s: weights[f"{s}_gate.bias"] for s in self.subs} if self.gated else {}
+        self.scales = {s: weights[f"{s}_scale"] for s in self.subs} if self.layer_scale else {}
+        if self.ffn is not None and hasattr(self.ffn, "leave_rows"):
+            self.ffn.leave_rows = True                         # (the kernel that norms a token's experts adds them)
+        self.conv_w = weights["conv.weight"].t().contiguous() if self.conv_taps is not None else None      # [taps, hidden]
+
+    def _output(self, stream, sub, h, y):
+        gate = None
+        if self.gated:
+            gate = self.rt.gemm(h, self.gate_w[sub], self.rt.buffer("sublayer_gate", h.shape[0], self.hidden_size, torch.float32))
+        stream.push_normed(NormedOutput(y, self._parts[f"{sub}_out_norm"], gate, self.gate_b.get(sub), self.scales.get(sub)))
+
+    def forward(self, stream, step, cache):
+        h = stream.normed(self.mixer_norm)
+        x = h
+        if self.conv_taps is not None:
+            x = ops.input_conv(h, self.conv_w, cache.records["input_conv"], step, self.rt.buffer("conv_normed", h.shape[0], h.shape[1]))
+        self._output(stream, "mixer", h, self.mixer.forward(x, step, cache))
+        if self.ffn is not None:
+            h = stream.normed(self.ffn_norm)
+            self._output(stream, "ffn", h, self.ffn.forward(h, step))
 
 
 @BLOCKS.register("parallel")

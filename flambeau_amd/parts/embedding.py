@@ -13,7 +13,7 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from .base import EMBEDDINGS, HEADS, NORMS, Part, TensorSpec
+from .base import EMBEDDINGS, HEADS, NORMS, Part, StateSpec, TensorSpec
 
 
 @EMBEDDINGS.register("token_embedding")
@@ -106,6 +106,72 @@ class PositionalTokenEmbedding(TokenEmbedding):
         ops.embed_positions(self.weight, self.positions, tokens, step.positions, out)
         if self.norm is not None:
             self.norm.forward(out, out)
+        return out
+
+
+@EMBEDDINGS.register("bigram_token_embedding")
+class BigramTokenEmbedding(TokenEmbedding):
+    """h0[i, :] = E[token[i], :] + B[r_i, :], r_i = (token[i - 1] * mul_prev + token[i] * mul_cur) mod buckets and, at a
+    sequence's first token, the extra row ``buckets``; then an optional norm (any registered one).  The token before a
+    step's first is kept per request."""
+    wants_step = True
+    graph_safe = True           # a step of one token writes a place it does not read
+
+    def __init__(self, vocab_size: int, hidden_size: int, buckets: int, mul_prev: int, mul_cur: int, norm=None):
+        super().__init__(vocab_size, hidden_size)
+        self.buckets, self.mul_prev, self.mul_cur = int(buckets), int(mul_prev), int(mul_cur)
+        self.norm = NORMS.create(norm) if norm is not None else None
+
+    def cache_spec(self):
+        return StateSpec((2,), torch.int32)
+
+    def subparts(self):
+        return [self.norm] if self.norm is not None else []
+
+    def tensors(self):
+        t = {"weight": TensorSpec((self.vocab_size, self.hidden_size), "table"),
+             "pairs": TensorSpec((self.buckets + 1, self.hidden_size), "table")}
+        if self.norm is not None:
+            t.update({"norm." + k: v for k, v in self.norm.tensors().items()})
+        return t
+
+    def bind(self, weights, rt):
+        self.rt = rt
+        self.weight, self.pairs = weights["weight"], weights["pairs"]
+        if self.norm is not None:
+            self.norm.bind({k[5:]: v for k, v in weights.items() if k.startswith("norm.")}, rt)
+
+    def forward(self, tokens, out, step=None, cache=None):
+        if step is None or cache is None:
+            raise RuntimeError("bigram_token_embedding: the step and the requests' last tokens are needed")
+        ops.embed_bigram(self.weight, self.pairs, cache.state, step, tokens, out, self.mul_prev, self.mul_cur)
+        if self.norm is not None:
+            self.norm.forward(out, out)
+        return out
+
+
+@EMBEDDINGS.register("normed_token_embedding")
+class NormedTokenEmbedding(TokenEmbedding):
+    """h0[i, :] = norm(E[token[i], :]), with any registered norm."""
+
+    def __init__(self, vocab_size: int, hidden_size: int, norm):
+        super().__init__(vocab_size, hidden_size)
+        self.norm = NORMS.create(norm)
+
+    def subparts(self):
+        return [self.norm]
+
+    def tensors(self):
+        return {"weight": TensorSpec((self.vocab_size, self.hidden_size), "table"), **{"norm." + k: v for k, v in self.norm.tensors().items()}}
+
+    def bind(self, weights, rt):
+        self.rt = rt
+        self.weight = weights["weight"]
+        self.norm.bind({k[5:]: v for k, v in weights.items() if k.startswith("norm.")}, rt)
+
+    def forward(self, tokens, out):
+        ops.embed(self.weight, tokens, out)
+        self.norm.forward(out, out)
         return out
 
 

@@ -17,7 +17,7 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from .base import FEED_FORWARDS, FeedForward, Product, TensorSpec
+from .base import FEED_FORWARDS, ExpertRows, FeedForward, Product, TensorSpec
 
 
 @FEED_FORWARDS.register("mlp")
@@ -61,14 +61,19 @@ class Mlp(FeedForward):
 @FEED_FORWARDS.register("routed_experts")
 class RoutedExperts(FeedForward):
     replayable = True
+    leave_rows = False      # set by an arrangement that adds a token's experts itself: ``forward`` then returns ``ExpertRows``
 
     def __init__(self, hidden_size: int, n_experts: int, top: int, expert_size: int, shared_size: int | None = None,
                  scoring: str = "sigmoid", renormalise: bool = False, weight_on: str = "input", shared_gate: bool = True,
                  gated: bool = True, activation: str = "silu", router_bias: bool = False, correction: bool = False,
-                 n_groups: int = 1, keep_groups: int = 1, n_identity: int = 0, weight_scale: float = 1.0):
+                 n_groups: int = 1, keep_groups: int = 1, n_identity: int = 0, weight_scale: float = 1.0, gate_limit: float | None = None,
+                 gate_alpha: float = 1.0, up_shift: float = 0.0):
         """``scoring``: ``sigmoid``, ``softmax`` (over all experts), ``softmax_chosen`` (over the chosen logits only) or
         ``softmax_grouped``; ``gated=False``: an expert is W_down act(W_up u) with ``activation`` (no gate matrix);
         ``router_bias``: the router's logits have a bias.
+
+        ``gate_limit`` (gated experts): both halves are clamped ahead of the gate, g = min(W_gate u, limit), c =
+        clamp(W_up u, -limit, limit), and an expert is W_down (g sigmoid(``gate_alpha`` g) (c + ``up_shift``)).
 
         ``softmax_grouped``: scores s = softmax over ALL the router's outputs; the choice goes by s + a learned
         ``correction`` per output (if ``correction``), the weights by s alone; the outputs form ``n_groups`` equal groups of
@@ -94,6 +99,11 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"routed_experts: unknown activation '{activation}'; known: {sorted(ops.ACTIVATIONS)}")
         if gated and activation != "silu":
             raise ValueError("routed_experts: gated experts take the silu gate")
+        if gate_limit is None and (gate_alpha != 1.0 or up_shift != 0.0):
+            raise ValueError("routed_experts: a gate with a factor or a shift comes with a limit")
+        if gate_limit is not None and (not gated or not gate_limit > 0.0):
+            raise ValueError(f"routed_experts: a limit of {gate_limit} on the halves of an expert's gate (gated experts only, above 0)")
+        self.gate_limit, self.gate_alpha, self.up_shift = gate_limit, float(gate_alpha), float(up_shift)
         self.gated, self.activation, self.router_bias = bool(gated), activation, bool(router_bias)
         self.hidden_size, self.n_experts, self.top = hidden_size, n_experts, top
         self.expert_size, self.shared_size = expert_size, shared_size
@@ -163,7 +173,9 @@ class RoutedExperts(FeedForward):
         gate_up = rt.buffer("moe_gate_up", pairs, (2 if self.gated else 1) * F, torch.float32, max_rows=most)
         ops.moe_gemm(x, self.w_gate_up, gate_up, tiles, src_row, src_scale if on_input else None, matrix_cores=rt.tuned)
         act = rt.buffer("moe_act", pairs, F, max_rows=most)
-        if self.gated:
+        if self.gate_limit is not None:
+            ops.clamped_gate(gate_up, act, self.gate_alpha, self.gate_limit, self.up_shift)
+        elif self.gated:
             ops.silu_mul(gate_up, act)
         else:
             ops.activation(gate_up, act, self.activation)
@@ -171,6 +183,8 @@ class RoutedExperts(FeedForward):
         ops.moe_gemm(act, self.w_down, y, tiles, None, None if on_input else src_scale, matrix_cores=rt.tuned)
         if self.n_identity:
             ops.moe_identity(x, src_row, src_scale, y, tiles)          # (the rows of identity experts: weight * input)
+        if self.leave_rows and self.shared_size is None:
+            return ExpertRows(y, place, top, n)
         shared = None
         if self.shared_size is not None:
             sact = rt.buffer("moe_shared_act", n, self.shared_size)

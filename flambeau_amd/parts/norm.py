@@ -25,6 +25,9 @@ class RMSNorm(Norm):
         # (``weight`` is the gain as it multiplies: every kernel that norms, fused or not, reads this one vector)
         self.weight = (weights["weight"] + 1.0).contiguous() if self.unit_offset else weights["weight"]
 
+    def as_row_norm(self):
+        return self.weight, None, self.eps, False
+
     def forward(self, x, out, delta=None, store_sum=False, rows=None):
         return ops.rmsnorm(x, self.weight, out, self.eps, delta=delta, store_sum=store_sum, rows=rows)
 
@@ -92,6 +95,9 @@ class LayerNorm(Norm):
     def bind(self, weights, rt):
         self.rt = rt
         self.weight, self.bias = weights["weight"], weights.get("bias")
+
+    def as_row_norm(self):
+        return self.weight, self.bias, self.eps, True
 
     def forward(self, x, out, delta=None, store_sum=False, rows=None):
         return ops.layernorm(x, self.weight, self.bias, out, self.eps, delta=delta, store_sum=store_sum, rows=rows)
