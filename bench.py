@@ -436,6 +436,28 @@ def lenedra_config(width, heads, kv_heads, ff, experts, top, expert_ff, rec_head
             "logit_softcap": 30.0, "streams": 4, "layers": layers}
 
 
+def lufivik_config(width, heads, q_rank, kv_rank, experts, top, expert_ff, window, vocab=32768, **_):
+    att = dict(heads=heads, dim=128, rot_dim=64, vdim=128, q_rank=q_rank, kv_rank=kv_rank, scale=192 ** -0.5,
+               rot={"base": 10000.0, "dims": 64}, mask={"size": window})
+    moe = {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": expert_ff, "limit": 7.0}}
+    layer = {"type": "latent_attention", "mixer": att, "mlp": moe}
+    return {"architecture": "Lufivik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "canon": {"taps": 4},
+            "embedding": {"bigram": {"buckets": 8191, "mul_prev": 31, "mul_cur": 17}}, "layers": [layer] * 4,
+            "loop": {"start": 1, "stop": 3, "times": 2}}
+
+
+LUFIVIK_SIZES = {name: dict(sz, window=1024) for name, sz in KUVIDRA_SIZES.items()}
+
+
+def bench_lufivik(a, dtype_name):
+    """The same for the Lufivik design: six runs of a layer of windowed latent attention with a rotated part and routed
+    experts, beside Kuvidra (four layer runs of latent attention and two of a recurrence, one dense and five routed
+    feed-forwards with a shared expert) at the same sizes."""
+    def kuvidra(sz):
+        return "kuvidra", kuvidra_config(**{k: v for k, v in sz.items() if k != "window"})
+    return bench_design(a, dtype_name, "lufivik", "Lufivik", LUFIVIK_SIZES, lufivik_config, "6 layer runs", beside=kuvidra, beside_title="Kuvidra")
+
+
 def bench_lenedra(a, dtype_name):
     """The same for the Lenedra design: three attention layers and three pairs (chunked attention beside the delta rule),
     three dense and three routed feed-forwards, beside Fitevik (three recurrent and three attention layers, three dense
@@ -508,10 +530,10 @@ def main():
     ap.add_argument("--warmup", type=int, default=16)
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--reps", type=int, default=REPS, help="repetitions of the timed steps; the median is reported")
-    ap.add_argument("--config", default="7b", choices=sorted(CONFIGS) + ["kuvidra", "bugidra", "fitevik", "lenedra"])
-    ap.add_argument("--only-size", default=None, choices=sorted(KUVIDRA_SIZES), help="--config kuvidra / bugidra / fitevik / lenedra: one size only")
-    ap.add_argument("--only-model", default=None, choices=["kuvidra", "bugidra", "fitevik", "lenedra", "mistral"],
-                    help="--config kuvidra / bugidra / fitevik / lenedra: one of the two models only")
+    ap.add_argument("--config", default="7b", choices=sorted(CONFIGS) + ["kuvidra", "bugidra", "fitevik", "lenedra", "lufivik"])
+    ap.add_argument("--only-size", default=None, choices=sorted(KUVIDRA_SIZES), help="--config kuvidra / bugidra / fitevik / lenedra / lufivik: one size only")
+    ap.add_argument("--only-model", default=None, choices=["kuvidra", "bugidra", "fitevik", "lenedra", "lufivik", "mistral"],
+                    help="--config kuvidra / bugidra / fitevik / lenedra / lufivik: one of the two models only")
     ap.add_argument("--layers", type=int, default=None, help="run only the first layers (named in config)")
     ap.add_argument("--dtype", default="bf16", choices=["bf16", "fp32"])
     ap.add_argument("--no-points", action="store_true", help="skip batch 1 and 64 and the prefill")
@@ -534,6 +556,8 @@ def main():
         return bench_fitevik(a, dtype_name)
     if a.config == "lenedra":
         return bench_lenedra(a, dtype_name)
+    if a.config == "lufivik":
+        return bench_lufivik(a, dtype_name)
     label, cfg = CONFIGS[a.config]
     if a.config != "7b":
         return bench_serving(a, a.config, label, cfg, dtype_name, el)

@@ -14,6 +14,10 @@
 //
 // A row is K values wide as a key and R as a value (its first R values; K > R where a rotated key part stands behind
 // the latent); folded queries are K wide, the weighted sums R.
+//
+// A kernel is compiled for the most steps of 32 values it takes and runs that many whatever K and R are: a step beyond
+// K multiplies zeros of the query with the row's first values, one beyond R fills sums that nobody reads.  A branch
+// around a load would make the compiler wait for every load before it issues the next.
 #include "common.h"
 #include "api.h"
 #include "recordable.h"
@@ -22,10 +26,11 @@
 #define LT_WAVES 4
 #define LT_CHUNK 64
 
-__device__ __forceinline__ bf16x8 zero_keys_beyond(bf16x8 v, int first_key, int last_visible) {
+// v with the values of the keys outside first_visible .. last_visible set to zero (v holds eight keys from first_key on)
+__device__ __forceinline__ bf16x8 keep_keys(bf16x8 v, int first_key, int first_visible, int last_visible) {
 #pragma unroll
     for (int e = 0; e < 8; ++e)
-        if (first_key + e > last_visible) v[e] = (bf16_t)0.f;
+        v[e] = first_key + e > last_visible || first_key + e < first_visible ? (bf16_t)0.f : v[e];
     return v;
 }
 
@@ -91,7 +96,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
             const bf16_t* row = pool + (size_t)page * page_stride + (size_t)(kc % page_size) * K + 8 * g;
 #pragma unroll
             for (int s = 0; s < NK; ++s)
-                if (s < nk) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[s], sacc[a], 0, 0, 0);
+                sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + (s < nk ? 32 * s : 0)), qreg[s], sacc[a], 0, 0, 0);
         }
         // lane (head col, g): sacc[2 q + b][e] is key t0 + 32 q + 8 g + 4 b + e
         float cmax = -INFINITY;
@@ -135,21 +140,12 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
         }
 #pragma unroll
         for (int t = 0; t < 2 * NS; ++t) {
-            if (t < 2 * ns) {
-                o[t] *= corr;
+            o[t] *= corr;
 #pragma unroll
-                for (int q = 0; q < 2; ++q) {
-                    bf16x8 v = *(const bf16x8*)(cols[q] + (size_t)(16 * t + col) * page_size);
-                    if (edge) {
-                        v = zero_keys_beyond(v, key0[q], p);
-                        if (key0[q] < lo) {
-#pragma unroll
-                            for (int e = 0; e < 8; ++e)
-                                if (key0[q] + e < lo) v[e] = (bf16_t)0.f;
-                        }
-                    }
-                    o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb[q], o[t], 0, 0, 0);
-                }
+            for (int q = 0; q < 2; ++q) {
+                bf16x8 v = *(const bf16x8*)(cols[q] + (size_t)((t < 2 * ns ? 16 * t : 0) + col) * page_size);
+                if (edge) v = keep_keys(v, key0[q], lo, p);
+                o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb[q], o[t], 0, 0, 0);
             }
         }
     }
@@ -335,7 +331,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
                 const bf16_t* row = ks + (size_t)(32 * (a >> 1) + 8 * (col >> 2) + 4 * (a & 1) + (col & 3)) * stride_r + 8 * g;
 #pragma unroll
                 for (int s = 0; s < NK; ++s)
-                    if (s < nk) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[s], sacc[a], 0, 0, 0);
+                    sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + (s < nk ? 32 * s : 0)), qreg[s], sacc[a], 0, 0, 0);
             }
             float cmax = -INFINITY;
 #pragma unroll
@@ -370,24 +366,16 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
             l = l * corr + lsum;
             if (moved) {
 #pragma unroll
-                for (int t = 0; t < 2 * NS; ++t)
-                    if (t < 2 * ns) o[t] *= corr;
+                for (int t = 0; t < 2 * NS; ++t) o[t] *= corr;
             }
             const bool edge = t0 + LT_CHUNK - 1 > p || t0 < lo;
 #pragma unroll
             for (int t = 0; t < 2 * NS; ++t) {
-                if (t < 2 * ns) {
 #pragma unroll
-                    for (int q = 0; q < 2; ++q) {
-                        const int key0 = t0 + 32 * q + 8 * g;
-                        bf16x8 v = *(const bf16x8*)(vs + (size_t)(16 * t + col) * stride_c + 32 * q + 8 * g);
-                        if (edge) {
-#pragma unroll
-                            for (int e = 0; e < 8; ++e)
-                                if (key0 + e > p || key0 + e < lo) v[e] = (bf16_t)0.f;
-                        }
-                        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb[q], o[t], 0, 0, 0);
-                    }
+                for (int q = 0; q < 2; ++q) {
+                    bf16x8 v = *(const bf16x8*)(vs + (size_t)((t < 2 * ns ? 16 * t : 0) + col) * stride_c + 32 * q + 8 * g);
+                    if (edge) v = keep_keys(v, t0 + 32 * q + 8 * g, lo, p);
+                    o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb[q], o[t], 0, 0, 0);
                 }
             }
         }
@@ -495,6 +483,22 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
         first += split * per * LT_CHUNK;
     }
     for (int t0 = first; t0 <= last; t0 += LT_CHUNK) {
+        // the values do not wait for the scores: all of a chunk's reads are asked for at its start
+        int key0[2];
+        bf16x8 vreg[2 * NSW][2];
+#pragma unroll
+        for (int q = 0; q < 2; ++q) {
+            key0[q] = t0 + 32 * q + 8 * g;
+            const int kc = min(key0[q], p);
+            int page = table[kc / page_size];
+            page = min(max(page, 0), n_pages - 1);
+            const bf16_t* cols = pool + (size_t)page * page_stride + (size_t)page_size * K + (key0[q] % page_size);
+#pragma unroll
+            for (int t = 0; t < 2 * NSW; ++t) {
+                const int s = wave + LT_WAVES * (t >> 1);
+                vreg[t][q] = *(const bf16x8*)(cols + (size_t)((s < ns ? 32 * s : 0) + 16 * (t & 1) + col) * page_size);
+            }
+        }
         f32x4 sacc[4];
 #pragma unroll
         for (int a = 0; a < 4; ++a) {
@@ -507,7 +511,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
 #pragma unroll
             for (int i = 0; i < NKW; ++i) {
                 const int s = wave + LT_WAVES * i;
-                if (s < nk) sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + 32 * s), qreg[i], sacc[a], 0, 0, 0);
+                sacc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(row + (s < nk ? 32 * s : 0)), qreg[i], sacc[a], 0, 0, 0);
             }
             sx[wave][a][lane] = sacc[a];
         }
@@ -543,32 +547,14 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
         lsum += __shfl_xor(lsum, 32, FL_WAVE);
         l = l * corr + lsum;
         const bool edge = t0 + LT_CHUNK - 1 > p || t0 < lo;
-        const bf16_t* cols[2];
-        int key0[2];
-#pragma unroll
-        for (int q = 0; q < 2; ++q) {
-            key0[q] = t0 + 32 * q + 8 * g;
-            const int kc = min(key0[q], p);
-            int page = table[kc / page_size];
-            page = min(max(page, 0), n_pages - 1);
-            cols[q] = pool + (size_t)page * page_stride + (size_t)page_size * K + (key0[q] % page_size);
-        }
 #pragma unroll
         for (int t = 0; t < 2 * NSW; ++t) {
-            const int s = wave + LT_WAVES * (t >> 1);
-            if (s < ns) {
-                const int dim = 32 * s + 16 * (t & 1) + col;
-                o[t] *= corr;
+            o[t] *= corr;
 #pragma unroll
-                for (int q = 0; q < 2; ++q) {
-                    bf16x8 v = *(const bf16x8*)(cols[q] + (size_t)dim * page_size);
-                    if (edge) {
-#pragma unroll
-                        for (int e = 0; e < 8; ++e)
-                            if (key0[q] + e > p || key0[q] + e < lo) v[e] = (bf16_t)0.f;
-                    }
-                    o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb[q], o[t], 0, 0, 0);
-                }
+            for (int q = 0; q < 2; ++q) {
+                bf16x8 v = vreg[t][q];
+                if (edge) v = keep_keys(v, key0[q], lo, p);
+                o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb[q], o[t], 0, 0, 0);
             }
         }
     }
@@ -648,16 +634,21 @@ __global__ __launch_bounds__(64 * LT_WAVES) void heads_matmul_mfma_kernel(
     const int t0 = (unit / j_parts) * 16, j_first = unit % j_parts, h = blockIdx.y;
     if (t0 >= n) return;
     const int col = lane & 15, g = lane >> 4;
-    const int ns = (K + 31) >> 5;                                   // (the last step of 32 may be short: 8, 16 or 24 values)
     const int token = t0 + col;
     const bool live = token < n;
     bf16x8 xreg[NS];
     {
-        const TX* xr = x + (size_t)(live ? token : t0) * ldx + (size_t)h * hx + 8 * g;
+        const TX* xr = x + (size_t)(live ? token : t0) * ldx + (size_t)h * hx;
 #pragma unroll
-        for (int s = 0; s < NS; ++s)
+        for (int s = 0; s < NS; ++s) {
+            const bool inside = 32 * s + 8 * g < K;
+            const TX* src = xr + (inside ? 32 * s + 8 * g : 0);        // (no branch around a load: what lies beyond K or n is set to zero afterwards)
+            TX v[8];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) xreg[s][e] = (32 * s + 8 * g < K && live) ? (bf16_t)to_f32(xr[32 * s + e]) : (bf16_t)0.f;
+            for (int e = 0; e < 8; ++e) v[e] = src[e];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) xreg[s][e] = inside && live ? (bf16_t)to_f32(v[e]) : (bf16_t)0.f;
+        }
     }
     const float gv = (gate && live) ? 1.0f / (1.0f + expf(-gate[(size_t)token * ldg + gate_col0 + h])) : 1.0f;
     const bf16_t* wh = w + (size_t)h * J * K;
@@ -667,7 +658,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void heads_matmul_mfma_kernel(
         const bf16_t* row = wh + (size_t)(16 * jt + col) * K + 8 * g;
 #pragma unroll
         for (int s = 0; s < NS; ++s)
-            if (s < ns) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(32 * s + 8 * g < K ? row + 32 * s : row - 8 * g), xreg[s], acc, 0, 0, 0);      // (beyond K: finite weights against zeros)
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(32 * s + 8 * g < K ? row + 32 * s : row - 8 * g), xreg[s], acc, 0, 0, 0);      // (beyond K: finite weights against zeros)
         if (live) {
             TOut* dst = out + ((size_t)token * H + h) * ho + 16 * jt + 4 * g;
 #pragma unroll
