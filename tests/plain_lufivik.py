@@ -52,7 +52,8 @@ def causal_convolution(h, w):
     y = np.zeros_like(h)
     for j in range(taps):
         back = taps - 1 - j
-        y[back:] += h[:h.shape[0] - back] * w[:, j] if back else h * w[:, j]
+        for i in range(back, h.shape[0]):
+            y[i] += h[i - back] * w[:, j]
     return y
 
 
