@@ -139,24 +139,28 @@ int fl_headnorm_gate(const float* x, const float* w, const float* gate, int ldg,
 // ---- routed experts, activations, re-entry of the stream (moe.hip) ----
 int fl_moe_route(const float* logits, int ld, int col0, int n, int E, int top, int kind, int renorm,
                  int* place, int* src_row, float* src_scale, float* pair_w, int* tiles, int max_tiles,
-                 hipStream_t stream);
+                 int tile_rows, hipStream_t stream);
 // the same for a router whose choice goes by softmax + correction inside the best groups of experts and whose last
 // n_identity outputs are identity experts (E counts all outputs); weights = chosen softmax / their sum * scale
 int fl_moe_route_grouped(const float* logits, int ld, int col0, int n, int E, int n_identity, int top,
                          const float* correction, int n_groups, int keep_groups, float scale, int* place,
                          int* src_row, float* src_scale, float* pair_w, int* tiles, int max_tiles,
-                         hipStream_t stream);
+                         int tile_rows, hipStream_t stream);
 // y[p] = src_scale[p] * x[src_row[p]] for the sorted places of identity experts' tiles
 int fl_moe_identity(const void* x, int dtype, const int* src_row, const float* src_scale, float* y,
                     const int* tiles, int max_tiles, int W, hipStream_t stream);
 int fl_moe_tile_rows(void);
 int fl_moe_gemm(const void* x, int dtype, const int* src_row, const float* src_scale, const void* w,
                 float* out, const int* tiles, int max_tiles, int N, int K, hipStream_t stream);
-// fl_moe_gemm on the matrix cores (bfloat16 x and w; moe_tuned.hip); n_rows: the sorted pairs of the step (few: the
-// form that only streams the weights)
-int fl_moe_gemm_mfma(const void* x, const int* src_row, const float* src_scale, const void* w, float* out,
-                     const int* tiles, int max_tiles, int n_rows, int N, int K, hipStream_t stream);
-int fl_moe_gemm_mfma_takes(int N, int K);
+// The experts' product on the matrix cores (bfloat16; moe_tuned.hip): out[p] = src_scale[p] * (x[src_row[p]] W_e^T), each
+// expert's matrix packed (kernels/packing.py), experts one after the other; tiles of tile_rows (64 or 128) rows; n_rows:
+// the sorted pairs of the step (few: the form that only streams the weights).  gate 0: out float [n_rows][N].  Else the
+// rows of W_e are gate and up rows interleaved in fours and out is bfloat16 [n_rows][N / 2]: 1 silu(gate) * up;
+// 2 g sigmoid(alpha g) (u + shift), g = min(gate, limit), u = clamp(up, -limit, limit)
+int fl_moe_packed(const void* x, const int* src_row, const float* src_scale, const void* w, void* out, const int* tiles,
+                  int max_tiles, int tile_rows, int n_rows, int N, int K, int gate, float alpha, float limit, float shift,
+                  hipStream_t stream);
+int fl_moe_packed_takes(int N, int K);
 // out[m][f] = sum_k x[m][k] w[f][k] for few features f: one wave per output, float sums in a fixed order
 int fl_gemm_few(const void* x, const void* w, float* out, int dtype, int M, int N, int K, hipStream_t stream);
 int fl_moe_combine(const float* y, const int* place, int top, const float* shared, const float* gate, int ldg,

@@ -13,7 +13,8 @@
 #include "api.h"
 #include "recordable.h"
 
-#define MOE_TILE 64           // rows of a tile of fl_moe_gemm
+#define MOE_TILE 64           // rows of a tile of fl_moe_gemm (the router cuts tiles of as many rows as it is asked for)
+#define MOE_MAX_TILE 128
 #define MOE_MAX_EXPERTS 1024
 #define MOE_MAX_TOP 16
 
@@ -201,7 +202,7 @@ __global__ __launch_bounds__(256) void moe_pick_grouped_kernel(const float* __re
 // products skip, and a 1 in the fourth place, which fl_moe_identity looks for.
 __global__ __launch_bounds__(1024) void moe_route_kernel(int n, int E, int E_real, int top, int* __restrict__ place,
                                                          int* __restrict__ src_row, float* __restrict__ src_scale,
-                                                         const float* __restrict__ pair_w, int* __restrict__ tiles, int max_tiles) {
+                                                         const float* __restrict__ pair_w, int* __restrict__ tiles, int max_tiles, int tile_rows) {
     __shared__ int count[MOE_MAX_EXPERTS];
     __shared__ int first[MOE_MAX_EXPERTS];
     for (int e = threadIdx.x; e < E; e += 1024) count[e] = 0;
@@ -212,10 +213,10 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(int n, int E, int E_rea
         int at = 0, tile = 0;
         for (int e = 0; e < E; ++e) {
             first[e] = at;
-            for (int r = 0; r < count[e] && tile < max_tiles; r += MOE_TILE, ++tile) {
+            for (int r = 0; r < count[e] && tile < max_tiles; r += tile_rows, ++tile) {
                 tiles[4 * tile + 0] = e < E_real ? e : -1;
                 tiles[4 * tile + 1] = at + r;
-                tiles[4 * tile + 2] = min(MOE_TILE, count[e] - r);
+                tiles[4 * tile + 2] = min(tile_rows, count[e] - r);
                 tiles[4 * tile + 3] = e < E_real ? 0 : 1;
             }
             at += count[e];
@@ -242,20 +243,21 @@ extern "C" int fl_moe_tile_rows(void) { return MOE_TILE; }
 
 extern "C" int fl_moe_route(const float* logits, int ld, int col0, int n, int E, int top, int kind, int renorm,
                             int* place, int* src_row, float* src_scale, float* pair_w, int* tiles, int max_tiles,
-                            hipStream_t stream) {
+                            int tile_rows, hipStream_t stream) {
+    FL_CHECK(tile_rows > 0 && tile_rows <= MOE_MAX_TILE, "moe_route: tiles of %d rows (at most %d)", tile_rows, MOE_MAX_TILE);
     FL_CHECK(n >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= MOE_MAX_TOP && top <= E,
              "moe_route: %d of %d experts (at most %d of %d)", top, E, MOE_MAX_TOP, MOE_MAX_EXPERTS);
     FL_CHECK(ld >= col0 + E && col0 >= 0, "moe_route: columns %d..%d of rows %d wide", col0, col0 + E, ld);
     {
-        const long pairs = (long)n * top;          // an expert's last tile may be short: pairs / 64 full tiles and one per expert at most
-        FL_CHECK((long)max_tiles >= pairs / MOE_TILE + (pairs < E ? pairs : E), "moe_route: %d tiles cannot hold %ld rows of %d experts", max_tiles, pairs, E);
+        const long pairs = (long)n * top;          // an expert's last tile may be short: pairs / tile_rows full tiles and one per expert at most
+        FL_CHECK((long)max_tiles >= pairs / tile_rows + (pairs < E ? pairs : E), "moe_route: %d tiles cannot hold %ld rows of %d experts", max_tiles, pairs, E);
     }
     FL_CHECK(kind >= 0 && kind <= 2, "moe_route: unknown scoring %d", kind);
     if (n == 0) return 0;
     const int pick_blocks = n < 4 * 1024 ? (n + 3) / 4 : 1024;
     moe_pick_kernel<<<pick_blocks, 256, 0, stream>>>(logits, ld, col0, n, E, top, kind, renorm, place, pair_w);
     FL_LAUNCH_CHECK();
-    moe_route_kernel<<<1, 1024, 0, stream>>>(n, E, E, top, place, src_row, src_scale, pair_w, tiles, max_tiles);
+    moe_route_kernel<<<1, 1024, 0, stream>>>(n, E, E, top, place, src_row, src_scale, pair_w, tiles, max_tiles, tile_rows);
     FL_LAUNCH_CHECK();
     return 0;
 }
@@ -266,7 +268,8 @@ FL_RECORDABLE(fl_moe_route)
 extern "C" int fl_moe_route_grouped(const float* logits, int ld, int col0, int n, int E, int n_identity, int top,
                                     const float* correction, int n_groups, int keep_groups, float scale, int* place,
                                     int* src_row, float* src_scale, float* pair_w, int* tiles, int max_tiles,
-                                    hipStream_t stream) {
+                                    int tile_rows, hipStream_t stream) {
+    FL_CHECK(tile_rows > 0 && tile_rows <= MOE_MAX_TILE, "moe_route_grouped: tiles of %d rows (at most %d)", tile_rows, MOE_MAX_TILE);
     FL_CHECK(n >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= MOE_MAX_TOP && top <= E,
              "moe_route_grouped: %d of %d experts (at most %d of %d)", top, E, MOE_MAX_TOP, MOE_MAX_EXPERTS);
     FL_CHECK(n_identity >= 0 && n_identity < E, "moe_route_grouped: %d identity experts among %d outputs", n_identity, E);
@@ -276,7 +279,7 @@ extern "C" int fl_moe_route_grouped(const float* logits, int ld, int col0, int n
     FL_CHECK(ld >= col0 + E && col0 >= 0, "moe_route_grouped: columns %d..%d of rows %d wide", col0, col0 + E, ld);
     {
         const long pairs = (long)n * top;
-        FL_CHECK((long)max_tiles >= pairs / MOE_TILE + (pairs < E ? pairs : E), "moe_route_grouped: %d tiles cannot hold %ld rows of %d experts", max_tiles, pairs, E);
+        FL_CHECK((long)max_tiles >= pairs / tile_rows + (pairs < E ? pairs : E), "moe_route_grouped: %d tiles cannot hold %ld rows of %d experts", max_tiles, pairs, E);
     }
     if (n == 0) return 0;
     const int pick_blocks = n < 4 * 1024 ? (n + 3) / 4 : 1024;
@@ -287,7 +290,7 @@ extern "C" int fl_moe_route_grouped(const float* logits, int ld, int col0, int n
     else FL_PICK(MOE_MAX_EXPERTS / 64);
 #undef FL_PICK
     FL_LAUNCH_CHECK();
-    moe_route_kernel<<<1, 1024, 0, stream>>>(n, E, E - n_identity, top, place, src_row, src_scale, pair_w, tiles, max_tiles);
+    moe_route_kernel<<<1, 1024, 0, stream>>>(n, E, E - n_identity, top, place, src_row, src_scale, pair_w, tiles, max_tiles, tile_rows);
     FL_LAUNCH_CHECK();
     return 0;
 }

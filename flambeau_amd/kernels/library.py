@@ -46,9 +46,9 @@ _SIGNATURES = {
     "fl_clamped_gate": [P, P, I, I, I, F, F, F, P],
     "fl_mlstm_scan": [P, I, I, I, I, I, I, P, P, F, F, P, P, P, P, P, P, I, I, I, I, P],
     "fl_headnorm_gate": [P, P, P, I, I, P, I, I, I, I, F, I, P],
-    "fl_moe_route": [P, I, I, I, I, I, I, I, P, P, P, P, P, I, P],
+    "fl_moe_route": [P, I, I, I, I, I, I, I, P, P, P, P, P, I, I, P],
     "fl_moe_gemm": [P, I, P, P, P, P, P, I, I, I, P],
-    "fl_moe_gemm_mfma": [P, P, P, P, P, P, I, I, I, I, P],
+    "fl_moe_packed": [P, P, P, P, P, P, I, I, I, I, I, I, F, F, F, P],
     "fl_gemm_few": [P, P, P, I, I, I, I, P],
     "fl_moe_combine": [P, P, I, P, P, I, I, P, I, I, P],
     "fl_activation": [P, P, I, L, I, P],
@@ -77,7 +77,7 @@ _SIGNATURES = {
     "fl_linear_scan_delta_channel": [P, I, P, I, P, I, P, I, P, I, P, L, P, P, P, P, I, I, I, I, I, P],
     "fl_channel_decay": [P, I, I, P, P, P, I, I, I, P],
     "fl_lowrank_expand": [P, I, I, P, P, I, P, I, I, I, P],
-    "fl_moe_route_grouped": [P, I, I, I, I, I, I, P, I, I, F, P, P, P, P, P, I, P],
+    "fl_moe_route_grouped": [P, I, I, I, I, I, I, P, I, I, F, P, P, P, P, P, I, I, P],
     "fl_moe_identity": [P, I, P, P, P, P, I, I, P],
     "fl_hyper_step": [P, I, I, I, P, P, P, P, P, P, I, P, P, F, P, I, P],
     "fl_hyper_spread": [P, P, I, I, I, P],

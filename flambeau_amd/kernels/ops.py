@@ -448,22 +448,23 @@ def moe_tile_rows() -> int:
     return load().fl_moe_tile_rows()
 
 
-def moe_max_tiles(n_pairs: int, n_experts: int) -> int:
+def moe_max_tiles(n_pairs: int, n_experts: int, tile_rows: int | None = None) -> int:
     """Upper bound of the row tiles of ``n_pairs`` (token, expert) pairs spread over ``n_experts``."""
-    return n_pairs // moe_tile_rows() + min(n_pairs, n_experts)
+    return n_pairs // (tile_rows or moe_tile_rows()) + min(n_pairs, n_experts)
 
 
 ROUTER_SCORINGS = {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2, "softmax_grouped": 3}     # (the last has a launch function of its own)
 
 
-def moe_route(logits, col0, n_experts, top, place, src_row, src_scale, pair_w, tiles, scoring="sigmoid", renormalise=False):
+def moe_route(logits, col0, n_experts, top, place, src_row, src_scale, pair_w, tiles, scoring="sigmoid", renormalise=False,
+              tile_rows: int | None = None):
     n, ld = logits.shape
     P_ = n * top
     call("fl_moe_route", _check(logits, "moe_route.logits", torch.float32), ld, int(col0), n, int(n_experts), int(top),
          ROUTER_SCORINGS[scoring], int(bool(renormalise)),
          _check(place, "moe_route.place", torch.int32, (P_,)), _check(src_row, "moe_route.src_row", torch.int32, (P_,)),
          _check(src_scale, "moe_route.src_scale", torch.float32, (P_,)), _check(pair_w, "moe_route.pair_w", torch.float32, (P_,)),
-         _check(tiles, "moe_route.tiles", torch.int32, (None, 4)), tiles.shape[0], stream_handle())
+         _check(tiles, "moe_route.tiles", torch.int32, (None, 4)), tiles.shape[0], int(tile_rows or moe_tile_rows()), stream_handle())
 
 
 def gemm_few(x, w, out):
@@ -475,21 +476,12 @@ def gemm_few(x, w, out):
     return out
 
 
-def moe_gemm(x, w, out, tiles, src_row=None, src_scale=None, matrix_cores=False):
-    """``out[p] = (src_scale[p] * x[src_row[p]]) @ w[e].T`` for the sorted places ``p`` of every tile, ``e`` the
-    tile's expert; ``w`` ``[E, N, K]``; without ``src_row`` the rows of ``x`` are the places themselves.
-    ``matrix_cores``: the bfloat16 kernel on the matrix cores where it takes the sizes."""
+def moe_gemm(x, w, out, tiles, src_row=None, src_scale=None):
+    """``out[p] = (src_scale[p] * x[src_row[p]]) @ w[e].T`` for the sorted places ``p`` of every tile (of at most
+    ``moe_tile_rows`` rows), ``e`` the tile's expert; ``w`` ``[E, N, K]``; without ``src_row`` the rows of ``x`` are the
+    places themselves."""
     E, N, K = w.shape
     P_ = out.shape[0]
-    if matrix_cores and w.dtype == torch.bfloat16:
-        from .library import load
-        if load().fl_moe_gemm_mfma_takes(N, K):
-            call("fl_moe_gemm_mfma", _check(x, "moe_gemm.x", w.dtype, (None, K)),
-                 _check(src_row, "moe_gemm.src_row", torch.int32, (P_,)) if src_row is not None else None,
-                 _check(src_scale, "moe_gemm.src_scale", torch.float32, (P_,)) if src_scale is not None else None,
-                 _check(w, "moe_gemm.w"), _check(out, "moe_gemm.out", torch.float32, (P_, N)),
-                 _check(tiles, "moe_gemm.tiles", torch.int32, (None, 4)), tiles.shape[0], P_, N, K, stream_handle())
-            return out
     call("fl_moe_gemm", _check(x, "moe_gemm.x", w.dtype, (None, K)), dtype_code(w.dtype),
          _check(src_row, "moe_gemm.src_row", torch.int32, (P_,)) if src_row is not None else None,
          _check(src_scale, "moe_gemm.src_scale", torch.float32, (P_,)) if src_scale is not None else None,
@@ -866,7 +858,7 @@ def lowrank_expand(x, col, w, wt, out):
 
 
 def moe_route_grouped(logits, col0, n_outputs, n_identity, top, correction, n_groups, keep_groups, scale, place, src_row, src_scale,
-                      pair_w, tiles):
+                      pair_w, tiles, tile_rows: int | None = None):
     """``moe_route`` for a router that scores by a softmax over all its ``n_outputs`` outputs (the last ``n_identity`` of
     them identity experts), chooses by score + ``correction`` inside the ``keep_groups`` best of ``n_groups`` groups of
     neighbours, and weights the chosen by their scores over their sum, times ``scale``."""
@@ -877,7 +869,7 @@ def moe_route_grouped(logits, col0, n_outputs, n_identity, top, correction, n_gr
          int(n_groups), int(keep_groups), float(scale),
          _check(place, "moe_route.place", torch.int32, (P_,)), _check(src_row, "moe_route.src_row", torch.int32, (P_,)),
          _check(src_scale, "moe_route.src_scale", torch.float32, (P_,)), _check(pair_w, "moe_route.pair_w", torch.float32, (P_,)),
-         _check(tiles, "moe_route.tiles", torch.int32, (None, 4)), tiles.shape[0], stream_handle())
+         _check(tiles, "moe_route.tiles", torch.int32, (None, 4)), tiles.shape[0], int(tile_rows or moe_tile_rows()), stream_handle())
 
 
 def moe_identity(x, src_row, src_scale, y, tiles):

@@ -10,13 +10,15 @@ The choice never leaves the device: a kernel sorts the (token, expert) pairs by 
 into row tiles, the two products of all experts run as one launch each over those tiles, and a last
 kernel adds each token's experts in rising order of rank.  The router's product is a kernel of its own
 (one wave per score: exact products, float sums in a fixed order), whatever the runtime's other products
-are; the experts' products run on the matrix cores in bfloat16 and as plain products in 32-bit.
+are; the experts' products are a kernel set (``kernels/experts.py``): on the matrix cores in bfloat16, plain products
+in 32-bit.
 """
 from __future__ import annotations
 
 import torch
 
 from ..kernels import ops
+from ..kernels.experts import ExpertActivation
 from .base import FEED_FORWARDS, ExpertRows, FeedForward, Product, TensorSpec
 
 
@@ -103,8 +105,8 @@ class RoutedExperts(FeedForward):
             raise ValueError("routed_experts: a gate with a factor or a shift comes with a limit")
         if gate_limit is not None and (not gated or not gate_limit > 0.0):
             raise ValueError(f"routed_experts: a limit of {gate_limit} on the halves of an expert's gate (gated experts only, above 0)")
-        self.gate_limit, self.gate_alpha, self.up_shift = gate_limit, float(gate_alpha), float(up_shift)
-        self.gated, self.activation, self.router_bias = bool(gated), activation, bool(router_bias)
+        self.between = ExpertActivation(bool(gated), activation, gate_limit, float(gate_alpha), float(up_shift))
+        self.gated, self.router_bias = bool(gated), bool(router_bias)
         self.hidden_size, self.n_experts, self.top = hidden_size, n_experts, top
         self.expert_size, self.shared_size = expert_size, shared_size
         self.scoring, self.renormalise, self.weight_on = scoring, bool(renormalise), weight_on
@@ -136,13 +138,14 @@ class RoutedExperts(FeedForward):
         # the router's rows and, behind them, the shared expert's gate: one plain product gives all logits
         rows = [weights["router.weight"]] + ([weights["shared.sg.weight"]] if self.shared_gate else [])
         self.w_logits = torch.cat(rows, dim=0).contiguous()
-        first = (lambda e: torch.cat([weights[f"e{e}.gate.weight"], weights[f"e{e}.up.weight"]], dim=0)) if self.gated else (lambda e: weights[f"e{e}.up.weight"])
-        self.w_gate_up = torch.stack([first(e) for e in range(E)]).contiguous()       # (ungated experts: the up matrices alone)
+        self.kernels = rt.kernels("routed_experts")
+        each = lambda k: [weights[f"e{e}.{k}.weight"] for e in range(E)]
+        self.w_first = self.kernels.prepare(each("up"), each("gate") if self.gated else None)       # (ungated experts: the up matrices alone)
         self.b_logits = None
         if self.router_bias:
             extra = self.w_logits.shape[0] - E
             self.b_logits = torch.cat([weights["router.bias"], torch.zeros(extra, dtype=torch.float32, device=weights["router.bias"].device)]).contiguous()
-        self.w_down = torch.stack([weights[f"e{e}.down.weight"] for e in range(E)]).contiguous()
+        self.w_down = self.kernels.prepare(each("down"))
         self.correction_w = weights.get("correction")
         if self.shared_size is not None:
             self.ws_gate_up = rt.prepare_gate_up(weights["shared.gate.weight"], weights["shared.up.weight"])
@@ -162,25 +165,18 @@ class RoutedExperts(FeedForward):
         src_row = ints("moe_src_row", pairs, 1, most).view(-1)
         src_scale = rt.buffer("moe_src_scale", pairs, 1, torch.float32, max_rows=most).view(-1)
         pair_w = rt.buffer("moe_pair_w", pairs, 1, torch.float32, max_rows=most).view(-1)
-        n_tiles = ops.moe_max_tiles(pairs, self.n_outputs)
-        tiles = ints("moe_tiles", n_tiles, 4, ops.moe_max_tiles(most, self.n_outputs))
+        tile_rows = self.kernels.tile_rows(pairs, E, self.w_first, self.w_down)
+        tiles = ints("moe_tiles", ops.moe_max_tiles(pairs, self.n_outputs, tile_rows), 4, ops.moe_max_tiles(most, self.n_outputs))
         if self.grouped:
             ops.moe_route_grouped(logits, 0, self.n_outputs, self.n_identity, top, self.correction_w, self.n_groups, self.keep_groups,
-                                  self.weight_scale, place, src_row, src_scale, pair_w, tiles)
+                                  self.weight_scale, place, src_row, src_scale, pair_w, tiles, tile_rows=tile_rows)
         else:
-            ops.moe_route(logits, 0, E, top, place, src_row, src_scale, pair_w, tiles, self.scoring, self.renormalise)
+            ops.moe_route(logits, 0, E, top, place, src_row, src_scale, pair_w, tiles, self.scoring, self.renormalise, tile_rows=tile_rows)
         on_input = self.weight_on == "input"
-        gate_up = rt.buffer("moe_gate_up", pairs, (2 if self.gated else 1) * F, torch.float32, max_rows=most)
-        ops.moe_gemm(x, self.w_gate_up, gate_up, tiles, src_row, src_scale if on_input else None, matrix_cores=rt.tuned)
         act = rt.buffer("moe_act", pairs, F, max_rows=most)
-        if self.gate_limit is not None:
-            ops.clamped_gate(gate_up, act, self.gate_alpha, self.gate_limit, self.up_shift)
-        elif self.gated:
-            ops.silu_mul(gate_up, act)
-        else:
-            ops.activation(gate_up, act, self.activation)
+        self.kernels.first(x, self.w_first, self.between, act, tiles, tile_rows, most, src_row, src_scale if on_input else None)
         y = rt.buffer("moe_y", pairs, W, torch.float32, max_rows=most)
-        ops.moe_gemm(act, self.w_down, y, tiles, None, None if on_input else src_scale, matrix_cores=rt.tuned)
+        self.kernels.product(act, self.w_down, y, tiles, tile_rows, None, None if on_input else src_scale)
         if self.n_identity:
             ops.moe_identity(x, src_row, src_scale, y, tiles)          # (the rows of identity experts: weight * input)
         if self.leave_rows and self.shared_size is None:
