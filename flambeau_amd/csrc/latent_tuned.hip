@@ -389,6 +389,194 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
         if (t < 2 * ns) *(f32x4*)(zr + 16 * t + 4 * g) = o[t] * inv;
 }
 
+// The same tiles for latents of 128, 256 or 512 values, eight waves to a block.  No wave holds a whole head: for the
+// scores of a chunk of 64 keys the waves deal out the keys (four runs of 16) and the steps of 32 values (two halves),
+// for the weighted sum the latent's dims, so that every row and every value of a chunk is read from memory by exactly
+// one wave of the block, straight into the registers it multiplies from (the values of a chunk are asked for before its
+// scores are formed, the rows of the next chunk before this one's are weighted).  What the waves share lies in LDS: the
+// folded queries of the tile's 64 (token, head) rows for the whole walk, the halves' scores, and the weights.
+//
+// Softmax: eight neighbouring threads take a row, eight keys each; a row's maximum and sum live in their registers.
+// The base of the exponents follows the maximum lazily, as in the kernel above; where it moved, all waves rescale.
+#define LS_S 68               // floats per row of scores (64 and four, so that rows start in different banks)
+#define LS_P 72               // values per row of weights
+// a barrier that waits for this wave's LDS accesses and not for its loads in flight
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+template <int NKH, int NDT>
+__global__ __launch_bounds__(512, 2) void latent_attention_spread_kernel(
+    const bf16_t* __restrict__ qa, float* __restrict__ z, const bf16_t* __restrict__ pool,
+    const int* __restrict__ positions, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
+    int max_blocks, int H, int K, int R, int page_size, int n_pages, float scale, int window, const int* __restrict__ tiles) {
+    constexpr int QS = NKH * 64 + 8;
+    extern __shared__ __attribute__((aligned(16))) unsigned char lt_smem[];
+    bf16_t* qs = (bf16_t*)lt_smem;                                  // [64 rows][QS]
+    float* ss = (float*)(qs + 64 * QS);                             // [2 halves][64 rows][LS_S]
+    bf16_t* ps = (bf16_t*)(ss + 2 * 64 * LS_S);                     // [64 rows][LS_P]
+    float* rs = (float*)(ps + 64 * LS_P);                           // [64 rows]: factor of a chunk, at the end 1 / sum
+    int* moved_at = (int*)(rs + 64);                                // the chunk in which some row's base moved last
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const int col = lane & 15, g = lane >> 4;
+    const int half = wave >> 2, kt = wave & 3;
+    const int tile = gridDim.x - 1 - blockIdx.x;                    // (a prompt's last tokens see the most keys: first)
+    const int t_first = tiles[4 * tile], n_tok = tiles[4 * tile + 1], g_first = tiles[4 * tile + 2], n_grp = tiles[4 * tile + 3];
+    const int nk = K >> 5;
+    const int p_max = positions[t_first + n_tok - 1];
+    const int* table = block_table + (size_t)tok_seq[t_first] * max_blocks;
+    const int lo_min = window > 0 ? max(0, positions[t_first] - window + 1) : 0;
+    const size_t page_stride = (size_t)page_size * (K + R);
+
+    // this thread's row in the softmax (and in filling the queries): unit row / 16 = (token, group of 16 heads)
+    const int row = tid >> 3, kk = tid & 7;
+    const int unit = row >> 4, tw = unit / n_grp, head = (g_first + unit - tw * n_grp) * 16 + (row & 15);
+    const bool live = tw < n_tok && head < H;
+    const int p = live ? positions[t_first + tw] : -1;
+    const int lo = window > 0 ? max(0, p - window + 1) : 0;
+    {
+        const bf16_t* qr = qa + ((size_t)(t_first + (live ? tw : 0)) * H + (live ? head : 0)) * K;
+        const bf16x8 zero = {(bf16_t)0.f, (bf16_t)0.f, (bf16_t)0.f, (bf16_t)0.f, (bf16_t)0.f, (bf16_t)0.f, (bf16_t)0.f, (bf16_t)0.f};
+        for (int c = kk; c < NKH * 8; c += 8) {
+            const bool inside = live && 8 * c < K;
+            const bf16x8 v = *(const bf16x8*)(qr + (inside ? 8 * c : 0));
+            *(bf16x8*)(qs + row * QS + 8 * c) = inside ? v : zero;
+        }
+        if (tid == 0) *moved_at = -1;
+    }
+    auto page_of = [&](int key) {                                   // (a run beyond the newest token: that token's page, masked below)
+        const int page = table[min(key, p_max & ~15) / page_size];
+        return pool + (size_t)min(max(page, 0), n_pages - 1) * page_stride;
+    };
+    bf16x8 kreg[NKH], vreg[NDT][2];
+    auto load_keys = [&](int t0) {
+        const int key = t0 + 16 * kt;
+        const bf16_t* src = page_of(key) + (size_t)(min(key, p_max & ~15) % page_size + col) * K + 8 * g;
+#pragma unroll
+        for (int i = 0; i < NKH; ++i) {
+            const int st = half * NKH + i;
+            kreg[i] = *(const bf16x8*)(src + (st < nk ? 32 * st : 0));
+        }
+    };
+    auto load_values = [&](int t0) {
+#pragma unroll
+        for (int q = 0; q < 2; ++q) {
+            const int run = t0 + 32 * q + 16 * (g >> 1);
+            const bf16_t* src = page_of(run) + (size_t)page_size * K + min(run, p_max & ~15) % page_size + 8 * (g & 1);
+#pragma unroll
+            for (int d = 0; d < NDT; ++d) vreg[d][q] = *(const bf16x8*)(src + (size_t)(16 * (NDT * wave + d) + col) * page_size);
+        }
+    };
+    f32x4 o[NDT][4];                                                // dims 16 (NDT wave + d) + 4 g + r of row 16 u + col
+#pragma unroll
+    for (int d = 0; d < NDT; ++d)
+#pragma unroll
+        for (int u = 0; u < 4; ++u) o[d][u] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    float m = -INFINITY, l = 0.f;
+    const int t_begin = lo_min & ~(LT_CHUNK - 1);
+    load_keys(t_begin);
+    __syncthreads();                                                // the queries are in place
+    for (int t0 = t_begin; t0 <= p_max; t0 += LT_CHUNK) {
+        load_values(t0);
+        f32x4 sacc[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) sacc[u] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < NKH; ++i)
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+                sacc[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[i], *(const bf16x8*)(qs + (16 * u + col) * QS + (half * NKH + i) * 32 + 8 * g), sacc[u], 0, 0, 0);
+        // lane (row col, g): keys 16 kt + 4 g .. + 3
+#pragma unroll
+        for (int u = 0; u < 4; ++u) *(f32x4*)(ss + (half * 64 + 16 * u + col) * LS_S + 16 * kt + 4 * g) = sacc[u];
+        if (t0 + LT_CHUNK <= p_max) load_keys(t0 + LT_CHUNK);
+        lds_barrier();
+        {
+            float sv[8], cmax = -INFINITY;
+#pragma unroll
+            for (int h4 = 0; h4 < 2; ++h4) {
+                const f32x4 a = *(const f32x4*)(ss + row * LS_S + 8 * kk + 4 * h4), b = *(const f32x4*)(ss + (64 + row) * LS_S + 8 * kk + 4 * h4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int key = t0 + 8 * kk + 4 * h4 + e;
+                    sv[4 * h4 + e] = key > p || key < lo ? -INFINITY : (a[e] + b[e]) * scale;
+                    cmax = fmaxf(cmax, sv[4 * h4 + e]);
+                }
+            }
+            cmax = fmaxf(cmax, __shfl_xor(cmax, 1, FL_WAVE));
+            cmax = fmaxf(cmax, __shfl_xor(cmax, 2, FL_WAVE));
+            cmax = fmaxf(cmax, __shfl_xor(cmax, 4, FL_WAVE));
+            const float m_new = cmax > m + 8.0f ? cmax : m;         // minus infinity while the row has seen no key
+            const float base = m_new == -INFINITY ? 0.f : m_new;
+            const float corr = expf(m - base);
+            bf16x8 w;
+            float lsum = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                w[e] = (bf16_t)expf(sv[e] - base);
+                lsum += (float)w[e];                                // the sum of the weights as they are multiplied
+            }
+            lsum += __shfl_xor(lsum, 1, FL_WAVE);
+            lsum += __shfl_xor(lsum, 2, FL_WAVE);
+            lsum += __shfl_xor(lsum, 4, FL_WAVE);
+            l = l * corr + lsum;
+            *(bf16x8*)(ps + row * LS_P + 8 * kk) = w;
+            if (kk == 0) rs[row] = corr;
+            if (m_new != m) *moved_at = t0;
+            m = m_new;
+        }
+        lds_barrier();
+        if (*moved_at == t0) {
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const float corr = rs[16 * u + col];
+#pragma unroll
+                for (int d = 0; d < NDT; ++d) o[d][u] *= corr;
+            }
+        }
+        const bool edge = t0 + LT_CHUNK - 1 > p_max || t0 < lo_min;
+#pragma unroll
+        for (int q = 0; q < 2; ++q) {
+            bf16x8 pb[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) pb[u] = *(const bf16x8*)(ps + (16 * u + col) * LS_P + 32 * q + 8 * g);
+#pragma unroll
+            for (int d = 0; d < NDT; ++d) {
+                bf16x8 v = vreg[d][q];
+                if (edge) v = keep_keys(v, t0 + 32 * q + 8 * g, lo_min, p_max);          // (what no row of the tile sees is zero, whatever the page holds)
+#pragma unroll
+                for (int u = 0; u < 4; ++u) o[d][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pb[u], o[d][u], 0, 0, 0);
+            }
+        }
+    }
+    __syncthreads();
+    if (kk == 0) rs[row] = l > 0.f ? 1.0f / l : 0.f;
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+        const int tu = u / n_grp, hu = (g_first + u - tu * n_grp) * 16 + col;
+        if (tu >= n_tok || hu >= H) continue;
+        const float inv = rs[16 * u + col];
+        float* zr = z + ((size_t)(t_first + tu) * H + hu) * R;
+#pragma unroll
+        for (int d = 0; d < NDT; ++d) *(f32x4*)(zr + 16 * (NDT * wave + d) + 4 * g) = o[d][u] * inv;
+    }
+}
+
+template <int NKH, int NDT>
+static int launch_spread(const void* qa, float* z, const void* pool, const int* positions, const int* tok_seq, const int* block_table,
+                         int max_blocks, int H, int K, int R, int page_size, int n_pages, float scale, int window, const int* tiles,
+                         int n_tiles, hipStream_t stream) {
+    constexpr int LDS = 64 * (NKH * 64 + 8) * 2 + 2 * 64 * LS_S * 4 + 64 * LS_P * 2 + 64 * 4 + 16;
+    static bool sized = false;
+    if (!sized) {
+        hipError_t e_ = hipFuncSetAttribute((const void*)latent_attention_spread_kernel<NKH, NDT>, hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
+        FL_CHECK(e_ == hipSuccess, "latent_attention_spread: %s", hipGetErrorString(e_));
+        sized = true;
+    }
+    latent_attention_spread_kernel<NKH, NDT><<<n_tiles, 512, LDS, stream>>>((const bf16_t*)qa, z, (const bf16_t*)pool, positions, tok_seq, block_table,
+                                                                            max_blocks, H, K, R, page_size, n_pages, scale, window, tiles);
+    return 0;
+}
+
 extern "C" long fl_latent_attention_shared_lds(int K, int R) { return (long)LT_CHUNK * (K + 8) * 2 + (long)R * (LT_CHUNK + 8) * 2; }
 
 // tiles [n_tiles][4] = (first token, tokens, first group of 16 heads, groups): tokens x groups <= 4, the tokens of one request
@@ -401,6 +589,14 @@ extern "C" int fl_latent_attention_shared(const void* qa, float* z, const void* 
     FL_CHECK((uintptr_t)qa % 16 == 0 && (uintptr_t)pool % 16 == 0 && (uintptr_t)z % 16 == 0, "latent_attention_shared: operands must be 16-byte aligned");
     FL_CHECK(window >= 0, "latent_attention_shared: negative window");
     if (n_tiles == 0) return 0;
+    if (R == 128 || R == 256 || R == 512) {
+#define FL_LSP(NKH, NDT) launch_spread<NKH, NDT>(qa, z, pool, positions, tok_seq, block_table, max_blocks, H, K, R, page_size, n_pages, scale, window, tiles, n_tiles, stream)
+        const int rc = R == 128 ? (K == R ? FL_LSP(2, 1) : FL_LSP(3, 1)) : R == 256 ? (K == R ? FL_LSP(4, 2) : FL_LSP(5, 2)) : K == R ? FL_LSP(8, 4) : FL_LSP(9, 4);
+#undef FL_LSP
+        if (rc != 0) return rc;
+        FL_LAUNCH_CHECK();
+        return 0;
+    }
     const size_t lds = (size_t)fl_latent_attention_shared_lds(K, R);
     const int ns = R / 32;
 #define FL_LTS(NK, NS)                                                                                                     \

@@ -430,7 +430,8 @@ def test_keys_dealt_out_to_several_waves(splits, H, R):
     assert (one - plain).abs().max().item() < 2e-2 * plain.abs().max().item()
 
 
-@pytest.mark.parametrize("H,R,ps", [(20, 96, 16), (32, 64, 32), (7, 512, 16), (40, 32, 16), (70, 160, 64)])
+@pytest.mark.parametrize("H,R,ps", [(20, 96, 16), (32, 64, 32), (7, 512, 16), (40, 32, 16), (70, 160, 64), (20, 128, 16), (32, 256, 32), (70, 512, 16),
+                                    (16, 256, 16), (64, 128, 64)])
 def test_blocks_that_share_their_keys(H, R, ps):
     """The matrix-core kernel whose four waves read every chunk of keys from LDS against the one whose waves
     fetch for themselves: portions of unequal requests (some start mid-context, one is a single token, one

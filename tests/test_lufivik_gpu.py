@@ -193,6 +193,7 @@ SHAPES = [
     # sizes that the matrix-core kernels take, all three or some of them
     (20, 32, 32, 48, 24, 96, 64, 100.0, None), (4, 64, 16, 16, 40, 160, 33, 5000.0, None), (16, 8, 64, 32, 8, 32, 100, 70.0, None),
     (2, 96, 24, 16, 16, 512, 40, 10000.0, None), (40, 40, 34, 16, 24, 256, 90, 10000.0, 18),
+    (40, 64, 32, 32, 24, 128, 70, 300.0, None), (36, 32, 64, 16, 24, 512, 100, 2000.0, None),
     (3, 24, 70, 16, 16, 64, 50, 300.0, None),          # a rotated part wider than they take beside the latent
 ]
 
@@ -216,6 +217,50 @@ def test_latent_attention_with_a_rotated_part_alone(dtype, H, D, Dr, Dv, Rq, R, 
     for cuts in ([n], [60, 5, 1, 1, 2, 30, 2, 6, 1, 42], [1] * 90 + [60]):
         got = run_mixer(mixer, rt, x, cuts, page_size=16 if H > 3 else 8)
         assert np.abs(got - want).max() < TOL[dtype] * np.abs(want).max(), cuts
+
+
+@pytest.mark.parametrize("H,R,rot,ps", [(20, 128, 32, 16), (5, 128, 64, 32), (32, 256, 64, 16), (64, 256, 0, 32), (70, 512, 64, 16), (16, 512, 32, 64), (33, 512, 0, 16),
+                                        (20, 96, 64, 16), (17, 192, 32, 16)])
+@pytest.mark.parametrize("window", [0, 1, 40, 64, 131])
+def test_the_prompt_kernels_of_latent_attention(H, R, rot, ps, window):
+    """The matrix-core kernels whose blocks share their keys against the float kernel: unequal requests, one of a single
+    token, some that start mid-context, one that ends at a page's border; every row that no query sees, in pages beyond
+    the newest token and behind the window alike, holds NaN; one (query, key) score per request stands out."""
+    from flambeau_amd.cache.storage import CacheStorage
+    from flambeau_amd.kernels import latent_attention as la
+    from flambeau_amd.kernels import ops
+    from flambeau_amd.parts import PagedRowSpec
+    n_pages, K = -(-1600 // ps), R + rot
+    store = CacheStorage([PagedRowSpec(K, window, R)], [None], torch.device(DEV), torch.bfloat16, n_pages=n_pages, page_size=ps, max_slots=4)
+    pool = store.pools[0][0]                                                # [pages, ps * (K + R)]
+    g = torch.Generator().manual_seed(H + R)
+    seqs = [(0, 150), (300, 7), (63, 1), (122, 70)]
+    step = make_step(seqs, ps, n_pages)
+    pool.fill_(float("nan"))
+    for s, (st, q) in enumerate(seqs):
+        for j in range(max(0, st - window + 1) if window else 0, st + q):
+            page, r = int(step.block_tables[0][s, j // ps]), j % ps
+            v = torch.randn(K, generator=g).to(torch.bfloat16).to(DEV) * 0.7
+            pool[page, r * K:(r + 1) * K] = v
+            pool[page, ps * K:].view(R, ps)[:, r] = v[:R]
+    n = step.n_tokens
+    qa = (torch.randn(n, H, K, generator=g) * 0.4).to(torch.bfloat16).to(DEV)
+    at = 0
+    for s, (st, q) in enumerate(seqs):                                      # the request's last query points at the oldest key it sees
+        key = max(0, st + q - 1 - (window or 10 ** 6) + 1)
+        page, r = int(step.block_tables[0][s, key // ps]), key % ps
+        qa[at + q - 1] = pool[page, r * K:(r + 1) * K]
+        at += q
+    qa = qa.view(n, H * K).contiguous()
+    cache = store.entries[0].kv
+    args = (cache, step.positions, step.tok_seq, step.block_tables[0], H, 0.25, window)
+    want = ops.latent_attention(qa.float(), torch.empty(n, H * R, device=DEV), *args)
+    tiles = torch.tensor(la.shared_tiles(step.host, -(-H // 16)), dtype=torch.int32, device=DEV)
+    got = la.latent_attention_shared(qa, torch.full((n, H * R), float("nan"), device=DEV), *args, tiles)
+    assert torch.isfinite(want).all() and torch.isfinite(got).all()
+    assert (got - want).abs().max().item() < 1e-2 * want.abs().max().item()
+    dealt = la.latent_attention_mfma(qa, torch.full((n, H * R), float("nan"), device=DEV), *args, dealt=True)
+    assert (dealt - want).abs().max().item() < 1e-2 * want.abs().max().item()
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
