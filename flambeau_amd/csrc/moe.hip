@@ -23,14 +23,13 @@
 // weights are divided by their sum (kind 2 always).
 // place [n * top]: where pair (t, k) lies in the sorted order; src_row / src_scale [n * top]: token and weight
 // of every sorted place; tiles [max_tiles][4] = (expert, first place, places, 0), expert -1: unused.
-__global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__ logits, int ld, int col0, int n, int E,
-                                                       int top, int kind, int renorm, int* __restrict__ place,
-                                                       float* __restrict__ pair_w) {
+__device__ __forceinline__ void moe_picks(const float* __restrict__ logits, int ld, int col0, int n, int E, int top, int kind,
+                                          int renorm, int* place, float* pair_w, int first, int stride) {
     // a wave per token: the lanes hold the token's logits (lane, lane + 64, ...), and every rank is a best-of-wave
     // (the larger logit, the lower index among equals)
     const int lane = threadIdx.x & 63;
     const int nu = (E + 63) >> 6;
-    for (int t = blockIdx.x * 4 + (threadIdx.x >> 6); t < n; t += gridDim.x * 4) {
+    for (int t = first; t < n; t += stride) {
         const float* z = logits + (size_t)t * ld + col0;
         float zv[MOE_MAX_EXPERTS / 64];
 #pragma unroll
@@ -83,6 +82,12 @@ __global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__
             }
         }
     }
+}
+
+__global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__ logits, int ld, int col0, int n, int E,
+                                                       int top, int kind, int renorm, int* __restrict__ place,
+                                                       float* __restrict__ pair_w) {
+    moe_picks(logits, ld, col0, n, E, top, kind, renorm, place, pair_w, blockIdx.x * 4 + (threadIdx.x >> 6), gridDim.x * 4);
 }
 
 // The picks of a router whose choice and weights differ: s = softmax(z) over all E outputs; the choice goes by
@@ -200,9 +205,9 @@ __global__ __launch_bounds__(256) void moe_pick_grouped_kernel(const float* __re
 // The (token, expert) pairs that moe_pick_kernel left (place[pair] = expert) counted, sorted by expert and cut into tiles.
 // Outputs E_real .. E - 1 of the router are identity experts (no matrices): their tiles carry expert -1, which the
 // products skip, and a 1 in the fourth place, which fl_moe_identity looks for.
-__global__ __launch_bounds__(1024) void moe_route_kernel(int n, int E, int E_real, int top, int* __restrict__ place,
-                                                         int* __restrict__ src_row, float* __restrict__ src_scale,
-                                                         const float* __restrict__ pair_w, int* __restrict__ tiles, int max_tiles, int tile_rows) {
+__device__ __forceinline__ void moe_sort_pairs(int n, int E, int E_real, int top, int* place, int* __restrict__ src_row,
+                                               float* __restrict__ src_scale, const float* pair_w,
+                                               int* __restrict__ tiles, int max_tiles, int tile_rows) {
     __shared__ int count[MOE_MAX_EXPERTS];
     __shared__ int first[MOE_MAX_EXPERTS];
     for (int e = threadIdx.x; e < E; e += 1024) count[e] = 0;
@@ -239,6 +244,24 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(int n, int E, int E_rea
     }
 }
 
+__global__ __launch_bounds__(1024) void moe_route_kernel(int n, int E, int E_real, int top, int* __restrict__ place,
+                                                         int* __restrict__ src_row, float* __restrict__ src_scale,
+                                                         const float* __restrict__ pair_w, int* __restrict__ tiles, int max_tiles, int tile_rows) {
+    moe_sort_pairs(n, E, E_real, top, place, src_row, src_scale, pair_w, tiles, max_tiles, tile_rows);
+}
+
+#define MOE_FEW_TOKENS 32
+// both at once, for steps of few tokens: the one block's 16 waves pick, then it sorts
+__global__ __launch_bounds__(1024) void moe_pick_route_kernel(const float* __restrict__ logits, int ld, int col0, int n, int E,
+                                                              int top, int kind, int renorm, int* place, int* __restrict__ src_row,
+                                                              float* __restrict__ src_scale, float* pair_w, int* __restrict__ tiles,
+                                                              int max_tiles, int tile_rows) {
+    moe_picks(logits, ld, col0, n, E, top, kind, renorm, place, pair_w, threadIdx.x >> 6, 16);
+    __threadfence_block();
+    __syncthreads();
+    moe_sort_pairs(n, E, E, top, place, src_row, src_scale, pair_w, tiles, max_tiles, tile_rows);
+}
+
 extern "C" int fl_moe_tile_rows(void) { return MOE_TILE; }
 
 extern "C" int fl_moe_route(const float* logits, int ld, int col0, int n, int E, int top, int kind, int renorm,
@@ -254,6 +277,11 @@ extern "C" int fl_moe_route(const float* logits, int ld, int col0, int n, int E,
     }
     FL_CHECK(kind >= 0 && kind <= 2, "moe_route: unknown scoring %d", kind);
     if (n == 0) return 0;
+    if (n <= MOE_FEW_TOKENS) {
+        moe_pick_route_kernel<<<1, 1024, 0, stream>>>(logits, ld, col0, n, E, top, kind, renorm, place, src_row, src_scale, pair_w, tiles, max_tiles, tile_rows);
+        FL_LAUNCH_CHECK();
+        return 0;
+    }
     const int pick_blocks = n < 4 * 1024 ? (n + 3) / 4 : 1024;
     moe_pick_kernel<<<pick_blocks, 256, 0, stream>>>(logits, ld, col0, n, E, top, kind, renorm, place, pair_w);
     FL_LAUNCH_CHECK();

@@ -256,43 +256,61 @@ FL_RECORDABLE(fl_moe_packed)
 
 // ------------------------------------------------------------------ a product with few output features
 // out[m][f] = sum_k x[m][k] w[f][k] for a handful of features (a router's scores, a gate's logit): one
-// wave per output element, the lanes stride over k and add their parts in a fixed tree, so an element
-// does not depend on how many rows the call has.  Products of stored values are exact in float; the
-// sums are float.
-template <typename T>
+// wave per row and FF neighbouring features (many rows: four, so that a row is read less often; few: one), the lanes
+// stride over k and add their parts in a fixed tree, so an element does not depend on how many rows the call
+// has.  Products of stored values are exact in float; the sums are float.
+template <typename T, int FF>
 __global__ __launch_bounds__(256) void gemm_few_kernel(const T* __restrict__ x, const T* __restrict__ w, float* __restrict__ out,
                                                        long total, int N, int K) {
     const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (unit >= total) return;
     const int lane = threadIdx.x & 63;
-    const long m = unit / N;
-    const int f = (int)(unit - m * N);
+    const int per_row = (N + FF - 1) / FF;
+    const long m = unit / per_row;
+    const int f = (int)(unit - m * per_row) * FF;
     const T* xr = x + (size_t)m * K;
-    const T* wr = w + (size_t)f * K;
-    float a0 = 0.f, a1 = 0.f, a2 = 0.f, a3 = 0.f;
+    const T* wr[FF];
+#pragma unroll
+    for (int q = 0; q < FF; ++q) wr[q] = w + (size_t)min(f + q, N - 1) * K;
+    float a[FF][4];
+#pragma unroll
+    for (int q = 0; q < FF; ++q)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) a[q][r] = 0.f;
     int k = 4 * lane;
     if (K % 4 == 0) {
         for (; k + 3 < K; k += 256) {
-            a0 = fmaf(to_f32(xr[k]), to_f32(wr[k]), a0);
-            a1 = fmaf(to_f32(xr[k + 1]), to_f32(wr[k + 1]), a1);
-            a2 = fmaf(to_f32(xr[k + 2]), to_f32(wr[k + 2]), a2);
-            a3 = fmaf(to_f32(xr[k + 3]), to_f32(wr[k + 3]), a3);
+            float xv[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) xv[r] = to_f32(xr[k + r]);
+#pragma unroll
+            for (int q = 0; q < FF; ++q)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) a[q][r] = fmaf(xv[r], to_f32(wr[q][k + r]), a[q][r]);
         }
     } else {
-        for (k = lane; k < K; k += 64) a0 = fmaf(to_f32(xr[k]), to_f32(wr[k]), a0);
+        for (k = lane; k < K; k += 64)
+#pragma unroll
+            for (int q = 0; q < FF; ++q) a[q][0] = fmaf(to_f32(xr[k]), to_f32(wr[q][k]), a[q][0]);
     }
-    const float s = wave_sum((a0 + a1) + (a2 + a3));
-    if (lane == 0) out[unit] = s;
+#pragma unroll
+    for (int q = 0; q < FF; ++q) {
+        const float s = wave_sum((a[q][0] + a[q][1]) + (a[q][2] + a[q][3]));
+        if (lane == 0 && f + q < N) out[m * N + f + q] = s;
+    }
 }
 
 extern "C" int fl_gemm_few(const void* x, const void* w, float* out, int dtype, int M, int N, int K, hipStream_t stream) {
     FL_CHECK(M >= 0 && N > 0 && K > 0, "gemm_few: bad sizes M=%d N=%d K=%d", M, N, K);
     if (M == 0) return 0;
-    const long total = (long)M * N;
+    const bool many = M >= 64;
+    const long total = (long)M * (many ? ceil_div(N, 4) : N);
     const long blocks = (total + 3) / 4;
     FL_CHECK(blocks < (1L << 31), "gemm_few: too many outputs");
-    if (dtype == FL_F32) gemm_few_kernel<float><<<(unsigned)blocks, 256, 0, stream>>>((const float*)x, (const float*)w, out, total, N, K);
-    else if (dtype == FL_BF16) gemm_few_kernel<bf16_t><<<(unsigned)blocks, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)w, out, total, N, K);
+#define FL_GF(T, FF) gemm_few_kernel<T, FF><<<(unsigned)blocks, 256, 0, stream>>>((const T*)x, (const T*)w, out, total, N, K)
+    if (dtype == FL_F32) { if (many) FL_GF(float, 4); else FL_GF(float, 1); }
+    else if (dtype == FL_BF16) { if (many) FL_GF(bf16_t, 4); else FL_GF(bf16_t, 1); }
+#undef FL_GF
     else FL_CHECK(false, "gemm_few: unknown dtype %d", dtype);
     FL_LAUNCH_CHECK();
     return 0;

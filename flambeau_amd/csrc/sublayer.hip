@@ -188,12 +188,12 @@ FL_RECORDABLE(fl_sublayer_step)
 // p % taps, so that a step of one token writes a place it does not read, and running it twice changes nothing.  A
 // request's first tokens of a step (those that reach behind it) and the ring itself belong to the threads of its first
 // token, which read the ring before they write it; all other tokens read rows of the step only.
-#define IC_TOKENS 8          // tokens per block of a step of many (a step of few: one)
-template <typename T, int VEC>
+template <typename T, int VEC, int TAPS>          // TAPS 0: as many as `n_taps` says, in a loop that is not unrolled
 __global__ __launch_bounds__(256) void input_conv_kernel(const T* __restrict__ h, const float* __restrict__ w, float* __restrict__ ring,
                                                          const int* __restrict__ positions, const int* __restrict__ tok_seq,
                                                          const int* __restrict__ seq_q_start, const int* __restrict__ seq_q_len,
-                                                         const int* __restrict__ seq_slots, T* __restrict__ out, int n, int C, int taps, int per_block) {
+                                                         const int* __restrict__ seq_slots, T* __restrict__ out, int C, int n_taps) {
+    const int taps = TAPS > 0 ? TAPS : n_taps;
     const int c = (blockIdx.x * 256 + threadIdx.x) * VEC;
     if (c >= C) return;
     auto load = [&](const auto* p, float* v) {
@@ -214,6 +214,7 @@ __global__ __launch_bounds__(256) void input_conv_kernel(const T* __restrict__ h
         float acc[VEC], x[VEC], wk[VEC], own[VEC];
 #pragma unroll
         for (int e = 0; e < VEC; ++e) acc[e] = 0.f;
+#pragma unroll
         for (int k = 0; k < taps; ++k) {
             if (!row(k, x)) continue;
             load(w + (size_t)k * C + c, wk);
@@ -225,31 +226,28 @@ __global__ __launch_bounds__(256) void input_conv_kernel(const T* __restrict__ h
         for (int e = 0; e < VEC; ++e) acc[e] += own[e];
         store(out + (size_t)t * C + c, acc);
     };
-    const int t_end = min(n, (int)(blockIdx.y + 1) * per_block);
-    for (int t = blockIdx.y * per_block; t < t_end; ++t) {
-        const int s = tok_seq[t], i = t - seq_q_start[s];
-        if (i >= taps - 1 && i > 0) {
-            token(t, [&](int k, float* x) { load(h + (size_t)(t - taps + 1 + k) * C + c, x); return true; });
-        } else if (i == 0) {
-            const int len = seq_q_len[s], slot = seq_slots[s], p0 = positions[t];
-            float* mine = slot >= 0 ? ring + (size_t)slot * taps * C : nullptr;          // (rows that pad a batch have no slot)
-            const int own = max(1, min(taps - 1, len));
-            for (int j = 0; j < own; ++j)
-                token(t + j, [&](int k, float* x) {
-                    const int p = p0 + j - taps + 1 + k;
-                    if (p < 0) return false;
-                    if (p >= p0) { load(h + (size_t)(t + p - p0) * C + c, x); return true; }
-                    if (!mine) return false;
-                    load(mine + (size_t)(p % taps) * C + c, x);
-                    return true;
-                });
-            if (mine && taps > 1)
-                for (int j = max(0, len - taps + 1); j < len; ++j) {
-                    float x[VEC];
-                    load(h + (size_t)(t + j) * C + c, x);
-                    store(mine + (size_t)((p0 + j) % taps) * C + c, x);
-                }
-        }
+    const int t = blockIdx.y, s = tok_seq[t], i = t - seq_q_start[s];
+    if (i >= taps - 1 && i > 0) {
+        token(t, [&](int k, float* x) { load(h + (size_t)(t - taps + 1 + k) * C + c, x); return true; });
+    } else if (i == 0) {
+        const int len = seq_q_len[s], slot = seq_slots[s], p0 = positions[t];
+        float* mine = slot >= 0 ? ring + (size_t)slot * taps * C : nullptr;          // (rows that pad a batch have no slot)
+        const int own = max(1, min(taps - 1, len));
+        for (int j = 0; j < own; ++j)
+            token(t + j, [&](int k, float* x) {
+                const int p = p0 + j - taps + 1 + k;
+                if (p < 0) return false;
+                if (p >= p0) { load(h + (size_t)(t + p - p0) * C + c, x); return true; }
+                if (!mine) return false;
+                load(mine + (size_t)(p % taps) * C + c, x);
+                return true;
+            });
+        if (mine && taps > 1)
+            for (int j = max(0, len - taps + 1); j < len; ++j) {
+                float x[VEC];
+                load(h + (size_t)(t + j) * C + c, x);
+                store(mine + (size_t)((p0 + j) % taps) * C + c, x);
+            }
     }
 }
 
@@ -259,14 +257,22 @@ extern "C" int fl_input_conv(const void* h, int dtype, const float* w, float* ri
     FL_CHECK(n >= 0 && C > 0 && taps > 0 && h && w && out && h != out, "input_conv: bad sizes or a missing tensor");
     FL_CHECK(ring && positions && tok_seq && seq_q_start && seq_q_len && seq_slots, "input_conv: the requests' kept inputs are missing");
     if (n == 0) return 0;
-    const int per_block = n >= 1024 ? IC_TOKENS : 1, tiles = ceil_div(n, per_block);
-    FL_CHECK(tiles <= 65535, "input_conv: %d rows are more than one grid takes", n);
+    FL_CHECK(n <= 65535, "input_conv: %d rows are more than one grid takes", n);
     const bool vec = C % 4 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)w % 16 == 0 && (uintptr_t)ring % 16 == 0 && (uintptr_t)out % 16 == 0;
-    dim3 grid(ceil_div(C, 256 * (vec ? 4 : 1)), tiles);
-#define FL_IC(T, V) input_conv_kernel<T, V><<<grid, 256, 0, stream>>>((const T*)h, w, ring, positions, tok_seq, seq_q_start, seq_q_len, seq_slots, (T*)out, n, C, taps, per_block)
-    if (dtype == FL_F32) { if (vec) FL_IC(float, 4); else FL_IC(float, 1); }
-    else if (dtype == FL_BF16) { if (vec) FL_IC(bf16_t, 4); else FL_IC(bf16_t, 1); }
+    dim3 grid(ceil_div(C, 256 * (vec ? 4 : 1)), n);
+#define FL_IC(T, V, N) input_conv_kernel<T, V, N><<<grid, 256, 0, stream>>>((const T*)h, w, ring, positions, tok_seq, seq_q_start, seq_q_len, seq_slots, (T*)out, C, taps)
+#define FL_IC_N(T)                                                         \
+    do {                                                                    \
+        if (!vec) FL_IC(T, 1, 0);                                          \
+        else if (taps == 2) FL_IC(T, 4, 2);                                \
+        else if (taps == 3) FL_IC(T, 4, 3);                                \
+        else if (taps == 4) FL_IC(T, 4, 4);                                \
+        else FL_IC(T, 4, 0);                                               \
+    } while (0)
+    if (dtype == FL_F32) FL_IC_N(float);
+    else if (dtype == FL_BF16) FL_IC_N(bf16_t);
     else FL_CHECK(false, "input_conv: unknown dtype %d", dtype);
+#undef FL_IC_N
 #undef FL_IC
     FL_LAUNCH_CHECK();
     return 0;
