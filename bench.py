@@ -34,6 +34,11 @@ routed feed-forwards with the squared relu) at two sizes, six layers, beside the
 window that keeps the first tokens, chunked attention with a sink beside a delta rule with decays per key dim, a grouped
 router with identity experts and a shared expert) at two sizes, six layers, beside the closest design the engine has,
 Fitevik, at the same widths, head counts, windows and experts; a line of the same shape.
+
+``--config lufivik``: the Lufivik design (norms on both sides of a sublayer with a gated, scaled residual, a convolution in
+front of every mixer, latent attention with a rotated key part and a window, experts with a clamped gate, a looped
+stretch) at two sizes, six layer runs, beside the closest design the engine has, Kuvidra, at the same sizes; a line of
+the same shape.
 """
 from __future__ import annotations
 
