@@ -63,10 +63,11 @@ int fl_sample_history(unsigned short* counts, int V, int slot, const int* tokens
 // ---- attention over one cached latent per token (latent.hip) ----
 // From the joined projection of a step's tokens (float rows) to the normed query latent (columns 0 .. q_width - 1) in
 // q_out and, with write_cache, the token's row in its page: the normed latent (R columns from kv_col on) and behind it
-// a rotated key part of rot_dim columns (rot of them turned by cs [n][rot / 2][2]); pool [n_pages][page_size * (K + V)],
+// a rotated key part of rot_dim columns (rot of them turned by cs [n][rot / 2][2], dimension i with i + rot / 2 or,
+// interleaved, 2i with 2i + 1); pool [n_pages][page_size * (K + V)],
 // a page's rows [page_size][K] = (latent, zeros to V, rotated part, zeros) and its values transposed, [V][page_size]
 int fl_latent_prepare(const float* x, int ld, int q_width, const float* qw, void* q_out, int kv_col, int R,
-                      const float* kw, float eps, int rot_dim, int rot, const float* cs, void* pool, int dtype,
+                      const float* kw, float eps, int rot_dim, int rot, int interleaved, const float* cs, void* pool, int dtype,
                       int K, int V, int n, const int* positions, const int* tok_seq, const int* block_table,
                       int max_blocks, int page_size, int n_pages, int write_cache, hipStream_t stream);
 // one small product per head: out[t][h][:] = x[t][h][:] W_h (transposed: W_h^T), optionally times the sigmoid of a gate
@@ -74,35 +75,36 @@ int fl_latent_prepare(const float* x, int ld, int q_width, const float* qw, void
 // for the head's rotated part: the rot_dim values behind its K in x, turned, to column rot_at of its row (rot_dim 0: none)
 int fl_heads_matmul(const float* x, int ldx, int hx, const void* w, int w_dtype, void* out, int out_dtype, int ho, int n,
                     int H, int K, int J, int transposed, const float* gate, int ldg, int gate_col0, int rot_dim, int rot,
-                    const float* cs, int rot_at, hipStream_t stream);
+                    int interleaved, const float* cs, int rot_at, hipStream_t stream);
 // z[t][h][0:R] = sum_j softmax_j(scale * qa[t][h] . row_j) row_j[0:R] over the visible rows (K values each) of the
-// token's request: j <= position, with window > 0 the newest `window` of them
+// token's request: j <= position, with window > 0 the newest `window` of them; sink (float [H], or null): e^sink joins
+// the head's denominator
 int fl_latent_attention(const float* qa, float* z, const void* pool, int dtype, const int* positions,
                         const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
-                        int page_size, int n_pages, float scale, int window, hipStream_t stream);
+                        int page_size, int n_pages, float scale, int window, const float* sink, hipStream_t stream);
 int fl_latent_max_width(void);
 // the same on the matrix cores for bfloat16 pools (latent_tuned.hip): qa bfloat16 [n][H][K], z float [n][H][R]
 int fl_latent_attention_mfma(const void* qa, float* z, const void* pool, const int* positions,
                              const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                              int page_size, int n_pages, float scale, int window, int n_split, float* part_o,
-                             float* part_ml, hipStream_t stream);
+                             float* part_ml, const float* sink, hipStream_t stream);
 int fl_latent_attention_mfma_takes(int K, int R, int page_size);
 // the same for prompt portions: blocks of four waves that share their keys through LDS; tiles [n_tiles][4] =
 // (first token, tokens, first group of 16 heads, groups), tokens x groups <= 4, the tokens of one request
 int fl_latent_attention_shared(const void* qa, float* z, const void* pool, const int* positions,
                                const int* tok_seq, const int* block_table, int max_blocks, int H, int K, int R,
                                int page_size, int n_pages, float scale, int window, const int* tiles, int n_tiles,
-                               hipStream_t stream);
+                               const float* sink, hipStream_t stream);
 long fl_latent_attention_shared_lds(int K, int R);
 // and for steps of few rows: a block of four waves per (token, 16 heads, part of the keys) that deal the latent's dims out among them
 int fl_latent_attention_dealt(const void* qa, float* z, const void* pool, const int* positions,
                               const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                               int page_size, int n_pages, float scale, int window, int n_split, float* part_o,
-                              float* part_ml, hipStream_t stream);
+                              float* part_ml, const float* sink, hipStream_t stream);
 // out[t][h][j] = sum_k x[t][h][k] w[h][j][k] on the matrix cores (w bfloat16 [H][J][K]); strides and rotated part as for fl_heads_matmul
 int fl_heads_matmul_mfma(const void* x, int x_dtype, int ldx, int hx, const void* w, void* out, int out_dtype, int ho, int n,
                          int H, int K, int J, const float* gate, int ldg, int gate_col0, int rot_dim, int rot,
-                         const float* cs, int rot_at, hipStream_t stream);
+                         int interleaved, const float* cs, int rot_at, hipStream_t stream);
 int fl_heads_matmul_mfma_takes(int K, int J);
 
 // ---- around a sublayer that is normed on both sides (sublayer.hip) ----
@@ -174,6 +176,13 @@ int fl_add_rowvec(float* x, const float* v, int n, int W, hipStream_t stream);
 // epilogue: 0 = plain product; 1 = SwiGLU over interleaved gate/up rows, out_cols <= N / 2
 int fl_gemm_skinny(const void* x, const void* w_packed, void* out, int out_dtype, int M, int N, int K,
                    int nw_hint, int epilogue, int out_cols, hipStream_t stream);
+// epilogue 1 with the clamped gate: out = g sigmoid(alpha g) (u + shift), g = min(gate, limit), u = up within +-limit
+int fl_gemm_skinny_clamped(const void* x, const void* w_packed, void* out, int out_dtype, int M, int N, int K,
+                           int out_cols, float alpha, float limit, float shift, hipStream_t stream);
+int fl_gemm_mid_clamped(const void* x, const void* w_packed, void* out, int out_dtype, int M, int N, int K,
+                        int out_cols, float alpha, float limit, float shift, hipStream_t stream);
+int fl_gemm_tiled_clamped(const void* x, const void* w_packed, void* out, int out_dtype, int M, int N, int K,
+                          int out_cols, float alpha, float limit, float shift, hipStream_t stream);
 
 // The same product fused with the norms around it (at most 16 rows).  in_ssq (or null): [M, in_parts]
 // partial sums of squares; every row of the result is multiplied by rsqrt(sum / K + eps).
@@ -304,15 +313,15 @@ int fl_reduce_dyt(const float* part, float* resid, const float* alpha, const flo
 int fl_attn_plain_capped(const void* q, void* out, const void* cache_base, int dtype,
                          const int* positions, const int* tok_seq, const int* block_table,
                          int max_blocks, int n, int nh, int nkv, int hd, int page_size, int n_pages,
-                         float scale, int window, float softcap, hipStream_t stream);
+                         float scale, int window, float softcap, const float* sink, hipStream_t stream);
 int fl_attn_decode_items_capped(const void* q, void* out, float* part_o, float* part_ml, const void* cache_base,
                                 const int* items, int n_items, const int* block_table, int max_blocks, int nh,
                                 int nkv, int hd, int page_size, int n_pages, float scale, int window,
-                                float softcap, const int* firsts, int n_rows, hipStream_t stream);
+                                float softcap, const float* sink, const int* firsts, int n_rows, hipStream_t stream);
 int fl_attn_prefill_capped(const void* q, void* out, const void* cache_base, const int* tiles,
                            int n_tiles, const int* positions, const int* block_table,
                            int max_blocks, int nh, int nkv, int hd, int page_size, int n_pages,
-                           float scale, int window, float softcap, int qt_hint, float* part_o, float* part_ml,
+                           float scale, int window, float softcap, const float* sink, int qt_hint, float* part_o, float* part_ml,
                            int n_split, hipStream_t stream);
 
 // ---- rows of the residual stream and of mixers' outputs (stream_ops.hip) ----
@@ -326,9 +335,10 @@ int fl_gated_act(const float* gu, void* out, int out_dtype, int n, int I, int ki
 // out = ca * a / rms(a) * wa + cb * b / rms(b) * wb per row
 int fl_norm_mix(const float* a, const float* wa, float ca, const float* b, const float* wb, float cb, float* out,
                 int n, int H, float eps, hipStream_t stream);
-// out[t][h][j < Dv] = x[t][h][j] * g(gate[t][gate_col0 + h * Dv + j]), heads of x ldh wide; g: 0 none, 1 sigmoid, 2 silu
-int fl_heads_gate(const void* x, int dtype, int ldh, const float* gate, int ldg, int gate_col0, int kind, void* out,
-                  int n, int H, int Dv, hipStream_t stream);
+// out[t][h][j < Dv] = scale * x[t][h][j] * g(gate[t][gate_col0 + h * Dv + j]) (per_head: gate[t][gate_col0 + h]), heads of x ldh
+// wide, rows of out ldo wide; g: 0 none, 1 sigmoid, 2 silu
+int fl_heads_gate(const void* x, int dtype, int ldh, const float* gate, int ldg, int gate_col0, int kind, int per_head,
+                  float scale, void* out, int ldo, int n, int H, int Dv, hipStream_t stream);
 
 // ---- between a joined q/k/v projection and attention (qkv_prepare.hip) ----
 int fl_qkv_prepare(const float* proj, int ld, int col_q, int col_k, int col_v, const int* positions,
@@ -363,9 +373,34 @@ int fl_channel_decay(const float* a, int ld, int col, const float* a_log, const 
 // (w_rows [N][R]: a step of few tokens reads it) and transposed (wt [R][N]); x float, the factor in dtype
 int fl_lowrank_expand(const float* x, int ld, int col, const void* w_rows, const void* wt, int dtype, float* out,
                       int n, int N, int R, hipStream_t stream);
+// the same with a forget gate behind it: out = sigmoid(sum + bias)^inv_tau
+int fl_lowrank_gate(const float* x, int ld, int col, const void* w_rows, const void* wt, int dtype, const float* bias,
+                    float inv_tau, float* out, int n, int N, int R, hipStream_t stream);
+// fl_linear_scan with a decay per token, head and key dim: S <- diag(g) S + k v^T, o = o_scale S^T q
+int fl_linear_scan_gated(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv,
+                         const float* decay, int ldd, float o_scale, float* state, long slot_stride,
+                         const int* seq_q_start, const int* seq_q_len, const int* seq_slots, float* out,
+                         int n_seqs, int H, int G, int D, int Dv, hipStream_t stream);
+// and with a decay and a write strength per token and head: S <- decay S + write k v^T, o = S^T q + skip[head] v
+int fl_linear_scan_written(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv,
+                           const float* decay, const float* write, int ldg, const float* skip, float* state,
+                           long slot_stride, const int* seq_q_start, const int* seq_q_len, const int* seq_slots,
+                           float* out, int n_seqs, int H, int G, int D, int Dv, hipStream_t stream);
 int fl_rotate_scale(const float* proj, int ld, int col_a, int col_b, const float* cs, int rot, int interleaved,
                     float scale_a, float scale_b, float* out_a, float* out_b, int n, int H, int D,
                     hipStream_t stream);
+
+// ---- around the walk of a state-space mixer (state_space.hip) ----
+// out[t][c] = silu(bias[c] + sum_k w[k][c] x_(t - taps + 1 + k)[c]), x the columns col0 .. of proj (w [taps][C]; ring, slot_stride
+// floats per slot: the kept inputs [taps][C]); gates[t] = (decay, step) per head: dt = softplus(proj[t][col_dt + h] + dt_bias[h]),
+// decay = exp(-exp(a_log[h]) dt)
+int fl_conv_steps(const float* proj, int ld, int col0, const float* w, const float* bias, float* ring, long slot_stride,
+                  const int* positions, const int* tok_seq, const int* seq_q_start, const int* seq_q_len,
+                  const int* seq_slots, float* out, int n, int C, int taps, int col_dt, int H, const float* dt_bias,
+                  const float* a_log, float* gates, hipStream_t stream);
+// out = v / rms(v) * w in `parts` equal parts of a row, v = y silu(gate[t][gate_col0 + i])
+int fl_gated_group_norm(const float* y, const float* gate, int ldg, int gate_col0, const float* w, void* out,
+                        int out_dtype, int ldo, int n, int W, int parts, float eps, hipStream_t stream);
 
 // ---- layer norm, learned positions, forget gates per key dim, attention whose heads' scores are mixed ----
 // out = (v - mean) / sqrt(var + eps) * w + b of v = x (+ delta); resid_out, rows as for fl_rmsnorm; b may be null

@@ -45,7 +45,7 @@ __global__ __launch_bounds__(256, HDP <= 128 ? 2 : 1) void attn_decode_kernel(
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, float* part_o,
     float* part_ml, PagedCache cache, const int4* __restrict__ items,
     const int* __restrict__ block_table, int max_blocks, int nh, float scale, int window,
-    int n_split, int q_tiles, int ps_shift, int item_base, float softcap) {
+    int n_split, int q_tiles, int ps_shift, int item_base, float softcap, const float* __restrict__ sink) {
     constexpr int QS = HDP / 32;     // k-steps of the score product
     constexpr int DT = HDP / 16;     // 16-wide tiles of head dims in the output
     constexpr bool PIPELINED = HDP <= 128;       // two chunks of keys and values fit the registers
@@ -251,7 +251,7 @@ __global__ __launch_bounds__(256, HDP <= 128 ? 2 : 1) void attn_decode_kernel(
         }
         // lane (head li, group g) holds dims 16 t + 4 g + r
         if (head_ok && n_split == 1) {
-            const float inv = ll > 0.f ? 1.0f / ll : 0.f;
+            const float inv = sink ? softmax_factor_with_sink(mm, ll, sink[head]) : ll > 0.f ? 1.0f / ll : 0.f;
             bf16_t* orow = out + ((size_t)token * nh + head) * hd;
 #pragma unroll
             for (int t = 0; t < DT; ++t) {
@@ -298,13 +298,13 @@ __global__ __launch_bounds__(256) void attn_decode_merge_items_kernel(const floa
                                                                       bf16_t* __restrict__ out,
                                                                       const int4* __restrict__ items,
                                                                       const int4* __restrict__ firsts, int nh,
-                                                                      int hd, int hdp) {
+                                                                      int hd, int hdp, const float* __restrict__ sink) {
     const int head = blockIdx.y;
     const int4 row = firsts[blockIdx.x];
     const int first = row.y, n_split = row.z;
     if (n_split <= 1) return;
     attn_merge_splits(part_o, part_ml, out + ((size_t)row.x * nh + head) * hd, (size_t)first * nh + head, hd, hdp, n_split,
-                      (size_t)nh);
+                      (size_t)nh, sink ? sink + head : nullptr);
 }
 
 extern "C" int fl_attn_decode_workspace(int n_items, int nh, int hd, int n_split, long* o_floats,
@@ -319,13 +319,14 @@ static int attn_decode_launch(const char* who, const void* q, void* out, float* 
                               const void* cache_base, const int* items, int n_items, const int* block_table,
                               int max_blocks, int nh, int nkv, int hd, int page_size, int n_pages,
                               float scale, int window, int n_split, hipStream_t stream, bool own_splits = false,
-                              const int* firsts = nullptr, int n_rows = 0, float softcap = 0.f) {
+                              const int* firsts = nullptr, int n_rows = 0, float softcap = 0.f, const float* sink = nullptr) {
     FL_CHECK(n_items >= 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "%s: bad head counts %d/%d", who, nh, nkv);
     FL_CHECK(hd > 0 && hd <= 256 && hd % 8 == 0, "%s: head size %d must be a multiple of 8 up to 256", who, hd);
     FL_CHECK(page_size % 8 == 0, "%s: page size %d must be a multiple of 8", who, page_size);
     FL_CHECK(n_split >= 1 && n_split <= 256, "%s: %d splits", who, n_split);
     FL_CHECK(n_split == 1 || (part_o && part_ml), "%s: splits need a workspace", who);
     FL_CHECK(window >= 0, "%s: negative window", who);
+    FL_CHECK(!sink || own_splits, "%s: a sink comes with rows that have splits of their own", who);
     FL_CHECK((uintptr_t)items % 16 == 0, "%s: the items must be 16-byte aligned", who);
     if (n_items == 0) return 0;
     int ps_shift = -1;
@@ -341,7 +342,7 @@ static int attn_decode_launch(const char* who, const void* q, void* out, float* 
 #define FL_DEC(HDP_)                                                                                  \
     attn_decode_kernel<HDP_><<<grid, 256, 0, stream>>>((const bf16_t*)q, (bf16_t*)out, part_o, part_ml, c,       \
                                                        (const int4*)items, block_table, max_blocks, nh, scale,   \
-                                                       window, n_split, q_tiles, ps_shift, item_base, softcap)
+                                                       window, n_split, q_tiles, ps_shift, item_base, softcap, sink)
         switch (hdp) {
             case 32: FL_DEC(32); break;
             case 64: FL_DEC(64); break;
@@ -360,7 +361,7 @@ static int attn_decode_launch(const char* who, const void* q, void* out, float* 
             FL_CHECK((uintptr_t)firsts % 16 == 0, "%s: the rows' first items must be 16-byte aligned", who);
             dim3 mg(n_rows, nh);
             attn_decode_merge_items_kernel<<<mg, 256, 0, stream>>>(part_o, part_ml, (bf16_t*)out, (const int4*)items,
-                                                                   (const int4*)firsts, nh, hd, hdp);
+                                                                   (const int4*)firsts, nh, hd, hdp, sink);
             FL_LAUNCH_CHECK();
         }
     } else if (n_split > 1) {
@@ -396,15 +397,16 @@ extern "C" int fl_attn_decode_items(const void* q, void* out, float* part_o, flo
 }
 FL_RECORDABLE(fl_attn_decode_items)
 
-// the same with the scores capped: score <- softcap * tanh(score / softcap) before the softmax (softcap > 0)
+// the same with the scores capped, score <- softcap * tanh(score / softcap) before the softmax (softcap > 0; 0: as they
+// are), and with a sink per query head in the denominator (sink float [nh], or null)
 extern "C" int fl_attn_decode_items_capped(const void* q, void* out, float* part_o, float* part_ml, const void* cache_base,
                                            const int* items, int n_items, const int* block_table, int max_blocks, int nh,
                                            int nkv, int hd, int page_size, int n_pages, float scale, int window,
-                                           float softcap, const int* firsts, int n_rows, hipStream_t stream) {
+                                           float softcap, const float* sink, const int* firsts, int n_rows, hipStream_t stream) {
     FL_CHECK(!firsts || (part_o && part_ml), "attn_decode_items: needs a workspace");
     FL_CHECK(softcap >= 0.f, "attn_decode_items: negative cap");
     return attn_decode_launch("attn_decode_items", q, out, part_o, part_ml, cache_base, items, n_items, block_table, max_blocks,
-                              nh, nkv, hd, page_size, n_pages, scale, window, 1, stream, true, firsts, n_rows, softcap);
+                              nh, nkv, hd, page_size, n_pages, scale, window, 1, stream, true, firsts, n_rows, softcap, sink);
 }
 FL_RECORDABLE(fl_attn_decode_items_capped)
 

@@ -4,14 +4,14 @@
 // without keys).  out[d] = sum_s part_o[s][d] e^(m_s - m) / sum_s l_s e^(m_s - m), m = max m_s.  One
 // block of 256 threads per (row, head): the pairs are read by one thread each, then every thread
 // owns head dims and adds the splits' outputs, loads issued eight at a time.  The order of the sums
-// is fixed (rising split).
+// is fixed (rising split).  A sink (`sink`: the head's score, or null) joins the denominator once.
 #pragma once
 #include "common.h"
 
 // Split s lies in slot base + s * stride.
 __device__ __forceinline__ void attn_merge_splits(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                                   bf16_t* __restrict__ out_row, size_t base, int hd, int hdp, int n_split,
-                                                  size_t stride = 1) {
+                                                  size_t stride = 1, const float* __restrict__ sink = nullptr) {
     __shared__ float s_f[256];       // exp(m_s - m_max) per split (n_split <= 256)
     __shared__ float s_l[256];
     __shared__ float s_inv;
@@ -34,7 +34,7 @@ __device__ __forceinline__ void attn_merge_splits(const float* __restrict__ part
     if (t == 0) {
         float ll = 0.f;
         for (int s = 0; s < n_split; ++s) ll += s_l[s];
-        s_inv = ll > 0.f ? 1.0f / ll : 0.f;
+        s_inv = sink ? softmax_factor_with_sink(mm, ll, *sink) : ll > 0.f ? 1.0f / ll : 0.f;
     }
     __syncthreads();
     const float inv = s_inv;

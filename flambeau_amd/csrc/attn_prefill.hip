@@ -45,7 +45,7 @@ __global__ __launch_bounds__(256, QT * HDP <= 256 ? 2 : 1) void attn_prefill_ker
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, PagedCache cache,
     const int* __restrict__ tiles, const int* __restrict__ positions,
     const int* __restrict__ block_table, int max_blocks, int nh, float scale_log2e, float cap_raw, int window,
-    int log2_ps, int mirror_from, float* __restrict__ part_o, float* __restrict__ part_ml) {
+    int log2_ps, int mirror_from, float* __restrict__ part_o, float* __restrict__ part_ml, const float* __restrict__ sink) {
     constexpr int QS = HDP / 32;              // k-steps of the score product
     constexpr int DT = HDP / 16;              // tiles of head dims in the output
     constexpr int KT = 4 * QS;                // 1 KB tiles of a K stage: [chunk (2)][a/b (2)][k-step]
@@ -379,8 +379,8 @@ __global__ __launch_bounds__(256, QT * HDP <= 256 ? 2 : 1) void attn_prefill_ker
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
         const float ll = l[t][0];
-        const float inv = ll > 0.f ? 1.0f / ll : 0.f;
         const int head = kvh * G + hg * QT + t;
+        const float inv = sink ? softmax_factor_with_sink(m[t] * scale_log2e * 0.6931471805599453f, ll, sink[head]) : ll > 0.f ? 1.0f / ll : 0.f;
         bf16_t* orow = out + ((size_t)(row0 + qtok) * nh + head) * hd;
 #pragma unroll
         for (int d = 0; d < DT; ++d) {
@@ -397,7 +397,7 @@ __global__ __launch_bounds__(256, QT * HDP <= 256 ? 2 : 1) void attn_prefill_ker
 template <int HDP, int QT, int NS>
 static void launch_prefill_one(dim3 grid, hipStream_t stream, const bf16_t* q, bf16_t* out, PagedCache c,
                                const int* tiles, const int* positions, const int* block_table, int max_blocks,
-                               int nh, float scale_log2e, float cap_raw, int window, int log2_ps, float* part_o, float* part_ml, int lds_pages) {
+                               int nh, float scale_log2e, float cap_raw, int window, int log2_ps, float* part_o, float* part_ml, int lds_pages, const float* sink) {
     // blocks that the chip holds at one time: one or two per compute unit
     const int units = fl_units();
     const int total = (int)(grid.x * grid.y * grid.z);
@@ -414,23 +414,23 @@ static void launch_prefill_one(dim3 grid, hipStream_t stream, const bf16_t* q, b
                                   min(RING + PF_MAX_PAGES * (int)sizeof(int), PF_LDS_BYTES));
         configured = true;
     }
-    kern<<<grid, 256, lds, stream>>>(q, out, c, tiles, positions, block_table, max_blocks, nh, scale_log2e, cap_raw, window, log2_ps, mirror_from, part_o, part_ml);
+    kern<<<grid, 256, lds, stream>>>(q, out, c, tiles, positions, block_table, max_blocks, nh, scale_log2e, cap_raw, window, log2_ps, mirror_from, part_o, part_ml, sink);
 }
 
 template <int HDP, int NS>
 static void launch_prefill(int qt, dim3 grid, hipStream_t stream, const bf16_t* q, bf16_t* out, PagedCache c,
                            const int* tiles, const int* positions, const int* block_table, int max_blocks, int nh,
-                           float scale_log2e, float cap_raw, int window, int log2_ps, float* part_o, float* part_ml, int lds_pages) {
+                           float scale_log2e, float cap_raw, int window, int log2_ps, float* part_o, float* part_ml, int lds_pages, const float* sink) {
     if constexpr (HDP <= 64) {            // four heads per wave only where two blocks still fit a compute unit
         if (qt == 4) {
-            launch_prefill_one<HDP, 4, NS>(grid, stream, q, out, c, tiles, positions, block_table, max_blocks, nh, scale_log2e, cap_raw, window, log2_ps, part_o, part_ml, lds_pages);
+            launch_prefill_one<HDP, 4, NS>(grid, stream, q, out, c, tiles, positions, block_table, max_blocks, nh, scale_log2e, cap_raw, window, log2_ps, part_o, part_ml, lds_pages, sink);
             return;
         }
     }
     if (qt >= 2)
-        launch_prefill_one<HDP, 2, NS>(grid, stream, q, out, c, tiles, positions, block_table, max_blocks, nh, scale_log2e, cap_raw, window, log2_ps, part_o, part_ml, lds_pages);
+        launch_prefill_one<HDP, 2, NS>(grid, stream, q, out, c, tiles, positions, block_table, max_blocks, nh, scale_log2e, cap_raw, window, log2_ps, part_o, part_ml, lds_pages, sink);
     else
-        launch_prefill_one<HDP, 1, NS>(grid, stream, q, out, c, tiles, positions, block_table, max_blocks, nh, scale_log2e, cap_raw, window, log2_ps, part_o, part_ml, lds_pages);
+        launch_prefill_one<HDP, 1, NS>(grid, stream, q, out, c, tiles, positions, block_table, max_blocks, nh, scale_log2e, cap_raw, window, log2_ps, part_o, part_ml, lds_pages, sink);
 }
 
 // Query heads per wave (QT, a divisor of the group size) and parts of the keys for a batch of n_tiles
@@ -524,7 +524,8 @@ extern "C" int fl_attn_prefill_workspace(int n_rows, int nh, int hd, int n_split
 __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const float* __restrict__ part_o,
                                                                  const float* __restrict__ part_ml,
                                                                  bf16_t* __restrict__ out, const int* __restrict__ tiles,
-                                                                 int nh, int hd, int hdp, int n_split, int blocks_per_tile) {
+                                                                 int nh, int hd, int hdp, int n_split, int blocks_per_tile,
+                                                                 const float* __restrict__ sink) {
     const int tile = blockIdx.x / blocks_per_tile;
     const int row0 = tiles[4 * tile + 1], cnt = tiles[4 * tile + 2], item0 = tiles[4 * tile + 3];
     const int quads = hdp >> 2;
@@ -553,7 +554,7 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const float* __
             acc += *(const f32x4*)(part_o + (base + s) * hdp + 4 * q4) * f;
         }
     }
-    const float inv = ll > 0.f ? 1.0f / ll : 0.f;
+    const float inv = sink ? softmax_factor_with_sink(mm, ll, sink[head]) : ll > 0.f ? 1.0f / ll : 0.f;
     const int d = 4 * q4;
     bf16_t* orow = out + ((size_t)(row0 + qtok) * nh + head) * hd;
     if (d + 4 <= hd) {
@@ -571,7 +572,7 @@ static int attn_prefill_launch(const void* q, void* out, const void* cache_base,
                                int n_tiles, const int* positions, const int* block_table,
                                int max_blocks, int nh, int nkv, int hd, int page_size, int n_pages,
                                float scale, int window, int qt_hint, float* part_o, float* part_ml, int n_split,
-                               float softcap, hipStream_t stream) {
+                               float softcap, const float* sink, hipStream_t stream) {
     FL_CHECK(n_tiles >= 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attn_prefill: bad head counts %d/%d", nh, nkv);
     FL_CHECK(hd > 0 && hd <= 256 && hd % 8 == 0, "attn_prefill: head size %d must be a multiple of 8 up to 256", hd);
     FL_CHECK(page_size >= 8 && (page_size & (page_size - 1)) == 0,
@@ -599,7 +600,7 @@ static int attn_prefill_launch(const void* q, void* out, const void* cache_base,
     // a ring of two stages: two blocks then fit a compute unit (three stages were no faster)
 #define FL_PF(HDP_)                                                                                            \
     launch_prefill<HDP_, 2>(qt, grid, stream, (const bf16_t*)q, (bf16_t*)out, c, tiles, positions, block_table, \
-                            max_blocks, nh, sl, cap_raw, window, log2_ps, part_o, part_ml, lds_pages)
+                            max_blocks, nh, sl, cap_raw, window, log2_ps, part_o, part_ml, lds_pages, sink)
     switch (hdp) {
         case 32: FL_PF(32); break;
         case 64: FL_PF(64); break;
@@ -615,7 +616,7 @@ static int attn_prefill_launch(const void* q, void* out, const void* cache_base,
     if (n_split > 1) {
         const int blocks_per_tile = ceil_div(PF_TOKENS * nh * (hdp / 4), 256);
         attn_prefill_merge_kernel<<<n_tiles * blocks_per_tile, 256, 0, stream>>>(part_o, part_ml, (bf16_t*)out, tiles, nh, hd,
-                                                                                 hdp, n_split, blocks_per_tile);
+                                                                                 hdp, n_split, blocks_per_tile, sink);
         FL_LAUNCH_CHECK();
     }
     return 0;
@@ -627,18 +628,19 @@ extern "C" int fl_attn_prefill(const void* q, void* out, const void* cache_base,
                                float scale, int window, int qt_hint, float* part_o, float* part_ml, int n_split,
                                hipStream_t stream) {
     return attn_prefill_launch(q, out, cache_base, tiles, n_tiles, positions, block_table, max_blocks, nh, nkv, hd, page_size,
-                               n_pages, scale, window, qt_hint, part_o, part_ml, n_split, 0.f, stream);
+                               n_pages, scale, window, qt_hint, part_o, part_ml, n_split, 0.f, nullptr, stream);
 }
 FL_RECORDABLE(fl_attn_prefill)
 
-// the same with the scores capped: score <- softcap * tanh(score / softcap) before the softmax (softcap > 0)
+// the same with the scores capped, score <- softcap * tanh(score / softcap) before the softmax (softcap > 0; 0: as they
+// are), and with a sink per query head in the denominator (sink float [nh], or null)
 extern "C" int fl_attn_prefill_capped(const void* q, void* out, const void* cache_base, const int* tiles,
                                       int n_tiles, const int* positions, const int* block_table,
                                       int max_blocks, int nh, int nkv, int hd, int page_size, int n_pages,
-                                      float scale, int window, float softcap, int qt_hint, float* part_o, float* part_ml,
+                                      float scale, int window, float softcap, const float* sink, int qt_hint, float* part_o, float* part_ml,
                                       int n_split, hipStream_t stream) {
     FL_CHECK(softcap >= 0.f, "attn_prefill: negative cap");
     return attn_prefill_launch(q, out, cache_base, tiles, n_tiles, positions, block_table, max_blocks, nh, nkv, hd, page_size,
-                               n_pages, scale, window, qt_hint, part_o, part_ml, n_split, softcap, stream);
+                               n_pages, scale, window, qt_hint, part_o, part_ml, n_split, softcap, sink, stream);
 }
 FL_RECORDABLE(fl_attn_prefill_capped)

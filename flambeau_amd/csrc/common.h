@@ -38,11 +38,13 @@ template <typename T> __device__ __forceinline__ T from_f32(float v);
 template <> __device__ __forceinline__ float from_f32<float>(float v) { return v; }
 template <> __device__ __forceinline__ bf16_t from_f32<bf16_t>(float v) { return (bf16_t)v; }
 
-// The gate of a gated feed-forward, act(gate) * up: 0 silu, 1 gelu in its tanh form, 2 gelu with the error function.
+// The gate of a gated feed-forward, act(gate) * up: 0 silu, 1 gelu in its tanh form, 2 gelu with the error function,
+// 3 the clamped gate below (which comes with constants: launch functions of its own take them).
 // (The codes that launch functions take in the bits of `epilogue` above the low four.)
 #define FL_GATE_SILU 0
 #define FL_GATE_GELU_TANH 1
 #define FL_GATE_GELU_ERF 2
+#define FL_GATE_CLAMPED 3
 template <int KIND>
 __device__ __forceinline__ float gate_activation(float z) {
     if (KIND == FL_GATE_GELU_TANH) return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
@@ -54,12 +56,21 @@ __device__ __forceinline__ float clamped_gate(float zg, float zu, float alpha, f
     const float g = fminf(zg, limit), u = fminf(fmaxf(zu, -limit), limit);
     return g / (1.0f + expf(-alpha * g)) * (u + shift);
 }
+struct GateConstants {
+    float alpha, limit, shift;
+};
+template <int KIND>
+__device__ __forceinline__ float gate_value(float g, float u, const GateConstants& c) {
+    if constexpr (KIND == FL_GATE_CLAMPED) return clamped_gate(g, u, c.alpha, c.limit, c.shift);
+    else return gate_activation<KIND>(g) * u;
+}
 // f(constant of the kind): the choice is made once, outside the loops over a block's values (a branch per value
 // cost the tiled gate/up product 7 % of its time)
 template <typename F>
 __device__ __forceinline__ void with_gate_kind(int kind, F&& f) {
     if (kind == FL_GATE_GELU_TANH) f(std::integral_constant<int, FL_GATE_GELU_TANH>{});
     else if (kind == FL_GATE_GELU_ERF) f(std::integral_constant<int, FL_GATE_GELU_ERF>{});
+    else if (kind == FL_GATE_CLAMPED) f(std::integral_constant<int, FL_GATE_CLAMPED>{});
     else f(std::integral_constant<int, FL_GATE_SILU>{});
 }
 
@@ -92,6 +103,14 @@ __device__ __forceinline__ float block_sum(float v, float* lds) {
 #pragma unroll
     for (int w = 0; w < NW; ++w) t += lds[w];
     return t;
+}
+
+// A sink in the denominator of a softmax: a score that has no key and no value.  `m` is the base the weights were
+// taken against and `l` their sum; what the weighted sum has to be multiplied by is e^(m - M) / (l e^(m - M) + e^(sink - M)),
+// M = max(m, sink).  (No key at all: m is minus infinity, and the factor 0.)
+__device__ __forceinline__ float softmax_factor_with_sink(float m, float l, float sink) {
+    const float top = fmaxf(m, sink), f = expf(m - top);
+    return f / fmaf(l, f, expf(sink - top));
 }
 
 // Paged cache of one layer: [n_pages][2 (K,V)][n_kv_heads][page_size * head_dim].

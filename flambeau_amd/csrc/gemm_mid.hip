@@ -47,7 +47,7 @@ template <> __device__ __forceinline__ void gm_store4<bf16_t>(bf16_t* p, f32x4 v
 template <int MT, int GM_NW, int GM_CH, typename TOut, bool SWIGLU>
 __global__ __launch_bounds__(GM_NW * 64) void gemm_mid_kernel(const bf16_t* x, const bf16_t* wp, TOut* out, int M, int N, int K,
                                                               int n_steps, int chunks_per_split, int out_cols,
-                                                              const float* in_ssq, int in_parts, float eps, int gate_kind) {
+                                                              const float* in_ssq, int in_parts, float eps, int gate_kind, GateConstants gate) {
     constexpr int FR = GM_CH * MT;                    // 1 KB operand tiles of x per chunk
     constexpr int XL = (FR + GM_NW - 1) / GM_NW;      // x loads per wave and chunk
     __shared__ __attribute__((aligned(16))) bf16_t slots[2][FR * 512];
@@ -226,7 +226,7 @@ __global__ __launch_bounds__(GM_NW * 64) void gemm_mid_kernel(const bf16_t* x, c
                 f32x4 act;
                 with_gate_kind(gate_kind, [&](auto kind) {
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) act[r] = gate_activation<decltype(kind)::value>(acc[mt][r]) * up[r];
+                    for (int r = 0; r < 4; ++r) act[r] = gate_value<decltype(kind)::value>(acc[mt][r], up[r], gate);
                 });
                 TOut* p = out + (size_t)tok * out_cols + f0;
                 if (out_cols % 4 == 0 && f0 + 4 <= out_cols) {
@@ -366,6 +366,7 @@ struct MidScale {              // the row scale of a product whose x is a norm i
     int in_parts;
     float eps;
     int gate_kind;             // the SwiGLU epilogue's activation of the gate (FL_GATE_*, 0 = silu)
+    GateConstants gate;        // of the clamped gate
 };
 
 template <int MT, int NW, int CH, typename TOut, bool SWIGLU>
@@ -376,7 +377,7 @@ static void launch_mid_shape(const bf16_t* x, const bf16_t* wp, TOut* out, int M
     const int per = ceil_div(n_chunks, splits);
     dim3 grid(ceil_div(ceil_div(N, 16), NW), splits);
     gemm_mid_kernel<MT, NW, CH, TOut, SWIGLU><<<grid, NW * 64, 0, stream>>>(x, wp, out, M, N, K, n_steps, per, out_cols,
-                                                                            sc.in_ssq, sc.in_parts, sc.eps, sc.gate_kind);
+                                                                            sc.in_ssq, sc.in_parts, sc.eps, sc.gate_kind, sc.gate);
 }
 
 template <int MT, typename TOut, bool SWIGLU>
@@ -411,16 +412,16 @@ static int mid_checks(const void* x, const void* w_packed, int M, int N, int K) 
 // from the N interleaved gate/up rows of w; K is not split then.  in_ssq (or null): [M, in_parts]
 // partial sums of squares of the rows that x was made from; every token's results are multiplied
 // by rsqrt(sum / K + eps).
-extern "C" int fl_gemm_mid_ex(const void* x, const void* w_packed, void* out, float* workspace, int out_dtype,
-                              int M, int N, int K, int epilogue, int out_cols, const float* in_ssq, int in_parts,
-                              float eps, int waves, int forced_splits, hipStream_t stream) {
+static int mid_entry(const void* x, const void* w_packed, void* out, float* workspace, int out_dtype,
+                     int M, int N, int K, int epilogue, int out_cols, const float* in_ssq, int in_parts,
+                     float eps, int waves, int forced_splits, const GateConstants& gate, hipStream_t stream) {
     FL_CHECK(waves == 0 || waves == 4 || waves == 8, "gemm_mid: %d waves per block (0, 4 or 8)", waves);
     if (mid_checks(x, w_packed, M, N, K)) return -1;
     FL_CHECK(out_dtype == FL_F32 || out_dtype == FL_BF16, "gemm_mid: unknown output dtype %d", out_dtype);
     const int gate_kind = epilogue >> 4;          // the bits above the low four: the activation of the gate (epilogue 1)
     epilogue &= 15;
     FL_CHECK(epilogue == 0 || epilogue == 1, "gemm_mid: unknown epilogue %d", epilogue);
-    FL_CHECK(gate_kind >= 0 && gate_kind <= FL_GATE_GELU_ERF && (gate_kind == 0 || epilogue == 1), "gemm_mid: gate activation %d", gate_kind);
+    FL_CHECK(gate_kind >= 0 && (gate_kind <= FL_GATE_GELU_ERF || (gate_kind == FL_GATE_CLAMPED && gate.limit > 0.f)) && (gate_kind == 0 || epilogue == 1), "gemm_mid: gate activation %d", gate_kind);
     FL_CHECK(epilogue == 0 ? out_cols == N : (N % 16 == 0 && out_cols > 0 && out_cols <= N / 2),
              "gemm_mid: %d output columns do not fit %d rows of w", out_cols, N);
     FL_CHECK((uintptr_t)out % 16 == 0, "gemm_mid: operands must be 16-byte aligned");
@@ -431,7 +432,7 @@ extern "C" int fl_gemm_mid_ex(const void* x, const void* w_packed, void* out, fl
     const int mt = ceil_div(M, 16);
     const bf16_t* xb = (const bf16_t*)x;
     const bf16_t* wb = (const bf16_t*)w_packed;
-    const MidScale sc = {in_ssq, in_parts, eps, gate_kind};
+    const MidScale sc = {in_ssq, in_parts, eps, gate_kind, gate};
     const MidPlan plan = epilogue ? MidPlan{mid_waves(N, waves), 1} : mid_plan(N, K, waves, forced_splits);
     const int splits = plan.splits;
     waves = plan.waves;
@@ -456,7 +457,21 @@ extern "C" int fl_gemm_mid_ex(const void* x, const void* w_packed, void* out, fl
     FL_LAUNCH_CHECK();
     return 0;
 }
+extern "C" int fl_gemm_mid_ex(const void* x, const void* w_packed, void* out, float* workspace, int out_dtype,
+                              int M, int N, int K, int epilogue, int out_cols, const float* in_ssq, int in_parts,
+                              float eps, int waves, int forced_splits, hipStream_t stream) {
+    return mid_entry(x, w_packed, out, workspace, out_dtype, M, N, K, epilogue, out_cols, in_ssq, in_parts, eps, waves, forced_splits,
+                     GateConstants{}, stream);
+}
 FL_RECORDABLE(fl_gemm_mid_ex)
+
+// epilogue 1 with the clamped gate (fl_gemm_skinny_clamped)
+extern "C" int fl_gemm_mid_clamped(const void* x, const void* w_packed, void* out, int out_dtype, int M, int N, int K,
+                                   int out_cols, float alpha, float limit, float shift, hipStream_t stream) {
+    return mid_entry(x, w_packed, out, nullptr, out_dtype, M, N, K, 1 | (FL_GATE_CLAMPED << 4), out_cols, nullptr, 0, 0.f, 0, 0,
+                     GateConstants{alpha, limit, shift}, stream);
+}
+FL_RECORDABLE(fl_gemm_mid_clamped)
 
 extern "C" int fl_gemm_mid_scaled(const void* x, const void* w_packed, void* out, float* workspace, int out_dtype,
                                   int M, int N, int K, int epilogue, int out_cols, const float* in_ssq, int in_parts,

@@ -56,6 +56,7 @@ struct SkinnyFusion {
     int gate_kind;            // epilogue 1: the gate's activation (FL_GATE_*, 0 = silu)
     const float* dyt_alpha;   // epilogue 2, or null: the norm that follows is tanh(alpha resid) * g + bias, which needs no
     const float* dyt_bias;    //   statistic: xg holds the finished norm and no sums of squares are left (bias may be null)
+    GateConstants gate;       // of the clamped gate (FL_GATE_CLAMPED)
 };
 
 #define SKINNY_SCALE_LOADS 4     // loads of partial sums per thread for the row scale
@@ -332,7 +333,7 @@ __global__ __launch_bounds__(T == 1 ? 1024 : 512) void gemm_skinny_kernel(const 
                     f32x4 act;
                     with_gate_kind(fu.gate_kind, [&](auto kind) {
 #pragma unroll
-                        for (int r = 0; r < 4; ++r) act[r] = gate_activation<decltype(kind)::value>(sum[r]) * up[r];
+                        for (int r = 0; r < 4; ++r) act[r] = gate_value<decltype(kind)::value>(sum[r], up[r], fu.gate);
                     });
                     TOut* p = out + (size_t)tok * out_cols + f0;
                     if (out_cols % 4 == 0 && f0 + 4 <= out_cols) {
@@ -456,7 +457,7 @@ static int skinny_entry(const void* x, const void* w_packed, void* out, int out_
     SkinnyFusion fu = fusion;
     fu.gate_kind = epilogue >> 4;
     epilogue &= 15;
-    FL_CHECK(fu.gate_kind >= 0 && fu.gate_kind <= FL_GATE_GELU_ERF && (fu.gate_kind == 0 || epilogue == EPI_SWIGLU),
+    FL_CHECK(fu.gate_kind >= 0 && (fu.gate_kind <= FL_GATE_GELU_ERF || (fu.gate_kind == FL_GATE_CLAMPED && fu.gate.limit > 0.f)) && (fu.gate_kind == 0 || epilogue == EPI_SWIGLU),
              "gemm_skinny: gate activation %d with epilogue %d", fu.gate_kind, epilogue);
     FL_CHECK(M >= 0 && N > 0 && K > 0, "gemm_skinny: bad sizes M=%d N=%d K=%d", M, N, K);
     FL_CHECK(M <= 64, "gemm_skinny: %d rows, at most 64", M);
@@ -517,6 +518,16 @@ extern "C" int fl_gemm_skinny(const void* x, const void* w_packed, void* out, in
     return skinny_entry(x, w_packed, out, out_dtype, M, N, K, nw_hint, epilogue, out_cols, none, RopeStore{}, stream);
 }
 FL_RECORDABLE(fl_gemm_skinny)
+
+// epilogue 1 with the clamped gate, out[M, out_cols] = g sigmoid(alpha g) (u + shift), g = min(gate, limit), u = up within
+// +-limit
+extern "C" int fl_gemm_skinny_clamped(const void* x, const void* w_packed, void* out, int out_dtype, int M, int N, int K,
+                                      int out_cols, float alpha, float limit, float shift, hipStream_t stream) {
+    SkinnyFusion fu = {nullptr, 0, 0.f, nullptr, nullptr, nullptr, nullptr};
+    fu.gate = {alpha, limit, shift};
+    return skinny_entry(x, w_packed, out, out_dtype, M, N, K, 0, EPI_SWIGLU | (FL_GATE_CLAMPED << 4), out_cols, fu, RopeStore{}, stream);
+}
+FL_RECORDABLE(fl_gemm_skinny_clamped)
 
 // The same product fused with the norms around it.  in_ssq (or null): [M, in_parts] partial sums of
 // squares of the rows that x was made from; every token's results are multiplied by

@@ -55,6 +55,7 @@ struct TiledFusion {
     int gate_kind;             // the SwiGLU epilogue's activation of the gate (FL_GATE_*, 0 = silu)
     const float* dyt_alpha;    // the residual epilogue, or null: the norm that follows is tanh(alpha resid) * g + bias, which
     const float* dyt_bias;     //   needs no statistic: xg holds the finished norm, out_ssq may be null (bias may be null)
+    GateConstants gate;        // of the clamped gate (FL_GATE_CLAMPED)
 };
 
 
@@ -349,7 +350,7 @@ __global__ __launch_bounds__(128 * WT, OCC) void gemm_async_kernel(const bf16_t*
                     if ((g & 1) == 0 && tok < M && f0 < out_cols) {
                         f32x4 act;
 #pragma unroll
-                        for (int r = 0; r < 4; ++r) act[r] = gate_activation<decltype(kind)::value>(acc[ta][tb][r]) * up[r];
+                        for (int r = 0; r < 4; ++r) act[r] = gate_value<decltype(kind)::value>(acc[ta][tb][r], up[r], fu.gate);
                         TOut* p = out + (size_t)tok * out_cols + f0;
                         if (out_cols % 4 == 0 && f0 + 4 <= out_cols) {
                             tg_store4<TOut>(p, act);
@@ -520,17 +521,16 @@ extern "C" int fl_gemm_tiled_shape(int M, int N, int K, int may_split) { return 
 // epilogue 0: out[M, N] = x w^T.  epilogue 1 (SwiGLU): out[M, out_cols] = silu(gate) * up from the
 // N interleaved gate/up rows of w (K is not split then).  in_ssq (or null): [M, in_parts] partial sums of
 // squares of the rows that x was made from; every token's results are multiplied by rsqrt(sum / K + eps).
-extern "C" int fl_gemm_tiled_ex(const void* x, const void* w_packed, void* out, float* workspace,
-                                int out_dtype, int M, int N, int K, int epilogue, int out_cols,
-                                const float* in_ssq, int in_parts, float eps, int variant, int forced_splits,
-                                hipStream_t stream) {
+static int tiled_entry(const void* x, const void* w_packed, void* out, float* workspace, int out_dtype, int M, int N, int K,
+                       int epilogue, int out_cols, const float* in_ssq, int in_parts, float eps, int variant,
+                       int forced_splits, const GateConstants& gate, hipStream_t stream) {
     FL_CHECK(M >= 0 && N > 0 && K > 0, "gemm_tiled: bad sizes M=%d N=%d K=%d", M, N, K);
     FL_CHECK(K % 8 == 0, "gemm_tiled: K=%d is no multiple of 8 (16-byte loads)", K);
     FL_CHECK(out_dtype == FL_F32 || out_dtype == FL_BF16, "gemm_tiled: unknown output dtype %d", out_dtype);
     const int gate_kind = epilogue >> 4;          // the bits above the low four: the activation of the gate (epilogue 1)
     epilogue &= 15;
     FL_CHECK(epilogue == 0 || epilogue == 1, "gemm_tiled: unknown epilogue %d", epilogue);
-    FL_CHECK(gate_kind >= 0 && gate_kind <= FL_GATE_GELU_ERF && (gate_kind == 0 || epilogue == 1), "gemm_tiled: gate activation %d", gate_kind);
+    FL_CHECK(gate_kind >= 0 && (gate_kind <= FL_GATE_GELU_ERF || (gate_kind == FL_GATE_CLAMPED && gate.limit > 0.f)) && (gate_kind == 0 || epilogue == 1), "gemm_tiled: gate activation %d", gate_kind);
     FL_CHECK(epilogue == 0 ? out_cols == N : (N % 16 == 0 && out_cols > 0 && out_cols <= N / 2),
              "gemm_tiled: %d output columns do not fit %d rows of w", out_cols, N);
     FL_CHECK(((uintptr_t)x % 16 == 0) && ((uintptr_t)w_packed % 16 == 0) && ((uintptr_t)out % 16 == 0),
@@ -546,7 +546,7 @@ extern "C" int fl_gemm_tiled_ex(const void* x, const void* w_packed, void* out, 
     const bf16_t* xb = (const bf16_t*)x;
     const bf16_t* wb = (const bf16_t*)w_packed;
     const RopeStore none{};
-    const TiledFusion fu = {in_ssq, in_parts, eps, nullptr, nullptr, nullptr, nullptr, gate_kind};
+    const TiledFusion fu = {in_ssq, in_parts, eps, nullptr, nullptr, nullptr, nullptr, gate_kind, nullptr, nullptr, gate};
     if (epilogue) {
         if (out_dtype == FL_F32)
             launch_tiled<float, TG_SWIGLU>(v, 1, stream, xb, wb, (float*)out, M, N, K, n_steps, per, out_cols, none, fu);
@@ -569,7 +569,22 @@ extern "C" int fl_gemm_tiled_ex(const void* x, const void* w_packed, void* out, 
     FL_LAUNCH_CHECK();
     return 0;
 }
+extern "C" int fl_gemm_tiled_ex(const void* x, const void* w_packed, void* out, float* workspace,
+                                int out_dtype, int M, int N, int K, int epilogue, int out_cols,
+                                const float* in_ssq, int in_parts, float eps, int variant, int forced_splits,
+                                hipStream_t stream) {
+    return tiled_entry(x, w_packed, out, workspace, out_dtype, M, N, K, epilogue, out_cols, in_ssq, in_parts, eps, variant, forced_splits,
+                       GateConstants{}, stream);
+}
 FL_RECORDABLE(fl_gemm_tiled_ex)
+
+// epilogue 1 with the clamped gate (fl_gemm_skinny_clamped)
+extern "C" int fl_gemm_tiled_clamped(const void* x, const void* w_packed, void* out, int out_dtype, int M, int N, int K,
+                                     int out_cols, float alpha, float limit, float shift, hipStream_t stream) {
+    return tiled_entry(x, w_packed, out, nullptr, out_dtype, M, N, K, 1 | (FL_GATE_CLAMPED << 4), out_cols, nullptr, 0, 0.f, 0, 0,
+                       GateConstants{alpha, limit, shift}, stream);
+}
+FL_RECORDABLE(fl_gemm_tiled_clamped)
 
 extern "C" int fl_gemm_tiled_scaled(const void* x, const void* w_packed, void* out, float* workspace,
                                     int out_dtype, int M, int N, int K, int epilogue, int out_cols,

@@ -21,14 +21,14 @@
 // x: float rows ld wide, the joined projection of a step's tokens.  Two blocks per token: one norms the query
 // latent, out[r, :] = v * w * rsqrt(mean(v^2) + eps), v = x[r, 0 : q_width]; the other norms the cached latent (the
 // columns kv_col .. kv_col + R - 1) and stores it in the page row of the token's position, and turns the rot_dim
-// columns behind it by the token's angles (cs [n][rot / 2][2]; dimension i with i + rot / 2, those from rot on as
-// they are) into the row's tail.  A page holds [page_size][K] rows and, behind them, [V][page_size] transposed
+// columns behind it by the token's angles (cs [n][rot / 2][2]; dimension i with i + rot / 2 or, interleaved, 2i with
+// 2i + 1, those from rot on as they are) into the row's tail.  A page holds [page_size][K] rows and, behind them, [V][page_size] transposed
 // values; the matrix cores want the index that is summed over contiguous, a row's values for the scores and the keys
 // for the weighted sum.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(
     const float* __restrict__ x, int ld, int q_width, const float* __restrict__ qw, T* __restrict__ q_out, int kv_col,
-    int R, const float* __restrict__ kw, float eps, int rot_dim, int rot, const float* __restrict__ cs,
+    int R, const float* __restrict__ kw, float eps, int rot_dim, int rot, int interleaved, const float* __restrict__ cs,
     T* __restrict__ pool, int K, int V, const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_table, int max_blocks, int page_size, int n_pages) {
     __shared__ float red[4];
@@ -56,14 +56,14 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
     for (int i = threadIdx.x; i < K; i += 256) {
         float v = 0.f;
         if (i < R) v = xr[i] * (w ? w[i] : 1.0f) * inv;
-        else if (i >= V && i < V + rot_dim) v = rotated_value(xt, i - V, rot, cs + (size_t)r * rot);
+        else if (i >= V && i < V + rot_dim) v = rotated_value(xt, i - V, rot, interleaved, cs + (size_t)r * rot);
         rows[(size_t)row * K + i] = from_f32<T>(v);
         if (i < V) cols[(size_t)i * page_size + row] = from_f32<T>(v);
     }
 }
 
 extern "C" int fl_latent_prepare(const float* x, int ld, int q_width, const float* qw, void* q_out, int kv_col, int R,
-                                 const float* kw, float eps, int rot_dim, int rot, const float* cs, void* pool, int dtype,
+                                 const float* kw, float eps, int rot_dim, int rot, int interleaved, const float* cs, void* pool, int dtype,
                                  int K, int V, int n, const int* positions, const int* tok_seq, const int* block_table,
                                  int max_blocks, int page_size, int n_pages, int write_cache, hipStream_t stream) {
     FL_CHECK(n >= 0 && q_width > 0 && R > 0 && kv_col >= 0 && rot_dim >= 0 && ld >= q_width && ld >= kv_col + R + rot_dim,
@@ -74,9 +74,9 @@ extern "C" int fl_latent_prepare(const float* x, int ld, int q_width, const floa
     if (n == 0) return 0;
     dim3 grid(n, write_cache ? 2 : 1);
     if (dtype == FL_F32)
-        latent_prepare_kernel<float><<<grid, 256, 0, stream>>>(x, ld, q_width, qw, (float*)q_out, kv_col, R, kw, eps, rot_dim, rot, cs, (float*)pool, K, V, positions, tok_seq, block_table, max_blocks, page_size, n_pages);
+        latent_prepare_kernel<float><<<grid, 256, 0, stream>>>(x, ld, q_width, qw, (float*)q_out, kv_col, R, kw, eps, rot_dim, rot, interleaved, cs, (float*)pool, K, V, positions, tok_seq, block_table, max_blocks, page_size, n_pages);
     else if (dtype == FL_BF16)
-        latent_prepare_kernel<bf16_t><<<grid, 256, 0, stream>>>(x, ld, q_width, qw, (bf16_t*)q_out, kv_col, R, kw, eps, rot_dim, rot, cs, (bf16_t*)pool, K, V, positions, tok_seq, block_table, max_blocks, page_size, n_pages);
+        latent_prepare_kernel<bf16_t><<<grid, 256, 0, stream>>>(x, ld, q_width, qw, (bf16_t*)q_out, kv_col, R, kw, eps, rot_dim, rot, interleaved, cs, (bf16_t*)pool, K, V, positions, tok_seq, block_table, max_blocks, page_size, n_pages);
     else
         FL_CHECK(false, "latent_prepare: unknown dtype %d", dtype);
     FL_LAUNCH_CHECK();
@@ -143,12 +143,12 @@ __global__ __launch_bounds__(256) void heads_matmul_kernel(const float* __restri
 
 extern "C" int fl_heads_matmul(const float* x, int ldx, int hx, const void* w, int w_dtype, void* out, int out_dtype, int ho,
                                int n, int H, int K, int J, int transposed, const float* gate, int ldg, int gate_col0,
-                               int rot_dim, int rot, const float* cs, int rot_at, hipStream_t stream) {
+                               int rot_dim, int rot, int interleaved, const float* cs, int rot_at, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && K > 0 && J > 0 && hx >= K + rot_dim && ho >= J && (long)ldx >= (long)(H - 1) * hx + K + rot_dim,
              "heads_matmul: bad sizes n=%d H=%d K=%d J=%d ld=%d head strides %d, %d", n, H, K, J, ldx, hx, ho);
     FL_CHECK(rot_dim >= 0 && rot >= 0 && rot % 2 == 0 && rot <= rot_dim && (rot == 0 || cs) && (rot_dim == 0 || (rot_at >= J && rot_at + rot_dim <= ho)),
              "heads_matmul: a rotated part of %d (%d turned) at %d of %d", rot_dim, rot, rot_at, ho);
-    const QueryTail tail = {ho - J, K, rot_at - J, rot_dim, rot, cs};
+    const QueryTail tail = {ho - J, K, rot_at - J, rot_dim, rot, interleaved, cs};
     const size_t lds = (size_t)HM_TOKENS * K * sizeof(float);
     FL_CHECK(lds <= 64 * 1024, "heads_matmul: %d values per head are more than a block keeps", K);
     FL_CHECK(!gate || ldg >= gate_col0 + H, "heads_matmul: gate columns %d..%d of rows %d wide", gate_col0, gate_col0 + H, ldg);
@@ -171,14 +171,15 @@ FL_RECORDABLE(fl_heads_matmul)
 // maximum and sum, then lanes own the latent's dims (R: a row's values, the first of its K) and add the chunk's weighted rows.  The query at
 // position p sees keys 0..p of its own request (window > 0: the newest `window` of them), all read
 // from the pages (this step's rows were stored before).  Rows beyond p are never loaded, so whatever
-// an unused or reused page holds cannot reach a sum.
+// an unused or reused page holds cannot reach a sum.  sink (float [H], or null): a score per head that joins the
+// denominator once, not scaled, with no key and no value.
 #define LA_WAVES 4
 #define LA_MAX_DIMS 16        // latent dims per lane: R <= 64 * LA_MAX_DIMS
 template <typename T, int VPL>
 __global__ __launch_bounds__(64 * LA_WAVES) void latent_attention_kernel(
     const float* __restrict__ qa, float* __restrict__ z, const T* __restrict__ pool, const int* __restrict__ positions,
     const int* __restrict__ tok_seq, const int* __restrict__ block_table, int max_blocks, int H, int K, int R, int page_size,
-    int n_pages, float scale, int window, int heads_per_block) {
+    int n_pages, float scale, int window, int heads_per_block, const float* __restrict__ sink) {
     extern __shared__ float lds[];                    // [heads_per_block][K] folded queries, then [LA_WAVES][64] weights
     const int token = blockIdx.x;
     const int h0 = blockIdx.y * heads_per_block;
@@ -233,7 +234,7 @@ __global__ __launch_bounds__(64 * LA_WAVES) void latent_attention_kernel(
             }
             __builtin_amdgcn_wave_barrier();
         }
-        const float inv = l > 0.f ? 1.0f / l : 0.f;
+        const float inv = sink ? softmax_factor_with_sink(m, l, sink[h0 + hh]) : l > 0.f ? 1.0f / l : 0.f;
         float* zr = z + ((size_t)token * H + h0 + hh) * R;
 #pragma unroll
         for (int u = 0; u < VPL; ++u) {
@@ -247,7 +248,7 @@ extern "C" int fl_latent_max_width(void) { return 64 * LA_MAX_DIMS; }
 
 extern "C" int fl_latent_attention(const float* qa, float* z, const void* pool, int dtype, const int* positions,
                                    const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
-                                   int page_size, int n_pages, float scale, int window, hipStream_t stream) {
+                                   int page_size, int n_pages, float scale, int window, const float* sink, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && R > 0 && K >= R && K <= 2 * 64 * LA_MAX_DIMS && page_size > 0 && n_pages > 0 && max_blocks > 0, "latent_attention: bad sizes");
     FL_CHECK(R <= 64 * LA_MAX_DIMS, "latent_attention: a latent of %d values, at most %d", R, 64 * LA_MAX_DIMS);
     FL_CHECK(window >= 0, "latent_attention: negative window");
@@ -262,7 +263,7 @@ extern "C" int fl_latent_attention(const float* qa, float* z, const void* pool, 
 #define FL_LA(TT, V)                                                                                                  \
     latent_attention_kernel<TT, V><<<grid, 64 * LA_WAVES, lds, stream>>>(qa, z, (const TT*)pool, positions, tok_seq, \
                                                                          block_table, max_blocks, H, K, R, page_size, \
-                                                                         n_pages, scale, window, hpb)
+                                                                         n_pages, scale, window, hpb, sink)
 #define FL_LA_V(TT)                                  \
     do {                                             \
         if (vpl <= 1) FL_LA(TT, 1);                  \

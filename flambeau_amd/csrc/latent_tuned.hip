@@ -14,6 +14,7 @@
 //
 // A row is K values wide as a key and R as a value (its first R values; K > R where a rotated key part stands behind
 // the latent); folded queries are K wide, the weighted sums R.
+// sink (float [H], or null): a score per head that joins the denominator once, not scaled, with no key and no value.
 //
 // A kernel is compiled for the most steps of 32 values it takes and runs that many whatever K and R are: a step beyond
 // K multiplies zeros of the query with the row's first values, one beyond R fills sums that nobody reads.  A branch
@@ -42,7 +43,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
     const bf16_t* __restrict__ qa, float* __restrict__ z, const bf16_t* __restrict__ pool,
     const int* __restrict__ positions, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
     int max_blocks, int n, int H, int K, int R, int page_size, int n_pages, float scale, int window, int groups_per_token,
-    int n_split, float* __restrict__ part_o, float* __restrict__ part_ml) {
+    int n_split, float* __restrict__ part_o, float* __restrict__ part_ml, const float* __restrict__ sink) {
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int unit = blockIdx.x * LT_WAVES + wave;                 // (token, group of 16 heads, part of the keys)
     if (unit >= n * groups_per_token * n_split) return;
@@ -162,7 +163,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
         return;
     }
     if (!head_live) return;
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    const float inv = sink ? softmax_factor_with_sink(m, l, sink[h0 + col]) : l > 0.f ? 1.0f / l : 0.f;
     float* zr = z + ((size_t)token * H + h0 + col) * R;
 #pragma unroll
     for (int t = 0; t < 2 * NS; ++t)
@@ -173,7 +174,8 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_mfma_kernel(
 // (rising s; an empty part left zeros and has weight 0).  A block takes 256 dims of one (token, head): its
 // first wave makes the parts' weights, then every thread adds its dim's parts, all loads independent.
 __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
-                                                           float* __restrict__ z, int H, int R, int groups, int n_split) {
+                                                           float* __restrict__ z, int H, int R, int groups, int n_split,
+                                                           const float* __restrict__ sink) {
     __shared__ float ws[64];
     __shared__ float inv_l;
     const int unit = blockIdx.x, d = blockIdx.y * 256 + threadIdx.x;
@@ -187,7 +189,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restri
         const float w = ms > -INFINITY ? expf(ms - M) : 0.f;
         const float L = wave_sum(ls * w);
         ws[lane] = w;
-        if (lane == 0) inv_l = L > 0.f ? 1.0f / L : 0.f;
+        if (lane == 0) inv_l = sink ? softmax_factor_with_sink(M, L, sink[h]) : L > 0.f ? 1.0f / L : 0.f;
     }
     __syncthreads();
     if (d >= R) return;
@@ -206,7 +208,7 @@ extern "C" int fl_latent_attention_mfma_takes(int K, int R, int page_size) {
 extern "C" int fl_latent_attention_mfma(const void* qa, float* z, const void* pool, const int* positions,
                                         const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                                         int page_size, int n_pages, float scale, int window, int n_split, float* part_o,
-                                        float* part_ml, hipStream_t stream) {
+                                        float* part_ml, const float* sink, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && n_pages > 0 && max_blocks > 0, "latent_attention_mfma: bad sizes");
     FL_CHECK(n_split >= 1 && n_split <= 64 && (n_split == 1 || (part_o && part_ml)), "latent_attention_mfma: %d parts of the keys (at most 64) need a workspace", n_split);
     FL_CHECK(fl_latent_attention_mfma_takes(K, R, page_size), "latent_attention_mfma: rows of %d and %d values in pages of %d are not taken", K, R, page_size);
@@ -222,7 +224,7 @@ extern "C" int fl_latent_attention_mfma(const void* qa, float* z, const void* po
     latent_attention_mfma_kernel<NK, NS><<<blocks, 64 * LT_WAVES, 0, stream>>>((const bf16_t*)qa, z, (const bf16_t*)pool,  \
                                                                            positions, tok_seq, block_table, max_blocks, \
                                                                            n, H, K, R, page_size, n_pages, scale, window, groups, \
-                                                                           n_split, part_o, part_ml)
+                                                                           n_split, part_o, part_ml, sink)
     if (K == R) {
         if (ns <= 2) FL_LT(2, 2);
         else if (ns <= 4) FL_LT(4, 4);
@@ -238,7 +240,7 @@ extern "C" int fl_latent_attention_mfma(const void* qa, float* z, const void* po
     FL_LAUNCH_CHECK();
     if (n_split > 1) {
         dim3 mgrid(n * H, ceil_div(R, 256));
-        latent_merge_kernel<<<mgrid, 256, 0, stream>>>(part_o, part_ml, z, H, R, groups, n_split);
+        latent_merge_kernel<<<mgrid, 256, 0, stream>>>(part_o, part_ml, z, H, R, groups, n_split, sink);
         FL_LAUNCH_CHECK();
     }
     return 0;
@@ -256,7 +258,8 @@ template <int NK, int NS>
 __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
     const bf16_t* __restrict__ qa, float* __restrict__ z, const bf16_t* __restrict__ pool,
     const int* __restrict__ positions, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
-    int max_blocks, int H, int K, int R, int page_size, int n_pages, float scale, int window, const int* __restrict__ tiles) {
+    int max_blocks, int H, int K, int R, int page_size, int n_pages, float scale, int window, const int* __restrict__ tiles,
+    const float* __restrict__ sink) {
     extern __shared__ __attribute__((aligned(16))) unsigned char lt_smem[];
     const int stride_r = K + 8, stride_c = LT_CHUNK + 8;
     bf16_t* ks = (bf16_t*)lt_smem;                                  // [64 keys][K + 8]
@@ -382,7 +385,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_shared_kernel(
         __syncthreads();
     }
     if (!head_live) return;
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    const float inv = sink ? softmax_factor_with_sink(m, l, sink[h0 + col]) : l > 0.f ? 1.0f / l : 0.f;
     float* zr = z + ((size_t)token * H + h0 + col) * R;
 #pragma unroll
     for (int t = 0; t < 2 * NS; ++t)
@@ -407,7 +410,8 @@ template <int NKH, int NDT>
 __global__ __launch_bounds__(512, 2) void latent_attention_spread_kernel(
     const bf16_t* __restrict__ qa, float* __restrict__ z, const bf16_t* __restrict__ pool,
     const int* __restrict__ positions, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
-    int max_blocks, int H, int K, int R, int page_size, int n_pages, float scale, int window, const int* __restrict__ tiles) {
+    int max_blocks, int H, int K, int R, int page_size, int n_pages, float scale, int window, const int* __restrict__ tiles,
+    const float* __restrict__ sink) {
     constexpr int QS = NKH * 64 + 8;
     extern __shared__ __attribute__((aligned(16))) unsigned char lt_smem[];
     bf16_t* qs = (bf16_t*)lt_smem;                                  // [64 rows][QS]
@@ -548,7 +552,7 @@ __global__ __launch_bounds__(512, 2) void latent_attention_spread_kernel(
         }
     }
     __syncthreads();
-    if (kk == 0) rs[row] = l > 0.f ? 1.0f / l : 0.f;
+    if (kk == 0) rs[row] = sink && live ? softmax_factor_with_sink(m, l, sink[head]) : l > 0.f ? 1.0f / l : 0.f;
     __syncthreads();
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
@@ -564,7 +568,7 @@ __global__ __launch_bounds__(512, 2) void latent_attention_spread_kernel(
 template <int NKH, int NDT>
 static int launch_spread(const void* qa, float* z, const void* pool, const int* positions, const int* tok_seq, const int* block_table,
                          int max_blocks, int H, int K, int R, int page_size, int n_pages, float scale, int window, const int* tiles,
-                         int n_tiles, hipStream_t stream) {
+                         int n_tiles, const float* sink, hipStream_t stream) {
     constexpr int LDS = 64 * (NKH * 64 + 8) * 2 + 2 * 64 * LS_S * 4 + 64 * LS_P * 2 + 64 * 4 + 16;
     static bool sized = false;
     if (!sized) {
@@ -573,7 +577,7 @@ static int launch_spread(const void* qa, float* z, const void* pool, const int* 
         sized = true;
     }
     latent_attention_spread_kernel<NKH, NDT><<<n_tiles, 512, LDS, stream>>>((const bf16_t*)qa, z, (const bf16_t*)pool, positions, tok_seq, block_table,
-                                                                            max_blocks, H, K, R, page_size, n_pages, scale, window, tiles);
+                                                                            max_blocks, H, K, R, page_size, n_pages, scale, window, tiles, sink);
     return 0;
 }
 
@@ -583,14 +587,14 @@ extern "C" long fl_latent_attention_shared_lds(int K, int R) { return (long)LT_C
 extern "C" int fl_latent_attention_shared(const void* qa, float* z, const void* pool, const int* positions,
                                           const int* tok_seq, const int* block_table, int max_blocks, int H, int K, int R,
                                           int page_size, int n_pages, float scale, int window, const int* tiles, int n_tiles,
-                                          hipStream_t stream) {
+                                          const float* sink, hipStream_t stream) {
     FL_CHECK(n_tiles >= 0 && H > 0 && n_pages > 0 && max_blocks > 0, "latent_attention_shared: bad sizes");
     FL_CHECK(fl_latent_attention_mfma_takes(K, R, page_size), "latent_attention_shared: rows of %d and %d values in pages of %d are not taken", K, R, page_size);
     FL_CHECK((uintptr_t)qa % 16 == 0 && (uintptr_t)pool % 16 == 0 && (uintptr_t)z % 16 == 0, "latent_attention_shared: operands must be 16-byte aligned");
     FL_CHECK(window >= 0, "latent_attention_shared: negative window");
     if (n_tiles == 0) return 0;
     if (R == 128 || R == 256 || R == 512) {
-#define FL_LSP(NKH, NDT) launch_spread<NKH, NDT>(qa, z, pool, positions, tok_seq, block_table, max_blocks, H, K, R, page_size, n_pages, scale, window, tiles, n_tiles, stream)
+#define FL_LSP(NKH, NDT) launch_spread<NKH, NDT>(qa, z, pool, positions, tok_seq, block_table, max_blocks, H, K, R, page_size, n_pages, scale, window, tiles, n_tiles, sink, stream)
         const int rc = R == 128 ? (K == R ? FL_LSP(2, 1) : FL_LSP(3, 1)) : R == 256 ? (K == R ? FL_LSP(4, 2) : FL_LSP(5, 2)) : K == R ? FL_LSP(8, 4) : FL_LSP(9, 4);
 #undef FL_LSP
         if (rc != 0) return rc;
@@ -610,7 +614,7 @@ extern "C" int fl_latent_attention_shared(const void* qa, float* z, const void* 
         }                                                                                                              \
         latent_attention_shared_kernel<NK, NS><<<n_tiles, 64 * LT_WAVES, lds, stream>>>(                                  \
             (const bf16_t*)qa, z, (const bf16_t*)pool, positions, tok_seq, block_table, max_blocks, H, K, R, page_size,   \
-            n_pages, scale, window, tiles);                                                                            \
+            n_pages, scale, window, tiles, sink);                                                                            \
     } while (0)
     if (K == R) {
         if (ns <= 2) FL_LTS(2, 2);
@@ -641,7 +645,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
     const bf16_t* __restrict__ qa, float* __restrict__ z, const bf16_t* __restrict__ pool,
     const int* __restrict__ positions, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
     int max_blocks, int n, int H, int K, int R, int page_size, int n_pages, float scale, int window, int groups_per_token,
-    int n_split, float* __restrict__ part_o, float* __restrict__ part_ml) {
+    int n_split, float* __restrict__ part_o, float* __restrict__ part_ml, const float* __restrict__ sink) {
     __shared__ f32x4 sx[LT_WAVES][4][64];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int unit = blockIdx.x;                                   // (token, group of 16 heads, part of the keys)
@@ -768,7 +772,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
         return;
     }
     if (!head_live) return;
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    const float inv = sink ? softmax_factor_with_sink(m, l, sink[h0 + col]) : l > 0.f ? 1.0f / l : 0.f;
     float* zr = z + ((size_t)token * H + h0 + col) * R;
 #pragma unroll
     for (int t = 0; t < 2 * NSW; ++t) {
@@ -781,7 +785,7 @@ __global__ __launch_bounds__(64 * LT_WAVES) void latent_attention_dealt_kernel(
 extern "C" int fl_latent_attention_dealt(const void* qa, float* z, const void* pool, const int* positions,
                                          const int* tok_seq, const int* block_table, int max_blocks, int n, int H, int K, int R,
                                          int page_size, int n_pages, float scale, int window, int n_split, float* part_o,
-                                         float* part_ml, hipStream_t stream) {
+                                         float* part_ml, const float* sink, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && n_pages > 0 && max_blocks > 0, "latent_attention_dealt: bad sizes");
     FL_CHECK(n_split >= 1 && n_split <= 64 && (n_split == 1 || (part_o && part_ml)), "latent_attention_dealt: %d parts of the keys (at most 64) need a workspace", n_split);
     FL_CHECK(fl_latent_attention_mfma_takes(K, R, page_size), "latent_attention_dealt: rows of %d and %d values in pages of %d are not taken", K, R, page_size);
@@ -796,7 +800,7 @@ extern "C" int fl_latent_attention_dealt(const void* qa, float* z, const void* p
     latent_attention_dealt_kernel<NKW, NSW><<<(unsigned)units, 64 * LT_WAVES, 0, stream>>>((const bf16_t*)qa, z, (const bf16_t*)pool, \
                                                                                       positions, tok_seq, block_table, max_blocks, \
                                                                                       n, H, K, R, page_size, n_pages, scale, window,  \
-                                                                                      groups, n_split, part_o, part_ml)
+                                                                                      groups, n_split, part_o, part_ml, sink)
     if (nkw <= 1) FL_LTD(1, 1);
     else if (nkw <= 2) FL_LTD(2, 2);
     else if (nsw <= 2 && nkw <= 3) FL_LTD(3, 2);
@@ -806,7 +810,7 @@ extern "C" int fl_latent_attention_dealt(const void* qa, float* z, const void* p
     FL_LAUNCH_CHECK();
     if (n_split > 1) {
         dim3 mgrid(n * H, ceil_div(R, 256));
-        latent_merge_kernel<<<mgrid, 256, 0, stream>>>(part_o, part_ml, z, H, R, groups, n_split);
+        latent_merge_kernel<<<mgrid, 256, 0, stream>>>(part_o, part_ml, z, H, R, groups, n_split, sink);
         FL_LAUNCH_CHECK();
     }
     return 0;
@@ -876,12 +880,12 @@ extern "C" int fl_heads_matmul_mfma_takes(int K, int J) { return K > 0 && K % 8 
 
 extern "C" int fl_heads_matmul_mfma(const void* x, int x_dtype, int ldx, int hx, const void* w, void* out, int out_dtype, int ho,
                                     int n, int H, int K, int J, const float* gate, int ldg, int gate_col0, int rot_dim, int rot,
-                                    const float* cs, int rot_at, hipStream_t stream) {
+                                    int interleaved, const float* cs, int rot_at, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && hx >= K + rot_dim && ho >= J && (long)ldx >= (long)(H - 1) * hx + K + rot_dim, "heads_matmul_mfma: bad sizes");
     FL_CHECK(rot_dim >= 0 && rot >= 0 && rot % 2 == 0 && rot <= rot_dim && (rot == 0 || cs) && (rot_dim == 0 || (rot_at >= J && rot_at + rot_dim <= ho)),
              "heads_matmul_mfma: a rotated part of %d (%d turned) at %d of %d", rot_dim, rot, rot_at, ho);
     FL_CHECK(ho == J || x_dtype == FL_F32, "heads_matmul_mfma: what stands behind a head's results is made of float rows");
-    const QueryTail tail = {ho - J, K, rot_at - J, rot_dim, rot, cs};
+    const QueryTail tail = {ho - J, K, rot_at - J, rot_dim, rot, interleaved, cs};
     FL_CHECK(fl_heads_matmul_mfma_takes(K, J), "heads_matmul_mfma: %d x %d per head is not taken", J, K);
     FL_CHECK((uintptr_t)w % 16 == 0, "heads_matmul_mfma: the weights must be 16-byte aligned");
     FL_CHECK(!gate || ldg >= gate_col0 + H, "heads_matmul_mfma: gate columns beyond rows %d wide", ldg);

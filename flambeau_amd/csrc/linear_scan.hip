@@ -3,10 +3,10 @@
 // fl_linear_scan: per request and head the state S [D][Dv] (float, in the request's slot between
 // steps, zero when the slot is claimed).  For every token, with a decay g (one per head, or one per
 // token and head), q and k of the head's query/key head and v of the head:
-//     S <- g S
-//     u = beta (v - S^T k)     (the delta rule; without beta: u = v)
+//     S <- g S                 (g may be a vector over the key dims: S <- diag(g) S)
+//     u = beta (v - S^T k)     (the delta rule; without beta: u = v; a write strength alone: u = beta v)
 //     S <- S + k u^T
-//     o = S^T q                (the read-out sees the token's own write)
+//     o = S^T q                (the read-out sees the token's own write; optionally times a factor, plus skip v)
 // The walk IS the recurrence, so a prompt cut anywhere leaves the same state and the same outputs.
 //
 // fl_conv_prepare: a short causal convolution over time per channel with silu behind it, for the
@@ -37,14 +37,17 @@
 // LDS after it, so that the trip to memory hides behind the walk.
 // MODE 0: a decay per head or per token and head, u = v; 1: the delta rule; 2: a decay per token, head AND key dim
 // (`k` holds the forget gates f; the key is 1 - f: what is forgotten makes room for what is written); 3: the delta rule
-// with a decay per token, head and key dim (`chan_decay`, rows ldc wide, heads x D: S <- diag(g) S before the correction)
+// with a decay per token, head and key dim (`chan_decay`, rows ldc wide, heads x D: S <- diag(g) S before the correction);
+// 4: such a decay without the correction (gated linear attention: u = v); 5: a decay and a write strength per token and
+// head without the correction (u = beta v), and skip[head] v added to what is read out
 template <int RPT, int MODE>
 __global__ __launch_bounds__(LS_GROUP * LS_COLS) void linear_scan_kernel(
     const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk, const float* __restrict__ v, int ldv,
     const float* __restrict__ head_decay, const float* __restrict__ tok_decay, const float* __restrict__ beta, int ldg,
     float* __restrict__ state, size_t slot_stride, const int* __restrict__ seq_q_start, const int* __restrict__ seq_q_len,
     const int* __restrict__ seq_slots, float* __restrict__ out, int H, int G, int D, int Dv,
-    const float* __restrict__ chan_decay = nullptr, int ldc = 0) {
+    const float* __restrict__ chan_decay = nullptr, int ldc = 0, float o_scale = 1.f, const float* __restrict__ skip = nullptr) {
+    constexpr bool CHAN = MODE == 3 || MODE == 4;
     constexpr int NT = LS_GROUP * LS_COLS;
     constexpr int DP = LS_GROUP * RPT;                                // a row of q or k in LDS
     constexpr int RUN = RPT <= 8 ? 32 : RPT <= 16 ? 16 : 8;          // tokens per run
@@ -63,11 +66,12 @@ __global__ __launch_bounds__(LS_GROUP * LS_COLS) void linear_scan_kernel(
         S[u] = (live && d < D) ? st[(size_t)j * D + d] : 0.f;
     }
     const float fixed = head_decay ? head_decay[head] : 1.f;
+    const float skip_h = MODE == 5 && skip ? skip[head] : 0.f;
     __shared__ __attribute__((aligned(16))) float qs[RUN * DP];
     __shared__ __attribute__((aligned(16))) float ks[RUN * DP];
     __shared__ float vs[RUN * LS_COLS], fs[RUN * 2];
-    __shared__ __attribute__((aligned(16))) float gs[MODE == 3 ? RUN * DP : 4];
-    float pq[PRE], pk[PRE], pd[MODE == 3 ? PRE : 1], pv[PRE_V], pf0 = 0.f, pf1 = 0.f;
+    __shared__ __attribute__((aligned(16))) float gs[CHAN ? RUN * DP : 4];
+    float pq[PRE], pk[PRE], pd[CHAN ? PRE : 1], pv[PRE_V], pf0 = 0.f, pf1 = 0.f;
     auto fetch = [&](int t0) {                     // the values of the run that starts at token t0, into registers
         const int cnt = min(RUN, len - t0);
 #pragma unroll
@@ -78,7 +82,7 @@ __global__ __launch_bounds__(LS_GROUP * LS_COLS) void linear_scan_kernel(
             const size_t row = (size_t)(start + t0 + (in ? tt : 0));
             pq[i] = in ? q[row * ldq + qk_head * D + d] : 0.f;
             pk[i] = in ? k[row * ldk + qk_head * D + d] : (MODE == 2 ? 1.f : 0.f);
-            if (MODE == 3) pd[i] = in ? chan_decay[row * ldc + head * D + d] : 1.f;
+            if (CHAN) pd[i] = in ? chan_decay[row * ldc + head * D + d] : 1.f;
         }
 #pragma unroll
         for (int i = 0; i < PRE_V; ++i) {
@@ -88,8 +92,8 @@ __global__ __launch_bounds__(LS_GROUP * LS_COLS) void linear_scan_kernel(
         }
         if (threadIdx.x < cnt) {
             const size_t row = (size_t)(start + t0 + threadIdx.x);
-            pf0 = (MODE != 3 && tok_decay) ? tok_decay[row * ldg + head] : fixed;
-            pf1 = (MODE == 1 || MODE == 3) ? beta[row * ldg + head] : 1.f;
+            pf0 = (!CHAN && tok_decay) ? tok_decay[row * ldg + head] : fixed;
+            pf1 = (MODE == 1 || MODE == 3 || MODE == 5) ? beta[row * ldg + head] : 1.f;
         }
     };
     if (len > 0) fetch(0);
@@ -100,7 +104,7 @@ __global__ __launch_bounds__(LS_GROUP * LS_COLS) void linear_scan_kernel(
         for (int i = 0; i < PRE; ++i) {
             qs[threadIdx.x + NT * i] = pq[i];
             ks[threadIdx.x + NT * i] = pk[i];
-            if (MODE == 3) gs[threadIdx.x + NT * i] = pd[i];
+            if (CHAN) gs[threadIdx.x + NT * i] = pd[i];
         }
 #pragma unroll
         for (int i = 0; i < PRE_V; ++i)
@@ -120,7 +124,7 @@ __global__ __launch_bounds__(LS_GROUP * LS_COLS) void linear_scan_kernel(
                 if (MODE == 2) {
                     S[u] *= kr[u];
                     kr[u] = 1.0f - kr[u];
-                } else if (MODE == 3) {
+                } else if (CHAN) {
                     S[u] *= gs[tt * DP + g * RPT + u];
                 } else {
                     S[u] *= decay;
@@ -135,6 +139,7 @@ __global__ __launch_bounds__(LS_GROUP * LS_COLS) void linear_scan_kernel(
                 }
                 uv = fs[2 * tt + 1] * (uv - row_sum16(seen0 + seen1));
             }
+            if (MODE == 5) uv *= fs[2 * tt + 1];
             float num0 = 0.f, num1 = 0.f;
 #pragma unroll
             for (int u = 0; u < RPT; u += 2) {
@@ -145,7 +150,9 @@ __global__ __launch_bounds__(LS_GROUP * LS_COLS) void linear_scan_kernel(
                     num1 = fmaf(S[u + 1], qr[u + 1], num1);
                 }
             }
-            const float num = row_sum16(num0 + num1);             // the 16 threads of a column are a row of lanes
+            float num = row_sum16(num0 + num1);                   // the 16 threads of a column are a row of lanes
+            if (MODE == 4) num *= o_scale;
+            if (MODE == 5 && skip) num = fmaf(skip_h, vs[tt * LS_COLS + c], num);
             if (live && g == 0) out[((size_t)(start + t0 + tt) * H + head) * Dv + j] = num;
         }
     }
@@ -162,9 +169,10 @@ static int linear_scan_launch(const float* q, int ldq, const float* k, int ldk, 
                               const float* head_decay, const float* tok_decay, const float* beta, int ldg, float* state,
                               long slot_stride, const int* seq_q_start, const int* seq_q_len, const int* seq_slots,
                               float* out, int n_seqs, int H, int G, int D, int Dv, bool channel_decay, hipStream_t stream,
-                              const float* chan_decay = nullptr, int ldc = 0) {
-    FL_CHECK(!chan_decay || (beta && !head_decay && !tok_decay && !channel_decay && ldc >= H * D),
-             "linear_scan: a decay per key dim under the delta rule comes with write strengths and without another decay");
+                              const float* chan_decay = nullptr, int ldc = 0, bool corrects = true, float o_scale = 1.f,
+                              const float* skip = nullptr) {
+    FL_CHECK(!chan_decay || (!beta == !corrects && !head_decay && !tok_decay && !channel_decay && ldc >= H * D),
+             "linear_scan: a decay per key dim comes without another decay, and under the delta rule with write strengths");
     FL_CHECK(n_seqs >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && Dv > 0, "linear_scan: bad sizes");
     FL_CHECK(D <= LS_GROUP * LS_MAX_ROWS, "linear_scan: %d key dims per head, at most %d", D, LS_GROUP * LS_MAX_ROWS);
     FL_CHECK(ldq >= G * D && ldk >= G * D && ldv >= H * Dv, "linear_scan: rows narrower than their heads");
@@ -179,10 +187,12 @@ static int linear_scan_launch(const float* q, int ldq, const float* k, int ldk, 
 #define FL_LS2(R, MODE)                                                                                               \
     linear_scan_kernel<R, MODE><<<grid, LS_GROUP * LS_COLS, 0, stream>>>(q, ldq, k, ldk, v, ldv, head_decay, tok_decay, beta, \
                                                                           ldg, state, (size_t)slot_stride, seq_q_start,        \
-                                                                          seq_q_len, seq_slots, out, H, G, D, Dv, chan_decay, ldc)
+                                                                          seq_q_len, seq_slots, out, H, G, D, Dv, chan_decay, ldc, o_scale, skip)
 #define FL_LS(R)             \
     do {                     \
-        if (chan_decay) FL_LS2(R, 3);    \
+        if (chan_decay && corrects) FL_LS2(R, 3); \
+        else if (chan_decay) FL_LS2(R, 4);    \
+        else if (beta && !corrects) FL_LS2(R, 5); \
         else if (channel_decay) FL_LS2(R, 2); \
         else if (beta) FL_LS2(R, 1);     \
         else FL_LS2(R, 0);               \
@@ -230,6 +240,30 @@ extern "C" int fl_linear_scan_delta_channel(const float* q, int ldq, const float
 }
 FL_RECORDABLE(fl_linear_scan_delta_channel)
 
+// Gated linear attention: S <- diag(g) S + k v^T, o = o_scale S^T q, with a decay per token, head and key dim (decay: rows
+// ldd wide, heads x D).
+extern "C" int fl_linear_scan_gated(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv,
+                                    const float* decay, int ldd, float o_scale, float* state, long slot_stride,
+                                    const int* seq_q_start, const int* seq_q_len, const int* seq_slots, float* out,
+                                    int n_seqs, int H, int G, int D, int Dv, hipStream_t stream) {
+    FL_CHECK(decay, "linear_scan_gated: the decays are missing");
+    return linear_scan_launch(q, ldq, k, ldk, v, ldv, nullptr, nullptr, nullptr, 0, state, slot_stride, seq_q_start, seq_q_len,
+                              seq_slots, out, n_seqs, H, G, D, Dv, false, stream, decay, ldd, false, o_scale);
+}
+FL_RECORDABLE(fl_linear_scan_gated)
+
+// State-space duality: S <- decay S + write k v^T, o = S^T q + skip v, with a decay and a write strength per token and head
+// (rows ldg wide) and skip per head (or null).
+extern "C" int fl_linear_scan_written(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv,
+                                      const float* decay, const float* write, int ldg, const float* skip, float* state,
+                                      long slot_stride, const int* seq_q_start, const int* seq_q_len, const int* seq_slots,
+                                      float* out, int n_seqs, int H, int G, int D, int Dv, hipStream_t stream) {
+    FL_CHECK(decay && write, "linear_scan_written: decays and write strengths are both needed");
+    return linear_scan_launch(q, ldq, k, ldk, v, ldv, nullptr, decay, write, ldg, state, slot_stride, seq_q_start, seq_q_len,
+                              seq_slots, out, n_seqs, H, G, D, Dv, false, stream, nullptr, 0, false, 1.f, skip);
+}
+FL_RECORDABLE(fl_linear_scan_written)
+
 // g[t][h][d] = exp(-exp(A_log[h]) * softplus(a[t][col + h * D + d] + dt_bias[h * D + d])): the decays of a recurrence
 // that forgets per head and key dim
 __global__ __launch_bounds__(256) void channel_decay_kernel(const float* __restrict__ a, int ld, int col, const float* __restrict__ a_log,
@@ -257,11 +291,22 @@ FL_RECORDABLE(fl_channel_decay)
 // storage type, float sums in rising order of r
 #define LR_TOKENS 8           // tokens a block of fl_lowrank_expand takes: a value of wt is read once for all of them
 #define LR_FEW 16             // up to this many tokens a thread reads its feature's own row of the factor as it is stored
+// What happens to a feature's sum z: nothing, or (a forget gate, inv_tau > 0) sigmoid(z + bias)^inv_tau, formed through its
+// logarithm, -softplus(-z): a gate near one keeps its digits.
+struct LowRankTail {
+    const float* bias;
+    float inv_tau;
+};
+__device__ __forceinline__ float lowrank_tail(const LowRankTail& tail, float z, int f) {
+    if (tail.inv_tau <= 0.f) return z;
+    if (tail.bias) z += tail.bias[f];
+    return expf(-(fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z)))) * tail.inv_tau);
+}
 // (a step of few tokens: a block per token and 256 features, a thread walks the R neighbouring values of its feature's
 // row, which the compiler fetches some at a time; the sums run in rising order of r as in the kernel below)
 template <typename T>
 __global__ __launch_bounds__(256) void lowrank_expand_rows_kernel(const float* __restrict__ x, int ld, int col, const T* __restrict__ w,
-                                                                  float* __restrict__ out, int N, int R) {
+                                                                  float* __restrict__ out, int N, int R, LowRankTail tail) {
     extern __shared__ float xr[];
     const int t = blockIdx.y;
     for (int r = threadIdx.x; r < R; r += 256) xr[r] = x[(size_t)t * ld + col + r];
@@ -271,12 +316,12 @@ __global__ __launch_bounds__(256) void lowrank_expand_rows_kernel(const float* _
     const T* wr = w + (size_t)f * R;
     float s = 0.f;
     for (int r = 0; r < R; ++r) s = fmaf(xr[r], to_f32(wr[r]), s);
-    out[(size_t)t * N + f] = s;
+    out[(size_t)t * N + f] = lowrank_tail(tail, s, f);
 }
 
 template <typename T>
 __global__ __launch_bounds__(256) void lowrank_expand_kernel(const float* __restrict__ x, int ld, int col, const T* __restrict__ w,
-                                                             float* __restrict__ out, int n, int N, int R) {
+                                                             float* __restrict__ out, int n, int N, int R, LowRankTail tail) {
     extern __shared__ float xr[];                         // [LR_TOKENS][R]
     const int t0 = blockIdx.y * LR_TOKENS, cnt = min(LR_TOKENS, n - t0);
     for (int e = threadIdx.x; e < LR_TOKENS * R; e += 256) {
@@ -297,18 +342,18 @@ __global__ __launch_bounds__(256) void lowrank_expand_kernel(const float* __rest
     }
 #pragma unroll
     for (int tt = 0; tt < LR_TOKENS; ++tt)
-        if (tt < cnt) out[(size_t)(t0 + tt) * N + f] = s[tt];
+        if (tt < cnt) out[(size_t)(t0 + tt) * N + f] = lowrank_tail(tail, s[tt], f);
 }
 
-extern "C" int fl_lowrank_expand(const float* x, int ld, int col, const void* w_rows, const void* w, int dtype, float* out,
-                                 int n, int N, int R, hipStream_t stream) {
+static int lowrank_launch(const float* x, int ld, int col, const void* w_rows, const void* w, int dtype, float* out,
+                          int n, int N, int R, const LowRankTail& tail, hipStream_t stream) {
     FL_CHECK(n >= 0 && N > 0 && R > 0 && R <= 1024 && col >= 0 && ld >= col + R, "lowrank_expand: columns %d..%d of rows %d wide (a rank of at most 1024)", col, col + R, ld);
     FL_CHECK(w_rows && w, "lowrank_expand: the factor is wanted as it is stored and transposed");
     if (n == 0) return 0;
     if (n <= LR_FEW) {
         dim3 grid(ceil_div(N, 256), n);
-        if (dtype == FL_F32) lowrank_expand_rows_kernel<float><<<grid, 256, R * sizeof(float), stream>>>(x, ld, col, (const float*)w_rows, out, N, R);
-        else if (dtype == FL_BF16) lowrank_expand_rows_kernel<bf16_t><<<grid, 256, R * sizeof(float), stream>>>(x, ld, col, (const bf16_t*)w_rows, out, N, R);
+        if (dtype == FL_F32) lowrank_expand_rows_kernel<float><<<grid, 256, R * sizeof(float), stream>>>(x, ld, col, (const float*)w_rows, out, N, R, tail);
+        else if (dtype == FL_BF16) lowrank_expand_rows_kernel<bf16_t><<<grid, 256, R * sizeof(float), stream>>>(x, ld, col, (const bf16_t*)w_rows, out, N, R, tail);
         else FL_CHECK(false, "lowrank_expand: unknown dtype %d", dtype);
         FL_LAUNCH_CHECK();
         return 0;
@@ -316,13 +361,26 @@ extern "C" int fl_lowrank_expand(const float* x, int ld, int col, const void* w_
     dim3 grid(ceil_div(N, 256), ceil_div(n, LR_TOKENS));
     FL_CHECK(grid.y <= 65535, "lowrank_expand: %d rows are more than one grid takes", n);
     const size_t lds = (size_t)LR_TOKENS * R * sizeof(float);
-    if (dtype == FL_F32) lowrank_expand_kernel<float><<<grid, 256, lds, stream>>>(x, ld, col, (const float*)w, out, n, N, R);
-    else if (dtype == FL_BF16) lowrank_expand_kernel<bf16_t><<<grid, 256, lds, stream>>>(x, ld, col, (const bf16_t*)w, out, n, N, R);
+    if (dtype == FL_F32) lowrank_expand_kernel<float><<<grid, 256, lds, stream>>>(x, ld, col, (const float*)w, out, n, N, R, tail);
+    else if (dtype == FL_BF16) lowrank_expand_kernel<bf16_t><<<grid, 256, lds, stream>>>(x, ld, col, (const bf16_t*)w, out, n, N, R, tail);
     else FL_CHECK(false, "lowrank_expand: unknown dtype %d", dtype);
     FL_LAUNCH_CHECK();
     return 0;
 }
+
+extern "C" int fl_lowrank_expand(const float* x, int ld, int col, const void* w_rows, const void* w, int dtype, float* out,
+                                 int n, int N, int R, hipStream_t stream) {
+    return lowrank_launch(x, ld, col, w_rows, w, dtype, out, n, N, R, LowRankTail{nullptr, 0.f}, stream);
+}
 FL_RECORDABLE(fl_lowrank_expand)
+
+// the same with a forget gate behind it: out = sigmoid(sum + bias)^inv_tau (bias float [N], or null)
+extern "C" int fl_lowrank_gate(const float* x, int ld, int col, const void* w_rows, const void* w, int dtype, const float* bias,
+                               float inv_tau, float* out, int n, int N, int R, hipStream_t stream) {
+    FL_CHECK(inv_tau > 0.f, "lowrank_gate: a power of %g", (double)inv_tau);
+    return lowrank_launch(x, ld, col, w_rows, w, dtype, out, n, N, R, LowRankTail{bias, inv_tau}, stream);
+}
+FL_RECORDABLE(fl_lowrank_gate)
 
 // What stands between the joined projection of a mixer with forget gates per key dim and its walk:
 // q = silu(q), f = lower + (1 - lower) * sigmoid(f + bias), both float, value by value.

@@ -11,9 +11,7 @@
 #define MG_NONE 0
 #define MG_SILU 1
 #define MG_CLAMPED 2
-struct MoeGate {
-    float alpha, limit, shift;
-};
+typedef GateConstants MoeGate;
 template <int GATE>
 __device__ __forceinline__ float moe_gate(const MoeGate& m, float g, float u) {
     if constexpr (GATE == MG_CLAMPED) return clamped_gate(g, u, m.alpha, m.limit, m.shift);

@@ -428,7 +428,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void attn_plain_kernel(
     const T* __restrict__ q, T* __restrict__ out, PagedCache cache,
     const int* __restrict__ positions, const int* __restrict__ tok_seq,
-    const int* __restrict__ block_table, int max_blocks, int nh, float scale, int window, float softcap) {
+    const int* __restrict__ block_table, int max_blocks, int nh, float scale, int window, float softcap, const float* __restrict__ sink) {
     __shared__ float s_m[4], s_l[4];
     __shared__ float s_acc[4][FL_PLAIN_MAX_HD];
     const int token = blockIdx.x, head = blockIdx.y;
@@ -489,7 +489,7 @@ __global__ __launch_bounds__(256) void attn_plain_kernel(
             ll += s_l[w] * f[w];
         }
         T* orow = out + ((size_t)token * nh + head) * hd;
-        const float inv = ll > 0.f ? 1.0f / ll : 0.f;
+        const float inv = sink ? softmax_factor_with_sink(mm, ll, sink[head]) : ll > 0.f ? 1.0f / ll : 0.f;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int d = lane + 64 * j;
@@ -509,7 +509,7 @@ extern "C" int fl_attn_max_head_dim(void) { return FL_PLAIN_MAX_HD; }
 static int attn_plain_launch(const void* q, void* out, const void* cache_base, int dtype,
                              const int* positions, const int* tok_seq, const int* block_table,
                              int max_blocks, int n, int nh, int nkv, int hd, int page_size,
-                             int n_pages, float scale, int window, float softcap, hipStream_t stream) {
+                             int n_pages, float scale, int window, float softcap, const float* sink, hipStream_t stream) {
     FL_CHECK(n >= 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attn: bad head counts %d/%d", nh, nkv);
     FL_CHECK(hd > 0 && hd <= FL_PLAIN_MAX_HD, "attn: head size %d not in 1..%d", hd, FL_PLAIN_MAX_HD);
     FL_CHECK(window >= 0, "attn: negative window");
@@ -517,9 +517,9 @@ static int attn_plain_launch(const void* q, void* out, const void* cache_base, i
     PagedCache c{(void*)cache_base, nkv, page_size, hd, n_pages};
     dim3 grid(n, nh);
     if (dtype == FL_F32)
-        attn_plain_kernel<float><<<grid, 256, 0, stream>>>((const float*)q, (float*)out, c, positions, tok_seq, block_table, max_blocks, nh, scale, window, softcap);
+        attn_plain_kernel<float><<<grid, 256, 0, stream>>>((const float*)q, (float*)out, c, positions, tok_seq, block_table, max_blocks, nh, scale, window, softcap, sink);
     else if (dtype == FL_BF16)
-        attn_plain_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)q, (bf16_t*)out, c, positions, tok_seq, block_table, max_blocks, nh, scale, window, softcap);
+        attn_plain_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)q, (bf16_t*)out, c, positions, tok_seq, block_table, max_blocks, nh, scale, window, softcap, sink);
     else
         FL_CHECK(false, "attn: unknown dtype %d", dtype);
     FL_LAUNCH_CHECK();
@@ -531,18 +531,19 @@ extern "C" int fl_attn_plain(const void* q, void* out, const void* cache_base, i
                              int max_blocks, int n, int nh, int nkv, int hd, int page_size,
                              int n_pages, float scale, int window, hipStream_t stream) {
     return attn_plain_launch(q, out, cache_base, dtype, positions, tok_seq, block_table, max_blocks, n, nh, nkv, hd, page_size,
-                             n_pages, scale, window, 0.f, stream);
+                             n_pages, scale, window, 0.f, nullptr, stream);
 }
 FL_RECORDABLE(fl_attn_plain)
 
-// the same with the scores capped: score <- softcap * tanh(score / softcap) before the softmax (softcap > 0)
+// the same with the scores capped, score <- softcap * tanh(score / softcap) before the softmax (softcap > 0; 0: as they
+// are), and with a sink per query head in the denominator (sink float [nh], or null)
 extern "C" int fl_attn_plain_capped(const void* q, void* out, const void* cache_base, int dtype,
                                     const int* positions, const int* tok_seq, const int* block_table,
                                     int max_blocks, int n, int nh, int nkv, int hd, int page_size,
-                                    int n_pages, float scale, int window, float softcap, hipStream_t stream) {
+                                    int n_pages, float scale, int window, float softcap, const float* sink, hipStream_t stream) {
     FL_CHECK(softcap >= 0.f, "attn: negative cap");
     return attn_plain_launch(q, out, cache_base, dtype, positions, tok_seq, block_table, max_blocks, n, nh, nkv, hd, page_size,
-                             n_pages, scale, window, softcap, stream);
+                             n_pages, scale, window, softcap, sink, stream);
 }
 FL_RECORDABLE(fl_attn_plain_capped)
 

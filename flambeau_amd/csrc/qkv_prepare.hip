@@ -4,8 +4,8 @@
 //     (x / sqrt(mean(x^2) + eps) * w over all heads at once), or none;
 //   * rotation of the first `rot` dims of every head from the step's table of cosines and sines, pairs
 //     (i, i + rot/2) ("half") or (2i, 2i + 1) ("interleaved");
-//   * every head of q and k divided by its root mean square after rotation, with no gain or with a gain per
-//     head dim that all heads of q (of k) share, or not;
+//   * every head of q and k divided by its root mean square, with no gain or with a gain per head dim that all heads
+//     of q (of k) share, after rotation or before it, or not;
 //   * values blended with those an earlier layer made for the same token,
 //     v <- (1 - lambda) v + lambda v_first, or kept as that first layer's for later ones;
 //   * q stored for the attention kernels, k and v stored into the paged cache at the token's position;
@@ -24,7 +24,7 @@ struct QkvPrepare {
     const int* positions; const int* tok_seq; const int* block_table; int max_blocks;
     int nh, D, Dv, hdp;
     int rot, interleaved; const float2* cs;
-    const float* qnorm_w; const float* knorm_w; int head_norm; float eps;
+    const float* qnorm_w; const float* knorm_w; int head_norm; float eps;      // head_norm: 0 none, 1 behind the rotation, 2 ahead of it
     const float* q_head_gain; const float* k_head_gain;   // [D] each, or null: the gain behind the heads' own norm
     float* v_first; int vmix_mode; const float* lambda;
     int write_cache;
@@ -85,7 +85,17 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(QkvPrepare a, T* __res
         const int src = (is_q ? a.col_q : a.col_k) + h * D;
         const float* gain = is_q ? a.qnorm_w : a.knorm_w;
         const float inv = is_q ? inv_q : inv_k;
-        auto value = [&](int d) { return gain ? at(src + d) * inv * gain[h * D + d] : at(src + d); };
+        const float* hg = is_q ? a.q_head_gain : a.k_head_gain;
+        float first_norm = 1.f;                           // the head's norm ahead of its rotation
+        if (a.head_norm == 2) {
+            float sq = 0.f;
+            for (int d = lane; d < D; d += 64) sq = fmaf(at(src + d), at(src + d), sq);
+            first_norm = 1.0f / sqrtf(wave_sum(sq) / (float)D + a.eps);
+        }
+        auto value = [&](int d) {
+            const float v = gain ? at(src + d) * inv * gain[h * D + d] : at(src + d);
+            return a.head_norm == 2 ? v * (hg ? first_norm * hg[d] : first_norm) : v;
+        };
         float r[4];
         float ss = 0.f;
 #pragma unroll
@@ -106,9 +116,8 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(QkvPrepare a, T* __res
             r[j] = v;
             ss = fmaf(v, v, ss);
         }
-        if (a.head_norm) {
+        if (a.head_norm == 1) {
             const float f = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
-            const float* hg = is_q ? a.q_head_gain : a.k_head_gain;
 #pragma unroll
             for (int j = 0; j < 4; ++j) r[j] *= (hg && lane + 64 * j < D) ? f * hg[lane + 64 * j] : f;
         }
@@ -152,6 +161,7 @@ extern "C" int fl_qkv_prepare(const float* proj, int ld, int col_q, int col_k, i
     FL_CHECK(ld >= col_q + nh * D && (col_k < 0 || (ld >= col_k + nkv * D && ld >= col_v + nkv * Dv)), "qkv_prepare: columns beyond rows %d wide", ld);
     FL_CHECK(col_k >= 0 || !write_cache, "qkv_prepare: a projection of queries alone writes no cache");
     FL_CHECK(col_k < 0 ? !knorm_w : !qnorm_w == !knorm_w, "qkv_prepare: the norm over the projection needs both gains");
+    FL_CHECK(head_norm >= 0 && head_norm <= 2 && !(head_norm == 2 && qnorm_w), "qkv_prepare: heads' norm %d (a norm ahead of the rotation stands alone)", head_norm);
     FL_CHECK(head_norm || (!q_head_gain && !k_head_gain), "qkv_prepare: a gain per head dim without the heads' norm");
     FL_CHECK(vmix_mode >= 0 && vmix_mode <= 2 && (vmix_mode == 0 || v_first) && (vmix_mode != 2 || lambda),
              "qkv_prepare: value blending %d without its buffers", vmix_mode);

@@ -197,28 +197,30 @@ FL_RECORDABLE(fl_norm_mix)
 // wider than Dv (padded); g: 0 none, 1 sigmoid, 2 silu.
 template <typename T>
 __global__ __launch_bounds__(256) void heads_gate_kernel(const T* __restrict__ x, int ldh, const float* __restrict__ gate, int ldg,
-                                                         int gate_col0, int kind, T* __restrict__ out, int H, int Dv) {
+                                                         int gate_col0, int kind, int per_head, float scale, T* __restrict__ out,
+                                                         int ldo, int H, int Dv) {
     const size_t t = blockIdx.x;
     for (int e = threadIdx.x; e < H * Dv; e += 256) {
         const int h = e / Dv, j = e - h * Dv;
-        float v = to_f32(x[(t * H + h) * ldh + j]);
+        float v = to_f32(x[(t * H + h) * ldh + j]) * scale;
         if (kind) {
-            const float z = gate[t * ldg + gate_col0 + e];
+            const float z = gate[t * ldg + gate_col0 + (per_head ? h : e)];
             v *= kind == 1 ? 1.0f / (1.0f + expf(-z)) : z / (1.0f + expf(-z));
         }
-        out[t * H * Dv + e] = from_f32<T>(v);
+        out[t * ldo + e] = from_f32<T>(v);
     }
 }
 
-extern "C" int fl_heads_gate(const void* x, int dtype, int ldh, const float* gate, int ldg, int gate_col0, int kind, void* out,
-                             int n, int H, int Dv, hipStream_t stream) {
+extern "C" int fl_heads_gate(const void* x, int dtype, int ldh, const float* gate, int ldg, int gate_col0, int kind, int per_head,
+                             float scale, void* out, int ldo, int n, int H, int Dv, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && Dv > 0 && ldh >= Dv, "heads_gate: bad sizes");
-    FL_CHECK(kind >= 0 && kind <= 2 && (kind == 0 || (gate && ldg >= gate_col0 + H * Dv)), "heads_gate: gate %d over rows %d wide", kind, ldg);
+    FL_CHECK(kind >= 0 && kind <= 2 && (kind == 0 || (gate && ldg >= gate_col0 + (per_head ? H : H * Dv))), "heads_gate: gate %d over rows %d wide", kind, ldg);
+    FL_CHECK(ldo >= H * Dv, "heads_gate: output rows of %d values for %d heads of %d", ldo, H, Dv);
     if (n == 0) return 0;
     if (dtype == FL_F32)
-        heads_gate_kernel<float><<<n, 256, 0, stream>>>((const float*)x, ldh, gate, ldg, gate_col0, kind, (float*)out, H, Dv);
+        heads_gate_kernel<float><<<n, 256, 0, stream>>>((const float*)x, ldh, gate, ldg, gate_col0, kind, per_head, scale, (float*)out, ldo, H, Dv);
     else if (dtype == FL_BF16)
-        heads_gate_kernel<bf16_t><<<n, 256, 0, stream>>>((const bf16_t*)x, ldh, gate, ldg, gate_col0, kind, (bf16_t*)out, H, Dv);
+        heads_gate_kernel<bf16_t><<<n, 256, 0, stream>>>((const bf16_t*)x, ldh, gate, ldg, gate_col0, kind, per_head, scale, (bf16_t*)out, ldo, H, Dv);
     else
         FL_CHECK(false, "heads_gate: unknown dtype %d", dtype);
     FL_LAUNCH_CHECK();

@@ -148,3 +148,13 @@ class Runtime:
         gu = self.buffer("ffn_gate_up", x.shape[0], w.rows, torch.float32)
         ops.gemm_plain(x, w.rowmajor, gu)
         return ops.silu_mul(gu, out) if gate == "silu" else ops.gated_act(gu, out, gate)
+
+    def gemm_clamped(self, x, w, out, alpha: float, limit: float, shift: float):
+        """``gemm_swiglu`` with the clamped gate: ``out = g sigmoid(alpha g) (u + shift)``, g = min(x Wg^T, limit),
+        u = x Wu^T within +-limit."""
+        if self.tuned:
+            from ..kernels import tuned
+            return tuned.gemm_clamped(x, w, out, self, alpha, limit, shift)
+        gu = self.buffer("ffn_gate_up", x.shape[0], w.rows, torch.float32)
+        ops.gemm_plain(x, w.rowmajor, gu)
+        return ops.clamped_gate(gu, out, alpha, limit, shift)

@@ -30,14 +30,15 @@ class PlainLatentAttention:
     def prepare(self, uk, uv, n_heads) -> LatentWeights:
         return LatentWeights(uk, uv, n_heads)
 
-    def attend(self, q, w: LatentWeights, cache, step, table, scale, window, gate, gate_col0, out, rotated=None):
+    def attend(self, q, w: LatentWeights, cache, step, table, scale, window, gate, gate_col0, out, rotated=None, sink=None):
         """``q`` float32 ``[n, H * (D + rotated dims)]`` -> ``out [n, H * Dv]`` (compute dtype): fold, attend, expand
-        and gate.  ``rotated`` (``ops.RotatedPart``): what a head's folded query carries behind the latent's values."""
+        and gate.  ``rotated`` (``ops.RotatedPart``): what a head's folded query carries behind the latent's values;
+        ``sink`` (float32 ``[H]``): a score per head that joins the softmax's denominator once."""
         rt, n, H = self.rt, q.shape[0], w.n_heads
         qa = rt.buffer("la_qa", n, H * cache.width, torch.float32)
         ops.heads_matmul(q, w.uk, qa, H, transposed=False, rotated=rotated)
         z = rt.buffer("la_z", n, H * cache.value_width, torch.float32)
-        ops.latent_attention(qa, z, cache, step.positions, step.tok_seq, table, H, scale, window)
+        ops.latent_attention(qa, z, cache, step.positions, step.tok_seq, table, H, scale, window, sink=sink)
         return ops.heads_matmul(z, w.uv, out, H, transposed=True, gate=gate, gate_col0=gate_col0)
 
     def signature(self, batch, n_heads: int, window: int = 0):
@@ -99,7 +100,7 @@ class TunedLatentAttention(PlainLatentAttention):
             w.uk_by_head = uk.view(n_heads, D, R).transpose(1, 2).contiguous()
         return w
 
-    def attend(self, q, w, cache, step, table, scale, window, gate, gate_col0, out, rotated=None):
+    def attend(self, q, w, cache, step, table, scale, window, gate, gate_col0, out, rotated=None, sink=None):
         rt, n, H, R = self.rt, q.shape[0], w.n_heads, cache.value_width
         rank, Dv = w.uk.shape[1], out.shape[1] // H
         lib = load()
@@ -115,7 +116,7 @@ class TunedLatentAttention(PlainLatentAttention):
         few = bool(window) and n * -(-H // 16) <= DEALT_UNITS
         if on_cores and tiles is not None and n_split == 1 and not few:
             # a step of many rows (prompt portions): blocks of four waves share every chunk of keys through LDS
-            latent_attention_shared(qa, z, cache, step.positions, step.tok_seq, table, H, scale, window, tiles)
+            latent_attention_shared(qa, z, cache, step.positions, step.tok_seq, table, H, scale, window, tiles, sink=sink)
         elif on_cores:
             part_o = part_ml = None
             if n_split > 1:
@@ -123,9 +124,9 @@ class TunedLatentAttention(PlainLatentAttention):
                 part_o = rt.buffer("la_part_o", rows, R, torch.float32, max_rows=16 * (SPLIT_TARGET_WAVES + 64))
                 part_ml = rt.buffer("la_part_ml", rows, 2, torch.float32, max_rows=16 * (SPLIT_TARGET_WAVES + 64))
             latent_attention_mfma(qa, z, cache, step.positions, step.tok_seq, table, H, scale, window, n_split, part_o, part_ml,
-                                  dealt=True)
+                                  dealt=True, sink=sink)
         else:
-            ops.latent_attention(qa, z, cache, step.positions, step.tok_seq, table, H, scale, window)
+            ops.latent_attention(qa, z, cache, step.positions, step.tok_seq, table, H, scale, window, sink=sink)
         if w.uv.dtype == torch.bfloat16 and lib.fl_heads_matmul_mfma_takes(rank, Dv):
             return heads_matmul_mfma(z, w.uv.view(H, Dv, rank), out, H, gate=gate, gate_col0=gate_col0)
         return ops.heads_matmul(z, w.uv, out, H, transposed=True, gate=gate, gate_col0=gate_col0)
@@ -147,7 +148,7 @@ def heads_matmul_mfma(x, w, out, n_heads, gate=None, gate_col0=0, rotated=None):
 
 
 def latent_attention_mfma(qa, z, cache, positions, tok_seq, block_table, n_heads, scale, window=0, n_split=1,
-                          part_o=None, part_ml=None, dealt=False):
+                          part_o=None, part_ml=None, dealt=False, sink=None):
     """``dealt``: the form with a block of four waves per (token, 16 heads, part of the keys), for steps of few rows
     (else one wave each).  ``n_split`` > 1: every token's keys are dealt out to that many waves; ``part_o`` (float32, at least
     ``n * ceil(H / 16) * n_split * 16`` rows of R) and ``part_ml`` (as many rows of 2) hold their sums."""
@@ -165,11 +166,12 @@ def latent_attention_mfma(qa, z, cache, positions, tok_seq, block_table, n_heads
          ops._check(tok_seq, "latent_attention.tok_seq", torch.int32, (n,)),
          ops._check(block_table, "latent_attention.block_table", torch.int32, (None, None)), block_table.shape[1],
          n, int(n_heads), K, R, cache.page_size, cache.n_pages, float(scale), int(window), int(n_split),
-         part_o.data_ptr() if n_split > 1 else None, part_ml.data_ptr() if n_split > 1 else None, ops.stream_handle())
+         part_o.data_ptr() if n_split > 1 else None, part_ml.data_ptr() if n_split > 1 else None,
+         ops._check(sink, "latent_attention.sink", torch.float32, (n_heads,)) if sink is not None else None, ops.stream_handle())
     return z
 
 
-def latent_attention_shared(qa, z, cache, positions, tok_seq, block_table, n_heads, scale, window, tiles):
+def latent_attention_shared(qa, z, cache, positions, tok_seq, block_table, n_heads, scale, window, tiles, sink=None):
     """The matrix-core kernel whose blocks share their keys; ``tiles``: ``shared_tiles`` on the device."""
     n, K, R = qa.shape[0], cache.width, cache.value_width
     call("fl_latent_attention_shared", ops._check(qa, "latent_attention.qa", torch.bfloat16, (n, n_heads * K)),
@@ -179,7 +181,8 @@ def latent_attention_shared(qa, z, cache, positions, tok_seq, block_table, n_hea
          ops._check(tok_seq, "latent_attention.tok_seq", torch.int32, (n,)),
          ops._check(block_table, "latent_attention.block_table", torch.int32, (None, None)), block_table.shape[1],
          int(n_heads), K, R, cache.page_size, cache.n_pages, float(scale), int(window),
-         ops._check(tiles, "latent_attention.tiles", torch.int32, (None, 4)), tiles.shape[0], ops.stream_handle())
+         ops._check(tiles, "latent_attention.tiles", torch.int32, (None, 4)), tiles.shape[0],
+         ops._check(sink, "latent_attention.sink", torch.float32, (n_heads,)) if sink is not None else None, ops.stream_handle())
     return z
 
 

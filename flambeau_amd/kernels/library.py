@@ -33,13 +33,13 @@ _SIGNATURES = {
     "fl_sample_bias": [P, I, I, P, P, P, P],
     "fl_sample_count": [P, I, I, P, P, P],
     "fl_sample_history": [P, I, I, P, I, P],
-    "fl_latent_prepare": [P, I, I, P, P, I, I, P, F, I, I, P, P, I, I, I, I, P, P, P, I, I, I, I, P],
-    "fl_heads_matmul": [P, I, I, P, I, P, I, I, I, I, I, I, I, P, I, I, I, I, P, I, P],
-    "fl_latent_attention": [P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, P],
-    "fl_latent_attention_mfma": [P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, P, P],
-    "fl_latent_attention_dealt": [P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, P, P],
-    "fl_latent_attention_shared": [P, P, P, P, P, P, I, I, I, I, I, I, F, I, P, I, P],
-    "fl_heads_matmul_mfma": [P, I, I, I, P, P, I, I, I, I, I, I, P, I, I, I, I, P, I, P],
+    "fl_latent_prepare": [P, I, I, P, P, I, I, P, F, I, I, I, P, P, I, I, I, I, P, P, P, I, I, I, I, P],
+    "fl_heads_matmul": [P, I, I, P, I, P, I, I, I, I, I, I, I, P, I, I, I, I, I, P, I, P],
+    "fl_latent_attention": [P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, P, P],
+    "fl_latent_attention_mfma": [P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, P, P, P],
+    "fl_latent_attention_dealt": [P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, P, P, P],
+    "fl_latent_attention_shared": [P, P, P, P, P, P, I, I, I, I, I, I, F, I, P, I, P, P],
+    "fl_heads_matmul_mfma": [P, I, I, I, P, P, I, I, I, I, I, I, P, I, I, I, I, I, P, I, P],
     "fl_sublayer_step": [P, P, I, P, P, I, P, P, P, F, P, I, P, P, F, P, I, I, I, P],
     "fl_input_conv": [P, I, P, P, P, P, P, P, P, P, I, I, I, P],
     "fl_embed_bigram": [P, P, I, P, P, P, P, P, P, P, P, I, I, I, I, L, L, P],
@@ -54,12 +54,12 @@ _SIGNATURES = {
     "fl_activation": [P, P, I, L, I, P],
     "fl_concat_cast": [P, P, P, I, I, I, P],
     "fl_add_rowvec": [P, P, I, I, P],
-    "fl_attn_plain_capped": [P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, F, P],
+    "fl_attn_plain_capped": [P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, F, P, P],
     "fl_dyt": [P, P, P, P, P, P, P, P, I, I, I, P],
     "fl_embed_scaled": [P, I, P, P, I, I, I, F, P],
     "fl_gated_act": [P, P, I, I, I, I, P],
     "fl_norm_mix": [P, P, F, P, P, F, P, I, I, F, P],
-    "fl_heads_gate": [P, I, I, P, I, I, I, P, I, I, I, P],
+    "fl_heads_gate": [P, I, I, P, I, I, I, I, F, P, I, I, I, I, P],
     "fl_qkv_prepare": [P, I, I, I, I, P, P, P, I, P, P, I, I, I, I, I, I, I, I, I, I, I, P, P, P, I, P, P, F, P, I, P, I, P, P, P],
     "fl_linear_scan": [P, I, P, I, P, I, P, P, P, I, P, L, P, P, P, P, I, I, I, I, I, P],
     "fl_conv_prepare": [P, I, I, I, I, P, P, P, P, L, P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, P],
@@ -83,6 +83,11 @@ _SIGNATURES = {
     "fl_hyper_spread": [P, P, I, I, I, P],
     "fl_scaled_sum": [P, F, P, F, P, L, P],
     "fl_softcap_inplace": [P, L, F, P],
+    "fl_linear_scan_gated": [P, I, P, I, P, I, P, I, F, P, L, P, P, P, P, I, I, I, I, I, P],
+    "fl_linear_scan_written": [P, I, P, I, P, I, P, P, I, P, P, L, P, P, P, P, I, I, I, I, I, P],
+    "fl_lowrank_gate": [P, I, I, P, P, I, P, F, P, I, I, I, P],
+    "fl_conv_steps": [P, I, I, P, P, P, L, P, P, P, P, P, P, I, I, I, I, I, P, P, P, P],
+    "fl_gated_group_norm": [P, P, I, I, P, P, I, I, I, I, I, F, P],
 }
 
 

@@ -179,18 +179,21 @@ def rope_kv_write(qkv, positions, tok_seq, block_table, q_out, cache: PagedLayer
     return q_out
 
 
-def attn_plain(q, out, cache: PagedLayerCache, positions, tok_seq, block_table, n_heads, scale, window, softcap: float = 0.0):
-    """``softcap`` > 0: scores are capped, ``softcap * tanh(score / softcap)``, before the softmax."""
+def attn_plain(q, out, cache: PagedLayerCache, positions, tok_seq, block_table, n_heads, scale, window, softcap: float = 0.0, sink=None):
+    """``softcap`` > 0: scores are capped, ``softcap * tanh(score / softcap)``, before the softmax; ``sink`` (float32
+    ``[n_heads]``): a score per query head that joins the softmax's denominator once."""
     n = q.shape[0]
     hd = cache.head_dim
     dt = cache.pool.dtype
-    call("fl_attn_plain_capped" if softcap else "fl_attn_plain", _check(q, "attn.q", dt, (n, n_heads * hd)),
+    extras = bool(softcap) or sink is not None
+    call("fl_attn_plain_capped" if extras else "fl_attn_plain", _check(q, "attn.q", dt, (n, n_heads * hd)),
          _check(out, "attn.out", dt, (n, n_heads * hd)), _check(cache.pool, "attn.cache"),
          dtype_code(dt), _check(positions, "attn.positions", torch.int32, (n,)),
          _check(tok_seq, "attn.tok_seq", torch.int32, (n,)),
          _check(block_table, "attn.block_table", torch.int32, (None, None)), block_table.shape[1],
          n, n_heads, cache.n_kv_heads, hd, cache.page_size, cache.n_pages, float(scale), int(window),
-         *((float(softcap),) if softcap else ()), stream_handle())
+         *((float(softcap), _check(sink, "attn.sink", torch.float32, (n_heads,)) if sink is not None else None) if extras else ()),
+         stream_handle())
     return out
 
 
@@ -307,16 +310,17 @@ class LatentLayerCache:
 
 
 def latent_prepare(low, q_width, q_gain, q_out, kv_col, kv_rank, kv_gain, eps, cache: LatentLayerCache, positions, tok_seq, block_table,
-                   rot_dim=0, rotated_dims=0, angles=None, write_cache=True):
+                   rot_dim=0, rotated_dims=0, angles=None, write_cache=True, interleaved=False):
     """From the float32 rows ``low`` of a joined projection: ``q_out = rmsnorm(low[:, :q_width]) * q_gain`` and, with
     ``write_cache``, the tokens' rows in their pages: ``rmsnorm(low[:, kv_col : kv_col + kv_rank]) * kv_gain`` and the
-    ``rot_dim`` columns behind it turned by ``angles`` ``[n, rotated_dims / 2, 2]``."""
+    ``rot_dim`` columns behind it turned by ``angles`` ``[n, rotated_dims / 2, 2]``, dimension i with i + rotated_dims / 2 or
+    (``interleaved``) 2i with 2i + 1."""
     n, ld = low.shape
     dt = q_out.dtype
     call("fl_latent_prepare", _check(low, "latent_prepare.low", torch.float32), ld, int(q_width),
          _check(q_gain, "latent_prepare.q_gain", torch.float32, (q_width,)), _check(q_out, "latent_prepare.q_out", None, (n, q_width)),
          int(kv_col), int(kv_rank), _check(kv_gain, "latent_prepare.kv_gain", torch.float32, (kv_rank,)), float(eps), int(rot_dim),
-         int(rotated_dims), _check(angles, "latent_prepare.angles", torch.float32, (n, rotated_dims // 2, 2)) if rotated_dims else None,
+         int(rotated_dims), int(bool(interleaved)), _check(angles, "latent_prepare.angles", torch.float32, (n, rotated_dims // 2, 2)) if rotated_dims else None,
          _check(cache.pool, "latent_prepare.pool", dt), dtype_code(dt), cache.width, cache.value_width, n,
          _check(positions, "latent_prepare.positions", torch.int32, (n,)), _check(tok_seq, "latent_prepare.tok_seq", torch.int32, (n,)),
          _check(block_table, "latent_prepare.block_table", torch.int32, (None, None)), block_table.shape[1],
@@ -332,13 +336,14 @@ class RotatedPart:
     rotated: int
     angles: torch.Tensor | None
     at: int
+    interleaved: bool = False       # dimension 2i turns with 2i + 1, else i with i + rotated / 2
 
     def args(self, n):
-        return (int(self.dim), int(self.rotated),
+        return (int(self.dim), int(self.rotated), int(bool(self.interleaved)),
                 _check(self.angles, "rotated_part.angles", torch.float32, (n, self.rotated // 2, 2)) if self.rotated else None, int(self.at))
 
 
-NO_ROTATED_PART = (0, 0, None, 0)
+NO_ROTATED_PART = (0, 0, 0, None, 0)
 
 
 def heads_matmul(x, w, out, n_heads, transposed, gate=None, gate_col0=0, rotated: RotatedPart | None = None):
@@ -364,8 +369,9 @@ def latent_max_width() -> int:
     return load().fl_latent_max_width()
 
 
-def latent_attention(qa, z, cache: LatentLayerCache, positions, tok_seq, block_table, n_heads, scale, window=0):
-    """``z[t, h] = sum_j softmax_j(scale * qa[t, h] . row_j) value_j`` over the cached rows of the token's request."""
+def latent_attention(qa, z, cache: LatentLayerCache, positions, tok_seq, block_table, n_heads, scale, window=0, sink=None):
+    """``z[t, h] = sum_j softmax_j(scale * qa[t, h] . row_j) value_j`` over the cached rows of the token's request; ``sink``
+    (float32 ``[n_heads]``): a score per head that joins the softmax's denominator once."""
     n = qa.shape[0]
     K, R = cache.width, cache.value_width
     call("fl_latent_attention", _check(qa, "latent_attention.qa", torch.float32, (n, n_heads * K)),
@@ -373,7 +379,8 @@ def latent_attention(qa, z, cache: LatentLayerCache, positions, tok_seq, block_t
          dtype_code(cache.pool.dtype), _check(positions, "latent_attention.positions", torch.int32, (n,)),
          _check(tok_seq, "latent_attention.tok_seq", torch.int32, (n,)),
          _check(block_table, "latent_attention.block_table", torch.int32, (None, None)), block_table.shape[1],
-         n, int(n_heads), K, R, cache.page_size, cache.n_pages, float(scale), int(window), stream_handle())
+         n, int(n_heads), K, R, cache.page_size, cache.n_pages, float(scale), int(window),
+         _check(sink, "latent_attention.sink", torch.float32, (n_heads,)) if sink is not None else None, stream_handle())
     return z
 
 
@@ -563,15 +570,24 @@ def norm_mix(a, weight_a, factor_a, b, weight_b, factor_b, out, eps):
 HEAD_GATES = {None: 0, "sigmoid": 1, "silu": 2}
 
 
-def heads_gate(x, head_stride, gate, gate_col0, kind, out, n_heads):
-    """``out[t, h, j] = x[t, h, j] * g(gate[t, gate_col0 + h * Dv + j])`` for ``j < Dv``; the heads of ``x`` are
-    ``head_stride`` wide (padded), those of ``out`` ``Dv``.  ``kind``: ``None``, ``sigmoid`` or ``silu``."""
+def _out_columns(t, name, n, width):
+    """``(address, row stride)`` of a ``[n, width]`` tensor or of such columns of a wider one."""
+    if not isinstance(t, torch.Tensor) or not t.is_cuda or t.dim() != 2 or t.shape != (n, width) or t.stride(1) != 1:
+        raise KernelError(f"{name}: want [{n}, {width}] on the device with unit stride along a row, got {tuple(getattr(t, 'shape', ()))}")
+    return t.data_ptr(), t.stride(0) if n > 1 else max(t.stride(0), width)
+
+
+def heads_gate(x, head_stride, gate, gate_col0, kind, out, n_heads, per_head: bool = False, scale: float = 1.0):
+    """``out[t, h, j] = scale * x[t, h, j] * g(gate[t, gate_col0 + h * Dv + j])`` for ``j < Dv`` (``per_head``: one logit per
+    head, ``gate[t, gate_col0 + h]``); the heads of ``x`` are ``head_stride`` wide (padded), those of ``out`` (which may be
+    columns of a wider tensor) ``Dv``.  ``kind``: ``None``, ``sigmoid`` or ``silu``."""
     n = x.shape[0]
     Dv = out.shape[1] // n_heads
+    po, ldo = _out_columns(out, "heads_gate.out", n, n_heads * Dv)
     call("fl_heads_gate", _check(x, "heads_gate.x", out.dtype, (n, n_heads * head_stride)), dtype_code(x.dtype), int(head_stride),
          _check(gate, "heads_gate.gate", torch.float32, (n, None)) if gate is not None else None,
          gate.shape[1] if gate is not None else 0, int(gate_col0), HEAD_GATES[kind if gate is not None else None],
-         _check(out, "heads_gate.out", None, (n, n_heads * Dv)), n, int(n_heads), Dv, stream_handle())
+         int(bool(per_head)), float(scale), po, ldo, n, int(n_heads), Dv, stream_handle())
     return out
 
 
@@ -581,7 +597,7 @@ def qkv_prepare(proj, cols, positions, tok_seq, block_table, q_out, cache: Paged
     """From the float32 rows of a joined projection (q, k, v at the columns ``cols``) to the rotated, normed
     queries in ``q_out`` and the token's keys and values in the cache, heads stored ``cache.head_dim`` wide.
     ``q_gain`` / ``k_gain``: gains of a norm over the whole projection of q and of k (before rotation);
-    ``head_norm``: every head divided by its root mean square after rotation, times ``q_head_gain`` / ``k_head_gain``
+    ``head_norm``: every head divided by its root mean square after rotation (``True`` or 1) or before it (2), times ``q_head_gain`` / ``k_head_gain``
     (float32 ``[dim]``, one gain per head dim that all heads share) where given; ``bias``: float32, one value per column of
     ``proj``, added to the projection as it is read (the projections' biases); ``value_mix``: 1 keeps the
     values in ``v_first``, 2 blends them with it by the device scalar ``mix``; ``row_scales``: float32 ``[n, 2]`` of
@@ -600,7 +616,7 @@ def qkv_prepare(proj, cols, positions, tok_seq, block_table, q_out, cache: Paged
          _check(table, "qkv_prepare.table", torch.float32, (n, half, 2)) if rotated_dims else None,
          _check(q_gain, "qkv_prepare.q_gain", torch.float32, (n_heads * dim,)) if q_gain is not None else None,
          _check(k_gain, "qkv_prepare.k_gain", torch.float32, (nkv * dim,)) if k_gain is not None else None,
-         int(bool(head_norm)),
+         int(head_norm),
          _check(q_head_gain, "qkv_prepare.q_head_gain", torch.float32, (dim,)) if q_head_gain is not None else None,
          _check(k_head_gain, "qkv_prepare.k_head_gain", torch.float32, (dim,)) if k_head_gain is not None else None, float(eps),
          _check(v_first, "qkv_prepare.v_first", torch.float32, (n, nkv * vdim)) if v_first is not None else None, int(value_mix),
@@ -669,6 +685,72 @@ def linear_scan(q, k, v, state, seq_q_start, seq_q_len, seq_slots, out, n_heads,
          _check(seq_q_start, "linear_scan.seq_q_start", torch.int32, (S,)), _check(seq_q_len, "linear_scan.seq_q_len", torch.int32, (S,)),
          _check(seq_slots, "linear_scan.seq_slots", torch.int32, (S,)), _check(out, "linear_scan.out", torch.float32, (n, n_heads * vdim)),
          S, int(n_heads), int(n_qk_heads), int(dim), int(vdim), stream_handle())
+    return out
+
+
+def _rows(t, name, n, width):
+    """``(address, row stride)`` of float32 rows, which may be columns of wider ones."""
+    if t.dtype != torch.float32 or not t.is_cuda or t.dim() != 2 or t.shape != (n, width) or t.stride(1) != 1:
+        raise KernelError(f"{name}: {t.dtype} {tuple(t.shape)}, want float32 [{n}, {width}] with unit stride")
+    return t.data_ptr(), t.stride(0) if n > 1 else max(t.stride(0), width)
+
+
+def linear_scan_gated(q, k, v, key_decay, state, step, out, n_heads, n_qk_heads, dim, vdim, out_scale: float = 1.0):
+    """``linear_scan`` with a decay per token, head and key dim and no correction: S <- diag(g) S + k v^T,
+    o = ``out_scale`` S^T q; ``key_decay`` float32 ``[n, n_heads * dim]``; ``step``: the batch's metadata."""
+    n, S = out.shape[0], step.seq_q_start.shape[0]
+    i = lambda t, name: _check(t, "linear_scan_gated." + name, torch.int32, (S,))
+    call("fl_linear_scan_gated", *_rows(q, "linear_scan_gated.q", n, n_qk_heads * dim), *_rows(k, "linear_scan_gated.k", n, n_qk_heads * dim),
+         *_rows(v, "linear_scan_gated.v", n, n_heads * vdim), *_rows(key_decay, "linear_scan_gated.key_decay", n, n_heads * dim), float(out_scale),
+         _check(state, "linear_scan_gated.state", torch.float32, (None, None)), state.shape[1], i(step.seq_q_start, "seq_q_start"),
+         i(step.seq_q_len, "seq_q_len"), i(step.seq_slots, "seq_slots"), _check(out, "linear_scan_gated.out", torch.float32, (n, n_heads * vdim)),
+         S, int(n_heads), int(n_qk_heads), int(dim), int(vdim), stream_handle())
+    return out
+
+
+def linear_scan_written(q, k, v, gates, skip, state, step, out, n_heads, n_qk_heads, dim, vdim):
+    """``linear_scan`` with a decay and a write strength per token and head and no correction: S <- g S + w k v^T,
+    o = S^T q + ``skip[h]`` v; ``gates`` float32 ``[n, 2 * n_heads]`` (decay, then write strength)."""
+    n, S = out.shape[0], step.seq_q_start.shape[0]
+    i = lambda t, name: _check(t, "linear_scan_written." + name, torch.int32, (S,))
+    pg = _check(gates, "linear_scan_written.gates", torch.float32, (n, 2 * n_heads))
+    call("fl_linear_scan_written", *_rows(q, "linear_scan_written.q", n, n_qk_heads * dim), *_rows(k, "linear_scan_written.k", n, n_qk_heads * dim),
+         *_rows(v, "linear_scan_written.v", n, n_heads * vdim), pg, pg + 4 * n_heads, 2 * n_heads,
+         _check(skip, "linear_scan_written.skip", torch.float32, (n_heads,)) if skip is not None else None,
+         _check(state, "linear_scan_written.state", torch.float32, (None, None)), state.shape[1], i(step.seq_q_start, "seq_q_start"),
+         i(step.seq_q_len, "seq_q_len"), i(step.seq_slots, "seq_slots"), _check(out, "linear_scan_written.out", torch.float32, (n, n_heads * vdim)),
+         S, int(n_heads), int(n_qk_heads), int(dim), int(vdim), stream_handle())
+    return out
+
+
+def conv_steps(proj, col0, weight, bias, state, ring_at, step, out, col_dt, n_heads, dt_bias, a_log, gates):
+    """A causal convolution over time per channel (columns ``col0`` on of the float32 rows ``proj``; ``weight`` float32
+    ``[taps, C]``, ``bias`` ``[C]``) with silu behind it, into ``out`` ``[n, C]``; and per head dt = softplus(proj[:, col_dt + h] +
+    dt_bias[h]) and the decay exp(-exp(a_log[h]) dt), into ``gates`` ``[n, 2 * heads]`` (decay, then dt).  A request's last inputs
+    live at ``ring_at`` floats into its record of ``state`` ``[slots, floats]`` (position p at ``p % taps``)."""
+    n, ld = proj.shape
+    taps, C = weight.shape
+    S = step.seq_q_start.shape[0]
+    if state.dim() != 2 or not state.is_contiguous() or state.shape[1] < ring_at + taps * C:
+        raise KernelError(f"conv_steps.state: shape {tuple(state.shape)} does not hold {taps} x {C} floats at {ring_at}")
+    f = lambda t, name, shape: _check(t, "conv_steps." + name, torch.float32, shape)
+    i = lambda t, name, k: _check(t, "conv_steps." + name, torch.int32, (k,))
+    call("fl_conv_steps", f(proj, "proj", None), ld, int(col0), f(weight, "weight", (taps, C)), f(bias, "bias", (C,)) if bias is not None else None,
+         f(state, "state", None) + 4 * int(ring_at), state.shape[1], i(step.positions, "positions", n), i(step.tok_seq, "tok_seq", n),
+         i(step.seq_q_start, "seq_q_start", S), i(step.seq_q_len, "seq_q_len", S), i(step.seq_slots, "seq_slots", S), f(out, "out", (n, C)), n, C,
+         taps, int(col_dt), int(n_heads), f(dt_bias, "dt_bias", (n_heads,)), f(a_log, "a_log", (n_heads,)), f(gates, "gates", (n, 2 * n_heads)),
+         stream_handle())
+    return out
+
+
+def gated_group_norm(y, gate, gate_col0, weight, out, parts, eps):
+    """``v = y * silu(gate[:, gate_col0 :])``, divided by its root mean square in ``parts`` equal parts, times ``weight``; ``out``
+    may be columns of a wider tensor."""
+    n, W = y.shape
+    po, ldo = _out_columns(out, "gated_group_norm.out", n, W)
+    call("fl_gated_group_norm", _check(y, "gated_group_norm.y", torch.float32), _check(gate, "gated_group_norm.gate", torch.float32, (n, None)),
+         gate.shape[1], int(gate_col0), _check(weight, "gated_group_norm.weight", torch.float32, (W,)), po, dtype_code(out.dtype), ldo, n, W,
+         int(parts), float(eps), stream_handle())
     return out
 
 
@@ -854,6 +936,18 @@ def lowrank_expand(x, col, w, wt, out):
         raise KernelError(f"lowrank_expand: a factor {tuple(w.shape)} with a transposed copy {tuple(wt.shape)}")
     call("fl_lowrank_expand", _check(x, "lowrank_expand.x", torch.float32), ld, int(col), _check(w, "lowrank_expand.w"), _check(wt, "lowrank_expand.wt"), dtype_code(w.dtype),
          _check(out, "lowrank_expand.out", torch.float32, (n, N)), n, N, R, stream_handle())
+    return out
+
+
+def lowrank_gate(x, col, w, wt, bias, tau: float, out):
+    """``lowrank_expand`` with a forget gate behind it: ``out = sigmoid(sum + bias)^(1 / tau)``, all in 32-bit."""
+    n, ld = x.shape
+    N, R = w.shape
+    if wt.shape != (R, N) or wt.dtype != w.dtype:
+        raise KernelError(f"lowrank_gate: a factor {tuple(w.shape)} with a transposed copy {tuple(wt.shape)}")
+    call("fl_lowrank_gate", _check(x, "lowrank_gate.x", torch.float32), ld, int(col), _check(w, "lowrank_gate.w"), _check(wt, "lowrank_gate.wt"),
+         dtype_code(w.dtype), _check(bias, "lowrank_gate.bias", torch.float32, (N,)) if bias is not None else None, 1.0 / float(tau),
+         _check(out, "lowrank_gate.out", torch.float32, (n, N)), n, N, R, stream_handle())
     return out
 
 

@@ -48,8 +48,11 @@ register_signatures({
     "fl_gemm_skinny_dyt": [P, P, I, I, I, P, P, P, P, P, P],
     "fl_gemm_tiled_dyt": [P, P, I, I, I, P, P, P, P, P, P],
     "fl_reduce_dyt": [P, P, P, P, P, P, I, I, I, P],
-    "fl_attn_decode_items_capped": [P, P, P, P, P, P, I, P, I, I, I, I, I, I, F, I, F, P, I, P],
-    "fl_attn_prefill_capped": [P, P, P, P, I, P, P, I, I, I, I, I, I, F, I, F, I, P, P, I, P],
+    "fl_attn_decode_items_capped": [P, P, P, P, P, P, I, P, I, I, I, I, I, I, F, I, F, P, P, I, P],
+    "fl_attn_prefill_capped": [P, P, P, P, I, P, P, I, I, I, I, I, I, F, I, F, P, I, P, P, I, P],
+    "fl_gemm_skinny_clamped": [P, P, P, I, I, I, I, I, F, F, F, P],
+    "fl_gemm_mid_clamped": [P, P, P, I, I, I, I, I, F, F, F, P],
+    "fl_gemm_tiled_clamped": [P, P, P, I, I, I, I, I, F, F, F, P],
 })
 
 SKINNY_MAX_ROWS = 64     # rows the decode kernels take
@@ -542,6 +545,27 @@ def gemm_swiglu(x, w: Weight, out, rt, gate: str = "silu"):
     return ops.silu_mul(gu, out) if gate == "silu" else ops.gated_act(gu, out, gate)
 
 
+def gemm_clamped(x, w: Weight, out, rt, alpha: float, limit: float, shift: float):
+    """``out = g sigmoid(alpha g) (u + shift)``, g = min(x Wg^T, limit), u = x Wu^T within +-limit; ``w`` comes from
+    ``prepare_gate_up``."""
+    M, K = x.shape
+    if w.packed is not None and w.swiglu_cols and x.dtype == torch.bfloat16 and K % 8 == 0:
+        if SKINNY_BEST_ROWS < M <= SKINNY_MAX_ROWS and K % 32 == 0:
+            name = "fl_gemm_mid_clamped"
+        else:
+            name = "fl_gemm_skinny_clamped" if M <= SKINNY_MAX_ROWS else "fl_gemm_tiled_clamped"
+        N = w.packed_rows
+        if w.packed.numel() != _packed_size(N, K):
+            raise KernelError(f"gemm.w: packed matrix of {w.packed.numel()} values, a [{N}, {K}] matrix packs to {_packed_size(N, K)}")
+        call(name, _check(x, "gemm.x", torch.bfloat16, (M, K)), _check(w.packed, "gemm.w", torch.bfloat16),
+             _check(out, "gemm.out", None, (M, w.swiglu_cols)), dtype_code(out.dtype), M, N, K, w.swiglu_cols, float(alpha), float(limit),
+             float(shift), stream_handle())
+        return out
+    gu = rt.buffer("ffn_gate_up", M, w.rows, torch.float32)
+    ops.gemm_plain(x, w.rowmajor, gu)
+    return ops.clamped_gate(gu, out, alpha, limit, shift)
+
+
 def prepare_weight(w: torch.Tensor) -> Weight:
     """The form of a weight matrix the tuned path wants: packed tiles when the kernels take the
     shape (the row-major matrix is dropped then), else row-major for the plain kernel."""
@@ -724,11 +748,12 @@ def decode_splits(n_items: int, n_kv_heads: int, group: int, max_ctx: int) -> in
 
 
 def attn_decode(q, out, cache, rows, table, n_heads, scale, window, n_split, part_o=None, part_ml=None, firsts=None,
-                softcap: float = 0.0):
+                softcap: float = 0.0, sink=None):
     """Attention of single query rows; ``rows[i] = (row of q and out, position, index of the request's
     row in ``table``, 0)``, every row's keys in ``n_split`` parts; or, with ``n_split`` = 0, rows with
     splits of their own as ``balanced_items`` lists them, with its list ``firsts`` of where each row's
-    items begin (``None``: no row has more than one split, nothing is merged)."""
+    items begin (``None``: no row has more than one split, nothing is merged).  ``sink`` (float32 ``[n_heads]``):
+    a score per query head that joins the softmax's denominator once."""
     n = q.shape[0]
     hd = cache.head_dim
     n_items = rows.shape[0]
@@ -743,10 +768,12 @@ def attn_decode(q, out, cache, rows, table, n_heads, scale, window, n_split, par
             _check(cache.pool, "attn.cache", torch.bfloat16), _check(rows, "attn.rows", torch.int32, (n_items, 4)), n_items,
             _check(table, "attn.block_table", torch.int32, (None, None)), table.shape[1], n_heads, cache.n_kv_heads,
             hd, cache.page_size, cache.n_pages, float(scale), int(window))
-    if softcap and n_split != 0:
-        raise KernelError("attn_decode: capped scores come with rows that have splits of their own (n_split = 0)")
-    if n_split == 0 and softcap:
+    extras = bool(softcap) or sink is not None
+    if extras and n_split != 0:
+        raise KernelError("attn_decode: capped scores and sinks come with rows that have splits of their own (n_split = 0)")
+    if n_split == 0 and extras:
         call("fl_attn_decode_items_capped", *head, float(softcap),
+             _check(sink, "attn.sink", torch.float32, (n_heads,)) if sink is not None else None,
              _check(firsts, "attn.firsts", torch.int32, (None, 4)) if firsts is not None else None,
              firsts.shape[0] if firsts is not None else 0, stream_handle())
     elif n_split == 0:
@@ -772,11 +799,12 @@ def attn_prefill_heads(n_tiles: int, n_heads: int, n_kv_heads: int, head_dim: in
 
 
 def attn_prefill(q, out, cache, tiles, positions, table, n_heads, scale, window, heads_per_wave: int = 0,
-                 n_split: int = 1, part_o=None, part_ml=None, softcap: float = 0.0):
+                 n_split: int = 1, part_o=None, part_ml=None, softcap: float = 0.0, sink=None):
     """Attention of the longer portions; ``tiles[i] = (request's row in ``table``, first row, rows,
     index of the first row among all rows of tiles)``.  With ``n_split`` > 1 the keys are split and
     merged; ``part_o`` / ``part_ml``: float32 workspaces of rows x heads x n_split x (head_dim rounded
-    up to 32, and 2) values, rows = all rows of tiles."""
+    up to 32, and 2) values, rows = all rows of tiles.  ``softcap`` and ``sink`` as in ``attn_decode``."""
+    extras = bool(softcap) or sink is not None
     n = q.shape[0]
     hd = cache.head_dim
     n_tiles = tiles.shape[0]
@@ -787,12 +815,13 @@ def attn_prefill(q, out, cache, tiles, positions, table, n_heads, scale, window,
             raise KernelError("attn_prefill: splits need a workspace")
         if n_rows is not None and (part_o.numel() < n_rows * n_heads * n_split * hdp or part_ml.numel() < n_rows * n_heads * n_split * 2):
             raise KernelError("attn_prefill: workspace too small for the splits")
-    call("fl_attn_prefill_capped" if softcap else "fl_attn_prefill", _check(q, "attn.q", torch.bfloat16, (n, n_heads * hd)),
+    call("fl_attn_prefill_capped" if extras else "fl_attn_prefill", _check(q, "attn.q", torch.bfloat16, (n, n_heads * hd)),
          _check(out, "attn.out", torch.bfloat16, (n, n_heads * hd)), _check(cache.pool, "attn.cache", torch.bfloat16),
          _check(tiles, "attn.tiles", torch.int32, (n_tiles, 4)), n_tiles,
          _check(positions, "attn.positions", torch.int32, (n,)),
          _check(table, "attn.block_table", torch.int32, (None, None)), table.shape[1], n_heads, cache.n_kv_heads, hd,
-         cache.page_size, cache.n_pages, float(scale), int(window), *((float(softcap),) if softcap else ()), int(heads_per_wave),
+         cache.page_size, cache.n_pages, float(scale), int(window),
+         *((float(softcap), _check(sink, "attn.sink", torch.float32, (n_heads,)) if sink is not None else None) if extras else ()), int(heads_per_wave),
          _check(part_o, "attn.part_o", torch.float32) if part_o is not None else None,
          _check(part_ml, "attn.part_ml", torch.float32) if part_ml is not None else None, int(n_split), stream_handle())
     return out
@@ -843,7 +872,7 @@ def attention_splits(batch, n_heads: int, n_kv_heads: int, head_dim: int, window
     return p_split, n_split
 
 
-def attention(rt, q, out, cache, step, table, n_heads, scale, window, softcap: float = 0.0):
+def attention(rt, q, out, cache, step, table, n_heads, scale, window, softcap: float = 0.0, sink=None):
     """Attention of one batch with the tuned kernels: rows of short portions through the split-K
     kernel, longer portions through the tiled kernel.  A cache shape one of them does not take
     sends the whole batch to the plain kernel."""
@@ -851,8 +880,8 @@ def attention(rt, q, out, cache, step, table, n_heads, scale, window, softcap: f
     batch = step.host
     items = step.extra.get(f"attn_items/{decode_blocks_per_row(n_heads, cache.n_kv_heads)}/{window or 0}") if rows is not None else None
     if rows is None or tiles is None or not decode_supported(cache) or (tiles.shape[0] and not prefill_supported(cache, table, window)) \
-            or (softcap and items is None):
-        return ops.attn_plain(q, out, cache, step.positions, step.tok_seq, table, n_heads, scale, window, softcap=softcap)
+            or ((softcap or sink is not None) and items is None):
+        return ops.attn_plain(q, out, cache, step.positions, step.tok_seq, table, n_heads, scale, window, softcap=softcap, sink=sink)
     key = ("attention_splits", n_heads, cache.n_kv_heads, cache.head_dim, window)
     splits = step.scratch.get(key)
     if splits is None:
@@ -868,7 +897,7 @@ def attention(rt, q, out, cache, step, table, n_heads, scale, window, softcap: f
             p_o = rt.buffer("attn_tile_part_o", n_rows * n_heads * p_split, hdp, torch.float32, max_rows=1 << 24)
             p_ml = rt.buffer("attn_tile_part_ml", n_rows * n_heads * p_split, 2, torch.float32, max_rows=1 << 24)
         attn_prefill(q, out, cache, tiles, step.positions, table, n_heads, scale, window, heads_per_wave=p_heads,
-                     n_split=p_split, part_o=p_o, part_ml=p_ml, softcap=softcap)
+                     n_split=p_split, part_o=p_o, part_ml=p_ml, softcap=softcap, sink=sink)
     if rows.shape[0] and items is not None:
         # rows with splits of their own; the list's length follows from the number of rows alone
         # (a list with a place per row and no more: no row is ever split, nothing to merge)
@@ -881,7 +910,7 @@ def attention(rt, q, out, cache, step, table, n_heads, scale, window, softcap: f
             slots = items.shape[0] * n_heads
             part_o = rt.buffer("attn_part_o", slots, hdp, torch.float32, max_rows=1 << 24)
             part_ml = rt.buffer("attn_part_ml", slots, 2, torch.float32, max_rows=1 << 24)
-        attn_decode(q, out, cache, items, table, n_heads, scale, window, 0, part_o, part_ml, firsts=firsts, softcap=softcap)
+        attn_decode(q, out, cache, items, table, n_heads, scale, window, 0, part_o, part_ml, firsts=firsts, softcap=softcap, sink=sink)
     elif rows.shape[0]:
         part_o = part_ml = None
         if n_split > 1:

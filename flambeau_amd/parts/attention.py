@@ -118,7 +118,7 @@ class NormedGQAAttention(PagedGQAAttention):
     * ``qk_norm``: ``"projection"``: q (and k) divided by the root mean square over ALL its heads at once,
       times a gain per value, before rotation; ``"head"``: every head of q and k divided by its own root
       mean square after rotation, no gain; ``"head_gain"``: the same with a gain per head dim that all heads of q
-      (of k) share; ``None``;
+      (of k) share; ``"head_gain_first"``: norm and gain ahead of the rotation; ``None``;
     * ``position``: any encoding that offers a table of cosines and sines and a ``layout`` (``half`` or
       ``interleaved``), or ``none``;
     * ``softcap``: score <- softcap * tanh(score / softcap) before the softmax;
@@ -126,23 +126,30 @@ class NormedGQAAttention(PagedGQAAttention):
       ``"blend"``: v <- (1 - lambda) v + lambda v_source with a learned lambda, and the blend is what
       the cache holds.  Both read and write ``StepState.scratch[value_mix_key]``;
     * ``gate``: the heads' outputs times ``sigmoid`` (or ``silu``) of a projection of the mixer's input,
-      value by value, before the output projection.
+      value by value, before the output projection; ``gate_per="head"``: one number per head;
+    * ``sink``: a score per query head whose exponential joins the softmax's denominator once, with no key and no value:
+      ``"learned"`` (a tensor), or a number that all heads share (0: one is added to the denominator).
 
     One joined product gives q, k, v and the gate's logits in 32-bit; norms, rotation and the blend are
     32-bit; this step's keys are stored before attention runs."""
     graph_safe = True
     lazy_input = True        # its input goes to the joined projection only
     replayable = True
+    joinable = True
 
     def __init__(self, hidden_size: int, n_heads: int, n_kv_heads: int, head_dim: int, position: PartSpec,
                  value_dim: int | None = None, window: int = 0, scale: float | None = None, qk_norm: str | None = None,
                  eps: float = 1e-6, softcap: float | None = None, value_mix: str | None = None,
-                 value_mix_key: str = "value_mix", gate: str | None = None):
+                 value_mix_key: str = "value_mix", gate: str | None = None, gate_per: str = "value", sink=None):
         value_dim = head_dim if value_dim is None else value_dim
         self.value_dim = value_dim
         self.stored_dim = -(-max(head_dim, value_dim) // 8) * 8
-        if qk_norm not in (None, "projection", "head", "head_gain"):
-            raise ValueError(f"normed_gqa_attention: qk_norm must be 'projection', 'head', 'head_gain' or None, got {qk_norm!r}")
+        if qk_norm not in (None, "projection", "head", "head_gain", "head_gain_first"):
+            raise ValueError(f"normed_gqa_attention: qk_norm must be 'projection', 'head', 'head_gain', 'head_gain_first' or None, got {qk_norm!r}")
+        if gate_per not in ("value", "head"):
+            raise ValueError(f"normed_gqa_attention: gate_per must be 'value' or 'head', got {gate_per!r}")
+        if isinstance(sink, str) and sink != "learned":
+            raise ValueError(f"normed_gqa_attention: sink must be 'learned', a number or None, got {sink!r}")
         if value_mix not in (None, "source", "blend"):
             raise ValueError(f"normed_gqa_attention: value_mix must be 'source', 'blend' or None, got {value_mix!r}")
         if gate not in ops.HEAD_GATES:
@@ -152,7 +159,8 @@ class NormedGQAAttention(PagedGQAAttention):
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(head_dim)
         self.qk_norm, self.eps = qk_norm, float(eps)
         self.softcap = float(softcap or 0.0)
-        self.value_mix, self.value_mix_key, self.gate = value_mix, value_mix_key, gate
+        self.value_mix, self.value_mix_key, self.gate, self.gate_per = value_mix, value_mix_key, gate, gate_per
+        self.attention_sink = sink if sink is None or isinstance(sink, str) else float(sink)
 
     def cache_spec(self):
         return PagedKVSpec(self.n_kv_heads, self.stored_dim, self.window)
@@ -170,27 +178,36 @@ class NormedGQAAttention(PagedGQAAttention):
         if self.qk_norm == "projection":
             t["q_norm.weight"] = TensorSpec((H * D,), "vector32")
             t["k_norm.weight"] = TensorSpec((G * D,), "vector32")
-        elif self.qk_norm == "head_gain":
+        elif self.qk_norm in ("head_gain", "head_gain_first"):
             t["q_norm.weight"] = TensorSpec((D,), "vector32")
             t["k_norm.weight"] = TensorSpec((D,), "vector32")
         if self.value_mix is not None:
             # (the layer whose values are the source has the scalar too, and does not use it)
             t["value_mix.weight"] = TensorSpec((), "vector32", init=lambda g, shape, device: torch.rand(shape, generator=g, device=device))
         if self.gate is not None:
-            t["g.weight"] = TensorSpec((H * Dv, W))
+            t["g.weight"] = TensorSpec((H if self.gate_per == "head" else H * Dv, W))
+        if self.attention_sink == "learned":
+            t["sink"] = TensorSpec((H,), "vector32", init="normal")
         return t
+
+    def join_weights(self, weights):
+        return [weights["q.weight"], weights["k.weight"], weights["v.weight"]] + ([weights["g.weight"]] if self.gate else []), weights["o.weight"]
 
     def bind(self, weights, rt):
         self.rt = rt
         self.kernels = rt.kernels("paged_attention")
         H, G, D, Dv = self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim
-        joined = [weights["q.weight"], weights["k.weight"], weights["v.weight"]] + ([weights["g.weight"]] if self.gate else [])
-        self.w_in = rt.prepare_weight(torch.cat(joined, dim=0).contiguous())
+        if not self.joined:
+            ins, w_o = self.join_weights(weights)
+            self.w_in = rt.prepare_weight(torch.cat(ins, dim=0).contiguous())
+            self.w_o = rt.prepare_weight(w_o)
         self.cols = (0, H * D, H * D + G * D)
         self.gate_col = H * D + G * D + G * Dv
         self._bind_gains(weights)
         self.mix = weights["value_mix.weight"].reshape(1) if self.value_mix == "blend" else None
-        self.w_o = rt.prepare_weight(weights["o.weight"])
+        self.sink = None
+        if self.attention_sink is not None:
+            self.sink = weights["sink"] if self.attention_sink == "learned" else torch.full((H,), self.attention_sink, dtype=torch.float32, device=rt.device)
         self.position.bind({}, rt)
         self.rotated_dims = int(getattr(self.position, "rotated_dims", 0) or 0)      # (the encoding 'none' has none)
         self.interleaved = getattr(self.position, "layout", "half") == "interleaved"
@@ -199,7 +216,7 @@ class NormedGQAAttention(PagedGQAAttention):
 
     def _bind_gains(self, weights):
         """The gains of the norm over the projection (one per value) or of the heads' own norm (one per head dim)."""
-        per_dim = self.qk_norm == "head_gain"
+        per_dim = self.qk_norm in ("head_gain", "head_gain_first")
         self.q_gain = None if per_dim else weights.get("q_norm.weight")
         self.k_gain = None if per_dim else weights.get("k_norm.weight")
         self.q_head_gain = weights.get("q_norm.weight") if per_dim else None
@@ -207,10 +224,18 @@ class NormedGQAAttention(PagedGQAAttention):
 
     def forward(self, x, step, cache):
         rt, n = self.rt, x.shape[0]
-        H, G, D, Dv, P = self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim, self.stored_dim
-        table = step.block_tables[cache.group]
         proj = rt.buffer("nattn_proj", n, self.w_in.rows, torch.float32)
         rt.gemm(x, self.w_in, proj)
+        return Product(self._attend(proj, 0, step, cache), self.w_o)
+
+    def forward_joined(self, proj, col0, step, cache, out, factor):
+        self._attend(proj, col0, step, cache, out, factor)
+
+    def _attend(self, proj, col0, step, cache, gated=None, factor=1.0):
+        """The heads' outputs from the columns ``col0`` on of the projection; in ``gated`` (times ``factor``) where it is given."""
+        rt, n = self.rt, proj.shape[0]
+        H, G, D, Dv, P = self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim, self.stored_dim
+        table = step.block_tables[cache.group]
         angles = self.position.rotary_table(rt, step) if self.rotated_dims else None
         v_first, mode = None, 0
         if self.value_mix == "source":
@@ -222,18 +247,21 @@ class NormedGQAAttention(PagedGQAAttention):
                 raise RuntimeError("normed_gqa_attention: no layer before this one has left values of this shape to blend with")
             mode = 2
         q = rt.buffer("nattn_q", n, H * P)
-        ops.qkv_prepare(proj, self.cols, step.positions, step.tok_seq, table, q, cache.kv, H, D, Dv, self.rotated_dims,
-                        self.interleaved, angles, self.q_gain, self.k_gain, self.qk_norm in ("head", "head_gain"), self.eps,
+        head_norm = {"head": 1, "head_gain": 1, "head_gain_first": 2}.get(self.qk_norm, 0)
+        ops.qkv_prepare(proj, tuple(col0 + c for c in self.cols), step.positions, step.tok_seq, table, q, cache.kv, H, D, Dv,
+                        self.rotated_dims, self.interleaved, angles, self.q_gain, self.k_gain, head_norm, self.eps,
                         v_first=v_first, value_mix=mode, mix=self.mix, write_cache=cache.writes,
                         row_scales=rt.buffer("nattn_row_scales", n, 2, torch.float32) if self.qk_norm == "projection" else None,
                         q_head_gain=self.q_head_gain, k_head_gain=self.k_head_gain)
         out = rt.buffer("nattn_out", n, H * P)
-        self.kernels.attention(q, out, cache.kv, step, table, H, self.scale, self.window, softcap=self.softcap)
-        if self.gate is not None or P != Dv:
-            gated = rt.buffer("nattn_gated", n, H * Dv)
-            ops.heads_gate(out, P, proj if self.gate is not None else None, self.gate_col, self.gate, gated, H)
+        self.kernels.attention(q, out, cache.kv, step, table, H, self.scale, self.window, softcap=self.softcap, sink=self.sink)
+        if self.gate is not None or P != Dv or gated is not None:
+            if gated is None:
+                gated = rt.buffer("nattn_gated", n, H * Dv)
+            ops.heads_gate(out, P, proj if self.gate is not None else None, col0 + self.gate_col, self.gate, gated, H,
+                           per_head=self.gate_per == "head", scale=factor)
             out = gated
-        return Product(out, self.w_o)
+        return out
 
 
 @MIXERS.register("mixed_heads_attention")
@@ -261,6 +289,7 @@ class MixedHeadsAttention(NormedGQAAttention):
     graph_safe = True
     lazy_input = True
     replayable = True
+    joinable = False
 
     def __init__(self, hidden_size: int, n_heads: int, n_kv_heads: int, head_dim: int, value_dim: int | None = None,
                  window: int = 0, scale: float | None = None, qk_norm: str | None = None, eps: float = 1e-6,

@@ -440,6 +440,21 @@ class Mixer(Part):
         """Mixers with equal groups give equal signatures (one of them is asked per step)."""
         return id(self)
 
+    # ---- joining: mixers that read one input side by side and whose outputs are added (``SideBySide``) may share their
+    # first and their last product.  A joinable mixer has ``joined`` (set before ``bind``: it then makes neither weight
+    # itself) and the three functions below.
+    joinable = False
+    joined = False
+
+    def join_weights(self, weights: dict):
+        """``(matrices that read the mixer's input, in the order of its columns; the output projection [hidden, K])``."""
+        raise NotImplementedError
+
+    def forward_joined(self, proj, col0: int, step, cache, out, factor: float):
+        """``forward`` from the columns ``col0`` on of a joined projection (float32 rows) to what the output projection
+        reads, times ``factor`` (applied in 32-bit), in ``out`` ``[n, K]`` (columns of a wider tensor)."""
+        raise NotImplementedError
+
     def forward(self, x, step: StepState, cache: LayerCache):
         """``x``: normed activations [n, hidden] in the compute dtype.  Returns the
         32-bit delta [n, hidden] that is added to the residual stream, or a ``Product`` that

@@ -9,6 +9,9 @@ Positions, if any, live apart from the latent: W_dkv h has ``rot_dim`` more rows
 heads share and that is not normed; every head of q has as many more values; both are rotated, and their product
 joins the score.  The token's cached row is then (c, rotated part), of which only c is summed.
 
+Options: no gate; a sink, a learned score per head that joins the softmax's denominator once (not scaled, with no key and
+no value).
+
 Only that row is cached (``PagedRowSpec``).  Since k and v are linear in c, the key expansion is applied to
 the query instead (qa = W_uk,a^T q_a, then qa . c_j = q_a . k_j) and the value expansion to the
 weighted sum of the rows (W_uv,a sum_j p_j c_j): no key or value is ever made for a cached token,
@@ -32,9 +35,10 @@ class LatentAttention(Mixer):
     replayable = True
 
     def __init__(self, hidden_size: int, n_heads: int, head_dim: int, value_dim: int, q_rank: int, kv_rank: int,
-                 scale: float, eps: float, window: int = 0, gated: bool = True, rot_dim: int = 0, position: PartSpec | None = None):
-        """``rot_dim`` with ``position`` (an encoding with a table of cosines and sines that pairs split halves): the size of
-        the rotated key part and of every head's rotated query part."""
+                 scale: float, eps: float, window: int = 0, gated: bool = True, rot_dim: int = 0, position: PartSpec | None = None,
+                 sink: bool = False):
+        """``rot_dim`` with ``position`` (an encoding with a table of cosines and sines and a ``layout``, split halves or
+        neighbours): the size of the rotated key part and of every head's rotated query part."""
         if bool(rot_dim) != (position is not None):
             raise ValueError("latent_attention: a rotated part and its position encoding come together")
         if kv_rank > ops.latent_max_width():
@@ -45,8 +49,10 @@ class LatentAttention(Mixer):
         self.rot_dim = int(rot_dim)
         self.position = POSITION_ENCODINGS.create(position) if position is not None else None
         self.rotated_dims = self.position.rotated_dims if self.position is not None else 0
-        if self.rotated_dims > self.rot_dim or (self.position is not None and getattr(self.position, "layout", None) != "half"):
-            raise ConfigError(f"latent_attention: {self.rotated_dims} rotated dims of a part of {self.rot_dim}, or another layout than split halves")
+        layout = getattr(self.position, "layout", None)
+        if self.rotated_dims > self.rot_dim or (self.position is not None and layout not in ("half", "interleaved")):
+            raise ConfigError(f"latent_attention: {self.rotated_dims} rotated dims of a part of {self.rot_dim}, or a layout that pairs neither halves nor neighbours")
+        self.interleaved, self.has_sink = layout == "interleaved", bool(sink)
         # what the cache holds per token: with a rotated part, latent and part in steps of 32 values with zeros between
         self.value_width = -(-kv_rank // 32) * 32 if self.rot_dim else kv_rank
         self.row_width = self.value_width + -(-self.rot_dim // 32) * 32
@@ -80,6 +86,8 @@ class LatentAttention(Mixer):
              "o.weight": TensorSpec((W, H * Dv))}
         if self.gated:
             t["g.weight"] = TensorSpec((H, W))
+        if self.has_sink:
+            t["sink"] = TensorSpec((H,), "vector32", init="normal")
         return t
 
     def bind(self, weights, rt):
@@ -91,6 +99,7 @@ class LatentAttention(Mixer):
         self.kernels = rt.kernels("latent_attention")
         self.expansions = self.kernels.prepare(weights["uk.weight"], weights["uv.weight"], self.n_heads)
         self.w_o = rt.prepare_weight(weights["o.weight"])
+        self.sink = weights.get("sink")
         if self.position is not None:
             self.position.bind({}, rt)
 
@@ -103,11 +112,12 @@ class LatentAttention(Mixer):
         rt.gemm(x, self.w_low, low)
         cq = rt.buffer("la_cq", n, Rq)
         ops.latent_prepare(low, Rq, self.dq_norm, cq, Rq, R, self.dkv_norm, self.eps, cache.kv, step.positions, step.tok_seq, table,
-                           rot_dim=Dr, rotated_dims=self.rotated_dims, angles=angles, write_cache=cache.writes)
+                           rot_dim=Dr, rotated_dims=self.rotated_dims, angles=angles, write_cache=cache.writes,
+                           interleaved=self.interleaved)
         q = rt.buffer("la_q", n, H * (D + Dr), torch.float32)
         rt.gemm(cq, self.w_uq, q)
         out = rt.buffer("la_out", n, H * Dv)
         self.kernels.attend(q, self.expansions, cache.kv, step, table, self.scale, self.window,
                             low if self.gated else None, Rq + R + Dr, out,
-                            rotated=ops.RotatedPart(Dr, self.rotated_dims, angles, self.value_width) if Dr else None)
+                            rotated=ops.RotatedPart(Dr, self.rotated_dims, angles, self.value_width, self.interleaved) if Dr else None, sink=self.sink)
         return Product(out, self.w_o)

@@ -21,6 +21,15 @@ HGRN2: the forget gate is a vector per head (one value per key dim) and also dec
 S <- diag(f) S + (1 - f) v^T, o = S^T q, with f = l + (1 - l) sigmoid(W_f h + b_f) above a learned lower bound
 l, q = silu(W_q h), no key of its own and no other scale.  Every head's o is divided by its root mean square
 and multiplied by a gain shared by the heads.
+
+Gated linear attention: a forget gate per head and key dim beside a key of its own, S <- diag(a) S + k v^T, o = S^T q times
+dim^(-1/2), a = sigmoid(W_2 (W_1 h) + b)^(1 / tau) through a projection of low rank.  Every head's o is divided by its root
+mean square, times a gain shared by the heads, times silu of a projection.
+
+State-space duality (Mamba-2): one joined projection gives a gate z, the channels of x, B and C, and a step dt per head; x, B
+and C pass a short causal convolution with a bias (silu behind it; its last inputs are state too); dt <- softplus(dt + b);
+S <- exp(-exp(A_log) dt) S + dt B x^T, y = S^T C + D x per head, B and C shared by groups of heads.  y is multiplied by
+silu(z) and then divided by its root mean square in equal parts of the row, times a gain.
 """
 from __future__ import annotations
 
@@ -265,3 +274,143 @@ class Hgrn2(Mixer):
         out = rt.buffer("hgrn_out", n, H * Dv)
         ops.headnorm_gate(hidden, self.norm, None, 0, out, H, self.eps)
         return Product(out, self.w_o)
+
+
+@MIXERS.register("gated_linear_attention")
+class GatedLinearAttention(Mixer):
+    graph_safe = False          # a step run twice advances the state twice
+    replayable = True
+    lazy_input = True           # its input goes to the joined projection only
+
+    def __init__(self, hidden_size: int, n_heads: int, head_dim: int, value_dim: int, decay_rank: int, tau: float, eps: float,
+                 query_scale: float | None = None):
+        if head_dim > ops.linear_scan_max_dim():
+            raise ConfigError(f"gated_linear_attention: 'dim' {head_dim} is beyond what the kernel takes ({ops.linear_scan_max_dim()})")
+        if decay_rank < 1 or not tau > 0.0:
+            raise ConfigError(f"gated_linear_attention: a decay of rank {decay_rank} with tau {tau}")
+        self.hidden_size, self.n_heads, self.head_dim, self.value_dim = hidden_size, n_heads, head_dim, value_dim
+        self.decay_rank, self.tau, self.eps = int(decay_rank), float(tau), float(eps)
+        self.query_scale = float(query_scale) if query_scale is not None else head_dim ** -0.5
+
+    def cache_spec(self):
+        return StateSpec((self.n_heads * self.head_dim * self.value_dim,), torch.float32)
+
+    def signature_group(self):
+        return ("gated_linear_attention",)
+
+    def step_signature(self, batch):
+        return ()
+
+    def tensors(self):
+        W, H, D, Dv, R = self.hidden_size, self.n_heads, self.head_dim, self.value_dim, self.decay_rank
+        return {"q.weight": TensorSpec((H * D, W)), "k.weight": TensorSpec((H * D, W)), "v.weight": TensorSpec((H * Dv, W)),
+                "g.weight": TensorSpec((H * Dv, W)), "a1.weight": TensorSpec((R, W)), "a2.weight": TensorSpec((H * D, R)),
+                "a2.bias": TensorSpec((H * D,), "vector32", init="normal"), "norm.weight": TensorSpec((Dv,), "vector32"),
+                "o.weight": TensorSpec((W, H * Dv))}
+
+    def bind(self, weights, rt):
+        self.rt = rt
+        H, D, Dv = self.n_heads, self.head_dim, self.value_dim
+        self.w_in = rt.prepare_weight(torch.cat([weights[k + ".weight"] for k in ("q", "k", "v", "g", "a1")], dim=0).contiguous())
+        self.col_k, self.col_v = H * D, 2 * H * D
+        self.col_g = self.col_v + H * Dv
+        self.col_a = self.col_g + H * Dv
+        self.w_a2 = (weights["a2.weight"].contiguous(), weights["a2.weight"].t().contiguous())
+        self.b_a2 = weights["a2.bias"]
+        self.norm = weights["norm.weight"].repeat(H).contiguous()          # one gain for every head, laid out heads x vdim
+        self.w_o = rt.prepare_weight(weights["o.weight"])
+
+    def forward(self, x, step, cache):
+        rt, n = self.rt, x.shape[0]
+        H, D, Dv = self.n_heads, self.head_dim, self.value_dim
+        proj = rt.buffer("gla_proj", n, self.w_in.rows, torch.float32)
+        rt.gemm(x, self.w_in, proj)
+        decay = ops.lowrank_gate(proj, self.col_a, *self.w_a2, self.b_a2, self.tau, rt.buffer("gla_decay", n, H * D, torch.float32))
+        hidden = rt.buffer("gla_hidden", n, H * Dv, torch.float32)
+        ops.linear_scan_gated(proj[:, :H * D], proj[:, self.col_k:self.col_k + H * D], proj[:, self.col_v:self.col_v + H * Dv], decay,
+                              cache.state, step, hidden, H, H, D, Dv, out_scale=self.query_scale)
+        out = rt.buffer("gla_out", n, H * Dv)
+        ops.headnorm_gate(hidden, self.norm, proj, self.col_g, out, H, self.eps, gate_kind="silu")
+        return Product(out, self.w_o)
+
+
+@MIXERS.register("state_space")
+class StateSpace(Mixer):
+    graph_safe = False
+    replayable = True
+    lazy_input = True
+    joinable = True
+
+    def __init__(self, hidden_size: int, n_heads: int, value_dim: int, state_dim: int, n_groups: int, conv_taps: int, norm_parts: int,
+                 eps: float):
+        if state_dim > ops.linear_scan_max_dim():
+            raise ConfigError(f"state_space: 'state' {state_dim} is beyond what the kernel takes ({ops.linear_scan_max_dim()})")
+        if conv_taps < 1:
+            raise ConfigError(f"state_space: a convolution of {conv_taps} taps")
+        if n_heads % n_groups:
+            raise ConfigError(f"state_space: {n_heads} heads are not a multiple of {n_groups} groups")
+        self.inner = n_heads * value_dim
+        if self.inner % norm_parts:
+            raise ConfigError(f"state_space: {self.inner} values do not divide into {norm_parts} parts")
+        self.hidden_size, self.n_heads, self.value_dim, self.state_dim, self.n_groups = hidden_size, n_heads, value_dim, state_dim, n_groups
+        self.conv_taps, self.norm_parts, self.eps = int(conv_taps), int(norm_parts), float(eps)
+        self.channels = self.inner + 2 * n_groups * state_dim
+        # where the kept inputs start in a slot's record (16-byte aligned, and the record a whole number of 16 bytes)
+        self.conv_at = -(-n_heads * state_dim * value_dim // 4) * 4
+
+    def cache_spec(self):
+        return StateSpec((-(-(self.conv_at + self.conv_taps * self.channels) // 4) * 4,), torch.float32)
+
+    def signature_group(self):
+        return ("state_space",)
+
+    def step_signature(self, batch):
+        return ()
+
+    def tensors(self):
+        W, H, C = self.hidden_size, self.n_heads, self.channels
+        uniform = lambda lo, hi: (lambda g, shape, device: lo + (hi - lo) * torch.rand(shape, generator=g, device=device))
+        return {"in.weight": TensorSpec((self.inner + C + H, W)), "conv.weight": TensorSpec((C, self.conv_taps), "vector32", init=uniform(-0.5, 0.5)),
+                "conv.bias": TensorSpec((C,), "vector32", init="normal"), "dt_bias": TensorSpec((H,), "vector32", init=uniform(-2.0, 1.0)),
+                "A_log": TensorSpec((H,), "vector32", init=uniform(-3.0, 0.5)), "D": TensorSpec((H,), "vector32"),
+                "norm.weight": TensorSpec((self.inner,), "vector32"), "o.weight": TensorSpec((W, self.inner))}
+
+    def join_weights(self, weights):
+        return [weights["in.weight"]], weights["o.weight"]
+
+    def bind(self, weights, rt):
+        self.rt = rt
+        if not self.joined:
+            self.w_in = rt.prepare_weight(weights["in.weight"])
+            self.w_o = rt.prepare_weight(weights["o.weight"])
+        self.conv_w = weights["conv.weight"].t().contiguous()              # [taps, channels]
+        self.conv_b, self.dt_bias, self.a_log, self.skip = (weights[k] for k in ("conv.bias", "dt_bias", "A_log", "D"))
+        self.norm, self._scaled = weights["norm.weight"], {}
+
+    def _gain(self, factor: float):
+        """The norm's gain times a factor on the mixer's output."""
+        if factor == 1.0:
+            return self.norm
+        if factor not in self._scaled:
+            self._scaled[factor] = (self.norm * factor).contiguous()
+        return self._scaled[factor]
+
+    def forward(self, x, step, cache):
+        rt, n = self.rt, x.shape[0]
+        proj = rt.buffer("ssd_proj", n, self.w_in.rows, torch.float32)
+        rt.gemm(x, self.w_in, proj)
+        out = rt.buffer("ssd_out", n, self.inner)
+        self.forward_joined(proj, 0, step, cache, out, 1.0)
+        return Product(out, self.w_o)
+
+    def forward_joined(self, proj, col0, step, cache, out, factor):
+        rt, n = self.rt, proj.shape[0]
+        H, Dv, N, G, inner, C = self.n_heads, self.value_dim, self.state_dim, self.n_groups, self.inner, self.channels
+        prep = rt.buffer("ssd_prep", n, C, torch.float32)
+        gates = rt.buffer("ssd_gates", n, 2 * H, torch.float32)
+        ops.conv_steps(proj, col0 + inner, self.conv_w, self.conv_b, cache.state, self.conv_at, step, prep, col0 + inner + C, H, self.dt_bias,
+                       self.a_log, gates)
+        hidden = rt.buffer("ssd_hidden", n, inner, torch.float32)
+        ops.linear_scan_written(prep[:, inner + G * N:], prep[:, inner:inner + G * N], prep[:, :inner], gates, self.skip, cache.state, step,
+                                hidden, H, G, N, Dv)
+        ops.gated_group_norm(hidden, proj, col0, self._gain(factor), out, self.norm_parts, self.eps)

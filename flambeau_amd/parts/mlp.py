@@ -51,3 +51,22 @@ class GatedMlp(SwiGLU):
         act = rt.buffer("ffn_act", n, I)
         rt.gemm_swiglu(x, self.w_gate_up, act, gate=self.activation)
         return Product(act, self.w_down)
+
+
+@FEED_FORWARDS.register("clamped_mlp")
+class ClampedMlp(SwiGLU):
+    """d = (g sigmoid(alpha g) (u + shift)) Wd^T with g = min(x Wg^T, limit) and u = x Wu^T clamped to +-limit.  Gate and up are
+    one joined product whose kernel clamps and gates (in 32-bit) before it stores."""
+    lazy_input = False
+
+    def __init__(self, hidden_size: int, intermediate_size: int, limit: float, alpha: float = 1.702, shift: float = 1.0):
+        if not limit > 0.0:
+            raise ValueError(f"clamped_mlp: a limit of {limit}")
+        super().__init__(hidden_size, intermediate_size)
+        self.limit, self.alpha, self.shift = float(limit), float(alpha), float(shift)
+
+    def forward(self, x, step):
+        rt, n, I = self.rt, x.shape[0], self.intermediate_size
+        act = rt.buffer("ffn_act", n, I)
+        rt.gemm_clamped(x, self.w_gate_up, act, self.alpha, self.limit, self.shift)
+        return Product(act, self.w_down)

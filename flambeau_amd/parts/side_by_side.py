@@ -2,7 +2,11 @@
 (root mean square, eps inside the root, a plain gain of its own) and the results are added with a factor
 each (a half each: their mean); with ``normed=False`` the outputs are added as they are, each with its factor.
 The members are any registered mixers; one of them may keep pages, the others records per slot, which the
-joined cache lays side by side."""
+joined cache lays side by side.
+
+Members whose outputs are added as they are and that can be joined (``Mixer.joinable``) share two products: one
+projection of the input gives the columns of both, and one product adds both outputs, its input being what the two
+output projections read, side by side, each times its factor."""
 from __future__ import annotations
 
 import torch
@@ -62,8 +66,20 @@ class SideBySide(Mixer):
 
     def bind(self, weights, rt):
         self.rt = rt
+        own = {p: {k[len(p) + 1:]: v for k, v in weights.items() if k.startswith(p + ".")} for p in self._members}
+        self.joined = not self.normed and all(m.joinable for m in self._members.values())
+        if self.joined:
+            ins, outs = zip(*(m.join_weights(own[p]) for p, m in self._members.items()))
+            self.out_widths = [w.shape[1] for w in outs]
+            # (the tuned kernels read rows in pieces of 8 values: members whose widths are out of step go alone)
+            self.joined = not (rt.tuned and any(w % 8 for w in self.out_widths))
+        if self.joined:
+            self.col_right = sum(w.shape[0] for w in ins[0])
+            self.w_in = rt.prepare_weight(torch.cat([w for member in ins for w in member], dim=0).contiguous())
+            self.w_o = rt.prepare_weight(torch.cat(outs, dim=1).contiguous())
         for p, m in self._members.items():
-            m.bind({k[len(p) + 1:]: v for k, v in weights.items() if k.startswith(p + ".")}, rt)
+            m.joined = self.joined
+            m.bind(own[p], rt)
         self.gain_left, self.gain_right = weights.get("left_out.weight"), weights.get("right_out.weight")
 
     def _member_cache(self, cache: LayerCache, index: int):
@@ -82,6 +98,14 @@ class SideBySide(Mixer):
 
     def forward(self, x, step, cache):
         rt, n, W = self.rt, x.shape[0], self.hidden_size
+        if self.joined:
+            proj = rt.buffer("sbs_proj", n, self.w_in.rows, torch.float32)
+            rt.gemm(x, self.w_in, proj)
+            both = rt.buffer("sbs_both", n, sum(self.out_widths))
+            at = self.out_widths[0]
+            self.left.forward_joined(proj, 0, step, self._member_cache(cache, 0), both[:, :at], self.factors[0])
+            self.right.forward_joined(proj, self.col_right, step, self._member_cache(cache, 1), both[:, at:], self.factors[1])
+            return Product(both, self.w_o)
         outs = []
         for index, (name, m) in enumerate(self._members.items()):
             d = m.forward(x, step, self._member_cache(cache, index))
