@@ -454,6 +454,32 @@ def lufivik_config(width, heads, q_rank, kv_rank, experts, top, expert_ff, windo
 LUFIVIK_SIZES = {name: dict(sz, window=1024) for name, sz in KUVIDRA_SIZES.items()}
 
 
+def fipitar_config(width, heads, kv_heads, ff, ret_heads, delta_heads, q_rank, kv_rank, vocab=32768, **_):
+    gla = {"type": "gla", "mixer": dict(heads=delta_heads, dim=128, vdim=128, tau=16.0, decay_rank=64)}
+    latent = {"type": "latent_attention", "mixer": dict(
+        heads=heads, dim=128, rot_dim=64, vdim=128, q_rank=q_rank, kv_rank=kv_rank, scale=192 ** -0.5,
+        rot={"base": 1e6, "dims": 64, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}})}
+    left = dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5, softcap=50.0, rot={"base": 50000.0, "dims": 64})
+    right = dict(heads=2 * ret_heads, vdim=64, state=128, groups=8, conv=4, norm_groups=8)
+    par = {"type": "parallel", "mixer": dict(left=left, right=right, left_scale=0.8, right_scale=1.2)}
+    mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+    return {"architecture": "Fipitar", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+            "layers": [dict(l, mlp=mlp) for l in (gla, par, latent, gla, par, latent)]}
+
+
+FIPITAR_SIZES = {name: dict(sz, q_rank=KUVIDRA_SIZES[name]["q_rank"], kv_rank=KUVIDRA_SIZES[name]["kv_rank"]) for name, sz in BUGIDRA_SIZES.items()}
+
+
+def bench_fipitar(a, dtype_name):
+    """The same for the Fipitar design: six layers (two of each kind: gated linear attention, grouped attention beside a
+    state-space recurrence, latent attention) with clamped dense feed-forwards, beside Bugidra (two delta rules, two pairs of
+    attention and retention, two attention layers, gated dense feed-forwards) at the same widths, head counts and
+    feed-forward sizes, with as much recurrent state per layer."""
+    def bugidra(sz):
+        return "bugidra", bugidra_config(**{k: v for k, v in sz.items() if k not in ("q_rank", "kv_rank")})
+    return bench_design(a, dtype_name, "fipitar", "Fipitar", FIPITAR_SIZES, fipitar_config, "6 layers", beside=bugidra, beside_title="Bugidra")
+
+
 def bench_lufivik(a, dtype_name):
     """The same for the Lufivik design: six runs of a layer of windowed latent attention with a rotated part and routed
     experts, beside Kuvidra (four layer runs of latent attention and two of a recurrence, one dense and five routed
@@ -535,10 +561,10 @@ def main():
     ap.add_argument("--warmup", type=int, default=16)
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--reps", type=int, default=REPS, help="repetitions of the timed steps; the median is reported")
-    ap.add_argument("--config", default="7b", choices=sorted(CONFIGS) + ["kuvidra", "bugidra", "fitevik", "lenedra", "lufivik"])
-    ap.add_argument("--only-size", default=None, choices=sorted(KUVIDRA_SIZES), help="--config kuvidra / bugidra / fitevik / lenedra / lufivik: one size only")
-    ap.add_argument("--only-model", default=None, choices=["kuvidra", "bugidra", "fitevik", "lenedra", "lufivik", "mistral"],
-                    help="--config kuvidra / bugidra / fitevik / lenedra / lufivik: one of the two models only")
+    ap.add_argument("--config", default="7b", choices=sorted(CONFIGS) + ["kuvidra", "bugidra", "fitevik", "lenedra", "lufivik", "fipitar"])
+    ap.add_argument("--only-size", default=None, choices=sorted(KUVIDRA_SIZES), help="--config kuvidra / bugidra / fitevik / lenedra / lufivik / fipitar: one size only")
+    ap.add_argument("--only-model", default=None, choices=["kuvidra", "bugidra", "fitevik", "lenedra", "lufivik", "fipitar", "mistral"],
+                    help="--config kuvidra / bugidra / fitevik / lenedra / lufivik / fipitar: one of the two models only")
     ap.add_argument("--layers", type=int, default=None, help="run only the first layers (named in config)")
     ap.add_argument("--dtype", default="bf16", choices=["bf16", "fp32"])
     ap.add_argument("--no-points", action="store_true", help="skip batch 1 and 64 and the prefill")
@@ -563,6 +589,8 @@ def main():
         return bench_lenedra(a, dtype_name)
     if a.config == "lufivik":
         return bench_lufivik(a, dtype_name)
+    if a.config == "fipitar":
+        return bench_fipitar(a, dtype_name)
     label, cfg = CONFIGS[a.config]
     if a.config != "7b":
         return bench_serving(a, a.config, label, cfg, dtype_name, el)

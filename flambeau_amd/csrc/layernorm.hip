@@ -11,7 +11,8 @@
 // adding its values in rising order and the block's partial sums in a fixed tree: a row's result does not
 // depend on what else the step holds.  In a step of few rows (where a pass over a row is a wait for memory and
 // little else), rows of up to 8,192 values whose length is a multiple of four are read once, 16 bytes at a time, and
-// stay in registers through both passes and the output; otherwise a row is read thrice.
+// stay in registers through both passes and the output; otherwise a row is read thrice.  fl_layernorm_add holds rows of up
+// to 16,384 values in every step, spread over as many threads as the row has groups of four.
 #include "common.h"
 #include "api.h"
 #include "recordable.h"
@@ -150,33 +151,59 @@ extern "C" int fl_layernorm(const float* x, const float* delta, float* resid_out
 }
 FL_RECORDABLE(fl_layernorm)
 
+// A row's VPT groups of four values per thread stay in registers; the number of threads follows from the row's length
+// alone, so a row's bits do not depend on what else the step holds.
+template <int NT, int VPT, typename TC>
+__global__ __launch_bounds__(NT) void layernorm_add_kernel(const float* __restrict__ delta, const float* __restrict__ w,
+                                                           const float* __restrict__ b, float* __restrict__ resid,
+                                                           TC* __restrict__ cast, int H, float eps) {
+    __shared__ float red[2 * (NT / 64)];
+    const size_t at = (size_t)blockIdx.x * H;
+    f32x4 v[VPT], r[VPT];
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int i = 4 * (threadIdx.x + NT * k);
+        v[k] = r[k] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        if (i >= H) continue;
+        v[k] = *(const f32x4*)(delta + at + i);
+        r[k] = *(const f32x4*)(resid + at + i);
+        s += (v[k][0] + v[k][1]) + (v[k][2] + v[k][3]);
+    }
+    const float mean = block_sum<NT / 64>(s, red) / (float)H;
+    float q = 0.f;
+#pragma unroll
+    for (int k = 0; k < VPT; ++k)
+        if (4 * (threadIdx.x + NT * k) < H) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float d = v[k][e] - mean;
+                q = fmaf(d, d, q);
+            }
+        }
+    const float inv = 1.0f / sqrtf(block_sum<NT / 64>(q, red + NT / 64) / (float)H + eps);
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int i = 4 * (threadIdx.x + NT * k);
+        if (i >= H) continue;
+        const f32x4 w4 = *(const f32x4*)(w + i), b4 = b ? *(const f32x4*)(b + i) : (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) r[k][e] += layernorm_value(v[k][e], mean, inv, w4[e], b4[e]);
+        *(f32x4*)(resid + at + i) = r[k];
+        if (cast) store4<TC>(cast + at + i, r[k]);
+    }
+}
+
+// rows whose length is no multiple of four, or that are too long to be held
 template <typename TC>
-__global__ __launch_bounds__(256) void layernorm_add_kernel(const float* __restrict__ delta, const float* __restrict__ w,
-                                                            const float* __restrict__ b, float* __restrict__ resid,
-                                                            TC* __restrict__ cast, int H, float eps, bool held) {
+__global__ __launch_bounds__(256) void layernorm_add_any_kernel(const float* __restrict__ delta, const float* __restrict__ w,
+                                                                const float* __restrict__ b, float* __restrict__ resid,
+                                                                TC* __restrict__ cast, int H, float eps) {
     __shared__ float lds[8];
     const float* dr = delta + (size_t)blockIdx.x * H;
     float* r = resid + (size_t)blockIdx.x * H;
     float mean, inv;
-    if (held) {
-        f32x4 v[LN_HELD];
-        layernorm_row_held(dr, nullptr, H, eps, lds, v, mean, inv);
-#pragma unroll
-        for (int k = 0; k < LN_HELD; ++k) {
-            const int i = 4 * (threadIdx.x + 256 * k);
-            if (i >= H) continue;
-            const f32x4 w4 = *(const f32x4*)(w + i), b4 = b ? *(const f32x4*)(b + i) : (f32x4){0.f, 0.f, 0.f, 0.f};
-            f32x4 y = *(const f32x4*)(r + i);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) y[e] += layernorm_value(v[k][e], mean, inv, w4[e], b4[e]);
-            *(f32x4*)(r + i) = y;
-            if (cast) store4<TC>(cast + (size_t)blockIdx.x * H + i, y);
-        }
-        return;
-    }
-    auto value = [&](int i) { return dr[i]; };
-    if ((H & 3) == 0) layernorm_row4(dr, nullptr, H, eps, lds, mean, inv);
-    else layernorm_row(value, H, eps, lds, mean, inv);
+    layernorm_row([&](int i) { return dr[i]; }, H, eps, lds, mean, inv);
     for (int i = threadIdx.x; i < H; i += 256) {
         const float v = r[i] + layernorm_value(dr[i], mean, inv, w[i], b ? b[i] : 0.f);
         r[i] = v;
@@ -188,8 +215,20 @@ extern "C" int fl_layernorm_add(const float* delta, const float* w, const float*
                                 int n, int H, float eps, hipStream_t stream) {
     FL_CHECK(n >= 0 && H > 0 && delta && w && resid, "layernorm_add: bad sizes or a missing tensor");
     if (n == 0) return 0;
-    if (!cast || cast_dtype == FL_F32) layernorm_add_kernel<float><<<n, 256, 0, stream>>>(delta, w, b, resid, (float*)cast, H, eps, layernorm_holds(n, H));
-    else if (cast_dtype == FL_BF16) layernorm_add_kernel<bf16_t><<<n, 256, 0, stream>>>(delta, w, b, resid, (bf16_t*)cast, H, eps, layernorm_holds(n, H));
+    auto aligned = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+    const bool whole = (H & 3) == 0 && H <= 4 * 1024 * 4 && aligned(delta) && aligned(w) && aligned(b) && aligned(resid) && aligned(cast);
+    auto run = [&](auto* c) {
+        typedef typename std::remove_pointer<decltype(c)>::type T;
+        if (!whole) layernorm_add_any_kernel<T><<<n, 256, 0, stream>>>(delta, w, b, resid, c, H, eps);
+        else if (H <= 4 * 64) layernorm_add_kernel<64, 1, T><<<n, 64, 0, stream>>>(delta, w, b, resid, c, H, eps);
+        else if (H <= 4 * 256) layernorm_add_kernel<256, 1, T><<<n, 256, 0, stream>>>(delta, w, b, resid, c, H, eps);
+        else if (H <= 4 * 512) layernorm_add_kernel<512, 1, T><<<n, 512, 0, stream>>>(delta, w, b, resid, c, H, eps);
+        else if (H <= 4 * 1024) layernorm_add_kernel<1024, 1, T><<<n, 1024, 0, stream>>>(delta, w, b, resid, c, H, eps);
+        else if (H <= 8 * 1024) layernorm_add_kernel<1024, 2, T><<<n, 1024, 0, stream>>>(delta, w, b, resid, c, H, eps);
+        else layernorm_add_kernel<1024, 4, T><<<n, 1024, 0, stream>>>(delta, w, b, resid, c, H, eps);
+    };
+    if (!cast || cast_dtype == FL_F32) run((float*)cast);
+    else if (cast_dtype == FL_BF16) run((bf16_t*)cast);
     else FL_CHECK(false, "layernorm_add: unknown dtype %d", cast_dtype);
     FL_LAUNCH_CHECK();
     return 0;

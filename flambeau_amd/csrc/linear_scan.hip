@@ -322,11 +322,11 @@ __global__ __launch_bounds__(256) void lowrank_expand_rows_kernel(const float* _
 template <typename T>
 __global__ __launch_bounds__(256) void lowrank_expand_kernel(const float* __restrict__ x, int ld, int col, const T* __restrict__ w,
                                                              float* __restrict__ out, int n, int N, int R, LowRankTail tail) {
-    extern __shared__ float xr[];                         // [LR_TOKENS][R]
+    extern __shared__ __attribute__((aligned(16))) float xr[];         // [R][LR_TOKENS]
     const int t0 = blockIdx.y * LR_TOKENS, cnt = min(LR_TOKENS, n - t0);
     for (int e = threadIdx.x; e < LR_TOKENS * R; e += 256) {
         const int tt = e / R, r = e - tt * R;
-        xr[e] = tt < cnt ? x[(size_t)(t0 + tt) * ld + col + r] : 0.f;
+        xr[r * LR_TOKENS + tt] = tt < cnt ? x[(size_t)(t0 + tt) * ld + col + r] : 0.f;
     }
     __syncthreads();
     const int f = blockIdx.x * 256 + threadIdx.x;
@@ -338,7 +338,7 @@ __global__ __launch_bounds__(256) void lowrank_expand_kernel(const float* __rest
     for (int r = 0; r < R; ++r) {
         const float wv = to_f32(w[(size_t)r * N + f]);
 #pragma unroll
-        for (int tt = 0; tt < LR_TOKENS; ++tt) s[tt] = fmaf(xr[tt * R + r], wv, s[tt]);
+        for (int tt = 0; tt < LR_TOKENS; ++tt) s[tt] = fmaf(xr[r * LR_TOKENS + tt], wv, s[tt]);
     }
 #pragma unroll
     for (int tt = 0; tt < LR_TOKENS; ++tt)

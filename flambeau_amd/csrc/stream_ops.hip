@@ -200,7 +200,8 @@ __global__ __launch_bounds__(256) void heads_gate_kernel(const T* __restrict__ x
                                                          int gate_col0, int kind, int per_head, float scale, T* __restrict__ out,
                                                          int ldo, int H, int Dv) {
     const size_t t = blockIdx.x;
-    for (int e = threadIdx.x; e < H * Dv; e += 256) {
+    // (a token's values are spread over blocks, so that a step of few tokens still fills units)
+    for (int e = blockIdx.y * 256 + threadIdx.x; e < H * Dv; e += 256 * gridDim.y) {
         const int h = e / Dv, j = e - h * Dv;
         float v = to_f32(x[(t * H + h) * ldh + j]) * scale;
         if (kind) {
@@ -217,10 +218,11 @@ extern "C" int fl_heads_gate(const void* x, int dtype, int ldh, const float* gat
     FL_CHECK(kind >= 0 && kind <= 2 && (kind == 0 || (gate && ldg >= gate_col0 + (per_head ? H : H * Dv))), "heads_gate: gate %d over rows %d wide", kind, ldg);
     FL_CHECK(ldo >= H * Dv, "heads_gate: output rows of %d values for %d heads of %d", ldo, H, Dv);
     if (n == 0) return 0;
+    const dim3 grid(n, min(ceil_div(H * Dv, 512), 64));
     if (dtype == FL_F32)
-        heads_gate_kernel<float><<<n, 256, 0, stream>>>((const float*)x, ldh, gate, ldg, gate_col0, kind, per_head, scale, (float*)out, ldo, H, Dv);
+        heads_gate_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, ldh, gate, ldg, gate_col0, kind, per_head, scale, (float*)out, ldo, H, Dv);
     else if (dtype == FL_BF16)
-        heads_gate_kernel<bf16_t><<<n, 256, 0, stream>>>((const bf16_t*)x, ldh, gate, ldg, gate_col0, kind, per_head, scale, (bf16_t*)out, ldo, H, Dv);
+        heads_gate_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, ldh, gate, ldg, gate_col0, kind, per_head, scale, (bf16_t*)out, ldo, H, Dv);
     else
         FL_CHECK(false, "heads_gate: unknown dtype %d", dtype);
     FL_LAUNCH_CHECK();

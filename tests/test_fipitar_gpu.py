@@ -117,6 +117,28 @@ def test_a_gate_and_a_norm_in_parts_alone(dtype, W, parts):
     assert (got[:, :8] == -7).all() and (got[:, 8 + W:] == -7).all()
 
 
+@pytest.mark.parametrize("W", [37, 40, 256, 516, 1000, 2048, 4096, 5000, 6002, 16384, 20000])
+def test_a_norm_on_its_way_into_the_stream_alone(W):
+    """Rows that are held in registers by blocks of every size and rows that are not: the same bits in a step of few rows and
+    of many, the stream in 32-bit and in the compute dtype beside it."""
+    from flambeau_amd.kernels import ops
+    g = torch.Generator().manual_seed(W)
+    n, eps = 300, 3e-4
+    y, x = torch.randn(n, W, generator=g) * 3 + 0.5, torch.randn(n, W, generator=g)
+    w, b = 1 + 0.3 * torch.randn(W, generator=g), torch.randn(W, generator=g)
+    want = x.double().numpy() + pf.layer_norm(y.double().numpy(), w.double().numpy(), b.double().numpy(), eps)
+    for bias in (b, None):
+        outs = []
+        for rows in (n, 3):
+            r, cast = dev(x[:rows]), torch.empty(rows, W, dtype=torch.bfloat16, device=DEV)
+            ops.layernorm_add(dev(y[:rows]), dev(w), dev(bias), r, eps, cast=cast)
+            assert torch.equal(cast, r.to(torch.bfloat16))
+            ref = want[:rows] - (0 if bias is not None else b.double().numpy())
+            assert np.abs(r.double().cpu().numpy() - ref).max() < 3e-6 * np.abs(want).max()
+            outs.append(r)
+        assert torch.equal(outs[0][:3], outs[1])
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("n,N,R,tau", [(1, 30, 5, 4.0), (16, 700, 1, 1.0), (17, 513, 64, 16.0), (50, 33, 200, 0.5)])
 def test_a_forget_gate_of_low_rank_alone(dtype, n, N, R, tau):
